@@ -20,8 +20,9 @@ _vp, _i64, _i32, _u32, _f32 = C.c_void_p, C.c_int64, C.c_int, C.c_uint32, C.c_fl
 def build(ref: bool = True) -> None:
     """Compile the C restatement, and the reference build when its checkout is present."""
     subprocess.check_call(["make", "-s", "-C", _HERE, "oracle"])
-    if ref and os.path.isdir(os.environ.get("PTM_REF", "/root/reference")):
-        subprocess.check_call(["make", "-s", "-C", _HERE, "ref", "REF=" + os.environ.get("PTM_REF", "/root/reference")])
+    ref_dir = os.environ.get("PTM_REF", "/root/reference")
+    if ref and os.path.exists(os.path.join(ref_dir, "c10", "core", "TensorImpl.cpp")):  # a checkout, not just a folder of that name
+        subprocess.check_call(["make", "-s", "-C", _HERE, "ref", "REF=" + ref_dir])
 
 
 def _p(a: np.ndarray):
