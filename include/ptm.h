@@ -494,6 +494,112 @@ const float* ptm_decode_logits(ptm_decoder* d);
 const float* ptm_decode_hidden(ptm_decoder* d);
 void* ptm_decode_stream(ptm_decoder* d);
 
+/* ---- decoders over bfloat16 weights, described layer by layer -----------------------------------
+ * A second way to make a ptm_decoder: instead of the one layer shape of ptm_decode_config, a list of blocks each of which
+ * names its token mixer and that mixer's sizes.  Everything else of the decode runtime (steps and their hipGraph, prompts in
+ * row batches, greedy and sampled generation, logits) is the same object with the same calls.
+ *
+ * One block, on the residual x (fp32):
+ *   x += RMSNorm(mixer(RMSNorm(x, norm1)), norm1b);   x += RMSNorm(W_down relu(W_up RMSNorm(x, norm2))^2, norm2b)
+ *   and with a per-layer token input: g = gelu_tanh(W_gate x) * e, e = the block's part of the token's row of a second
+ *   embedding table; x += RMSNorm(W_proj g, side_norm)
+ * Mixers:
+ *   PTM_MIX_ATTENTION  GQA; q and k RMS-normed over the whole projection, rotated, scores scale * q.k, optionally
+ *                      softcap * tanh(score / softcap), sliding window with kept first positions
+ *   PTM_MIX_LATENT     q per head [dim | rot_dim]; one latent c (RMS-normed) and one rotated key part per position are
+ *                      cached; per head k = [W_uk c | rotated part], v = W_uv c.  A decode step never expands the cache:
+ *                      W_uk moves onto the query and W_uv onto the attended latent.
+ * Weights are bfloat16 matrices (ggml_type PTM_TYPE_BF16), rows zero-padded to multiples of 64 values
+ * (ptm_dense_cols); vectors are fp32, zero-padded alike; `vec64` below marks such a vector. */
+#define PTM_TYPE_BF16 30u
+enum { PTM_MIX_ATTENTION = 0, PTM_MIX_LATENT = 1 };
+enum { PTM_PRECISION_16 = 0, /* bfloat16 caches and prompt GEMM operands, fp32 accumulation and fp32 decode activations */
+       PTM_PRECISION_32 = 1  /* fp32 caches and activations throughout (weights stay bfloat16: exact in fp32) */ };
+
+/* Rotation of the pairs (2i, 2i + 1), i < dims / 2, by position * f_i, f_i = base^(-2i / dims); factor > 0: YaRN blend of f_i
+ * and f_i / factor between the dimensions that turn `fast` and `slow` times over `original` positions, cos and sin times
+ * 0.1 ln(factor) + 1. */
+typedef struct {
+    double base, factor, original, fast, slow;
+    int32_t dims;
+} ptm_rotation;
+/* table[max_seq][dims / 2][2] = (cos, sin); angles in double, host memory. */
+int ptm_rope_pairs_host(float* table, int max_seq, const ptm_rotation* rot);
+
+typedef struct {
+    int32_t mixer;                       /* PTM_MIX_* */
+    int32_t heads, kv_heads, dim, vdim;  /* latent: kv_heads is ignored */
+    int32_t rot_dim, kv_rank;            /* latent only */
+    int32_t window, keep_first;          /* 0 / 0: every earlier position */
+    float scale, softcap;                /* softcap 0: none */
+    ptm_rotation rot;
+    ptm_qweight in;      /* attention: rows [q | k | v]; latent: rows [q | c and rotated key part] */
+    ptm_qweight expand;  /* latent: per head dim rows of W_uk, padded to a multiple of 8 rows, then W_uv alike */
+    ptm_qweight out;     /* columns per head vdim, padded to a multiple of 8 */
+    const float *q_norm, *k_norm;        /* attention: whole projections; latent: k_norm is the latent's, q_norm unused */
+    const float *norm1, *norm1b;         /* vec64 [hidden] */
+    int32_t ff;                          /* 0: no feed-forward */
+    ptm_qweight up, down;
+    const float *norm2, *norm2b;         /* vec64 [hidden] */
+    ptm_qweight side_gate, side_proj;    /* data NULL: no per-layer token input */
+    const float* side_norm;              /* vec64 [hidden] */
+    int32_t side_offset;                 /* first column of the block's part of the side table */
+} ptm_block;
+
+typedef struct {
+    int32_t vocab, hidden, n_blocks, max_seq;
+    float eps;
+    int32_t precision;                   /* PTM_PRECISION_* */
+    int32_t use_graph;
+    const ptm_block* blocks;             /* HOST array (copied) */
+    /* blocks loop_start .. loop_stop - 1 run loop_times times; each pass has its own caches; before each pass but the first
+     * the embedding output is added to x, before every pass row t of loop_step */
+    int32_t loop_start, loop_stop, loop_times;  /* loop_times 0: no loop */
+    const float* loop_step;              /* device [loop_times][ptm_dense_cols(hidden)] */
+    ptm_qweight embedding;               /* BF16 [vocab][hidden] */
+    ptm_qweight side_table;              /* BF16 [vocab][n_blocks * side_dim]; data NULL: none */
+    int32_t side_dim;
+    const float* out_norm;               /* vec64 */
+    ptm_qweight lm_head;                 /* BF16 [vocab][hidden] */
+} ptm_block_config;
+
+int ptm_dense_cols(int cols);            /* cols rounded up to a multiple of 64 */
+/* Allocates the caches ([layer runs], zeroed) and all decode scratch; weights stay the caller's.  Prompt scratch as in
+ * ptm_decode_reserve_prefill. */
+int ptm_decode_create_blocks(const ptm_block_config* cfg, ptm_decoder** out);
+/* Layer runs of a decoder: blocks, with those of a loop counted once per pass (n_layers for the others). */
+int ptm_decode_layer_runs(const ptm_decoder* d);
+/* ptm_decode_prefill that also returns logits: want[n_want] are ascending places among the n tokens, logits_host
+ * [n_want][vocab] (host) receives theirs.  *next_token as ptm_decode_prefill.  Any decoder. */
+int ptm_decode_prefill_logits(ptm_decoder* d, const int32_t* tokens, int n, int chunk_rows, const int32_t* want, int n_want,
+                              float* logits_host, int64_t* next_token);
+/* Logits of the last step, copied to host memory [vocab]. */
+int ptm_decode_read_logits(ptm_decoder* d, float* logits_host);
+/* ptm_decode_prefill in one chunk that also copies out the residual rows after every layer run:
+ * trace_host[layer runs][n][hidden] fp32 (host).  Decoders made by ptm_decode_create_blocks only. */
+int ptm_decode_prefill_trace(ptm_decoder* d, const int32_t* tokens, int n, int64_t* next_token, float* trace_host);
+
+/* The pieces by themselves.  y[N] = W . x: W bfloat16 [N][ld], ld >= ptm_dense_cols(K), columns past K zero; x fp32 vec64. */
+int ptm_dense_gemv(const void* W_bf16, const float* x, float* y, int K, int N, int64_t ld, ptm_stream_t stream);
+/* C[M][N] fp32 = A[M][lda] . W[N][ldw]^T; A bfloat16 (a_fp32 = 0, matrix cores in bfloat16) or fp32 (matrix cores in fp32);
+ * lda and ldw >= ptm_dense_cols(K), W's columns past K zero, A's finite. */
+int ptm_dense_gemm(const void* A, int a_fp32, int64_t lda, const void* W_bf16, int64_t ldw, float* C, int64_t ldc, int M, int N,
+                   int K, ptm_stream_t stream);
+/* Softmax attention of query rows r (position pos0 + r) over keys j <= pos0 + r with pos0 + r - j < window or
+ * j < keep_first (window 0: no limit).  The key of (j, kv head g) is K1[j][g][dim1] followed by K2[j][dim2] shared by all
+ * heads (dim2 may be 0).  Strides in elements, dims multiples of 8; element type bfloat16 (fp32 = 0) or fp32, of Q
+ * [row][head][dim1 + dim2], K1, K2, V and O [row][head][vdim].  Row 0 of K1 / K2 / V is position kv_pos0. */
+typedef struct {
+    const void *Q, *K1, *K2, *V;
+    void* O;
+    int64_t q_row, k1_row, k1_head, k2_row, v_row, v_head, o_row;
+    int32_t rows, heads, kv_heads, dim1, dim2, vdim, window, keep_first;
+    int64_t pos0, kv_pos0;
+    float scale, softcap;
+    int32_t fp32;
+} ptm_attention_args;
+int ptm_attention_rows(const ptm_attention_args* a, ptm_stream_t stream);
+
 /* ---- GGUF files: container reader and model loader --------------------------------------- */
 /* Reader for GGUF v2/v3 (the reference's GGUFReader, torch/io/gguf_loader.h:386-630): the file is
  * memory-mapped; tensor data pointers are HOST pointers into the mapping, valid until close.
@@ -544,6 +650,29 @@ ptm_decoder* ptm_model_decoder(ptm_model* m); /* owned by the model */
 int ptm_model_config(const ptm_model* m, ptm_decode_config* out);
 int ptm_model_layer(const ptm_model* m, int i, ptm_layer* out);
 void ptm_model_free(ptm_model* m);
+
+/* ---- model folders: config.json + model.safetensors -------------------------------------------------
+ * Reader of a safetensors file (u64 header length, JSON header, data): memory-mapped, tensor data are HOST pointers into
+ * the mapping, valid until close. */
+typedef struct ptm_safetensors ptm_safetensors;
+typedef struct {
+    const char* name;
+    const char* dtype; /* as in the file: "BF16", "F32", "I32", ... */
+    int32_t n_dims;
+    int64_t dims[8];
+    int64_t nbytes;
+    const void* data;
+} ptm_st_tensor;
+int ptm_safetensors_open(const char* path, ptm_safetensors** out);
+void ptm_safetensors_close(ptm_safetensors* f);
+int64_t ptm_safetensors_n_tensors(const ptm_safetensors* f);
+int ptm_safetensors_tensor_at(const ptm_safetensors* f, int64_t i, ptm_st_tensor* out);
+int ptm_safetensors_find(const ptm_safetensors* f, const char* name, ptm_st_tensor* out);
+
+/* Any model: a .gguf file (ptm_model_load_gguf; precision chooses the fp16 or fp32 cache) or a folder, whose config.json
+ * names the architecture: "Tovasun" (a list of attention / latent_attention layers, optionally with a loop and a per-layer
+ * token input). */
+int ptm_model_load(const char* path, int max_seq, int precision, int use_graph, ptm_model** out);
 
 /* ---- tokenizer and chat template (host only) ----------------------------------------------------
  * GGUFTokenizer (torch/io/tokenizer.h:24-643): byte-level BPE ("gpt2": Qwen, Llama-3) or word-marker BPE /

@@ -57,6 +57,36 @@ class GgufTensor(C.Structure):
                 ("data", vp)]
 
 
+class Rotation(C.Structure):
+    _fields_ = [(n, C.c_double) for n in ("base", "factor", "original", "fast", "slow")] + [("dims", C.c_int32)]
+
+
+class Block(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "rot_dim", "kv_rank", "window", "keep_first")] + \
+               [("scale", f32), ("softcap", f32), ("rot", Rotation), ("in_", QWeight), ("expand", QWeight), ("out", QWeight)] + \
+               [(n, vp) for n in ("q_norm", "k_norm", "norm1", "norm1b")] + \
+               [("ff", C.c_int32), ("up", QWeight), ("down", QWeight), ("norm2", vp), ("norm2b", vp), ("side_gate", QWeight),
+                ("side_proj", QWeight), ("side_norm", vp), ("side_offset", C.c_int32)]
+
+
+class BlockConfig(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("vocab", "hidden", "n_blocks", "max_seq")] + \
+               [("eps", f32), ("precision", C.c_int32), ("use_graph", C.c_int32), ("blocks", C.POINTER(Block)),
+                ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("loop_step", vp),
+                ("embedding", QWeight), ("side_table", QWeight), ("side_dim", C.c_int32), ("out_norm", vp), ("lm_head", QWeight)]
+
+
+class AttentionArgs(C.Structure):
+    _fields_ = [(n, vp) for n in ("Q", "K1", "K2", "V", "O")] + \
+               [(n, i64) for n in ("q_row", "k1_row", "k1_head", "k2_row", "v_row", "v_head", "o_row")] + \
+               [(n, C.c_int32) for n in ("rows", "heads", "kv_heads", "dim1", "dim2", "vdim", "window", "keep_first")] + \
+               [("pos0", i64), ("kv_pos0", i64), ("scale", f32), ("softcap", f32), ("fp32", C.c_int32)]
+
+
+class StTensor(C.Structure):
+    _fields_ = [("name", C.c_char_p), ("dtype", C.c_char_p), ("n_dims", C.c_int32), ("dims", i64 * 8), ("nbytes", i64), ("data", vp)]
+
+
 # name -> (restype, argtypes); every function declared in include/ptm.h
 SIGNATURES = {
     "ptm_strerror": (C.c_char_p, [i32]),
@@ -177,6 +207,22 @@ SIGNATURES = {
     "ptm_tokenizer_token": (i32, [vp, C.c_int32, C.c_char_p, i64, C.POINTER(i64)]),
     "ptm_chat_template": (i32, [C.c_char_p, C.c_char_p, C.c_char_p, i32, C.c_char_p, C.c_char_p, i64, C.POINTER(i64)]),
     "ptm_model_load_gguf": (i32, [C.c_char_p, i32, i32, i32, C.POINTER(vp)]),
+    "ptm_rope_pairs_host": (i32, [vp, i32, C.POINTER(Rotation)]),
+    "ptm_dense_cols": (i32, [i32]),
+    "ptm_decode_create_blocks": (i32, [C.POINTER(BlockConfig), C.POINTER(vp)]),
+    "ptm_decode_layer_runs": (i32, [vp]),
+    "ptm_decode_prefill_logits": (i32, [vp, C.POINTER(C.c_int32), i32, i32, C.POINTER(C.c_int32), i32, vp, C.POINTER(i64)]),
+    "ptm_decode_read_logits": (i32, [vp, vp]),
+    "ptm_decode_prefill_trace": (i32, [vp, C.POINTER(C.c_int32), i32, C.POINTER(i64), vp]),
+    "ptm_dense_gemv": (i32, [vp, vp, vp, i32, i32, i64, vp]),
+    "ptm_dense_gemm": (i32, [vp, i32, i64, vp, i64, vp, i64, i32, i32, i32, vp]),
+    "ptm_attention_rows": (i32, [C.POINTER(AttentionArgs), vp]),
+    "ptm_safetensors_open": (i32, [C.c_char_p, C.POINTER(vp)]),
+    "ptm_safetensors_close": (None, [vp]),
+    "ptm_safetensors_n_tensors": (i64, [vp]),
+    "ptm_safetensors_tensor_at": (i32, [vp, i64, C.POINTER(StTensor)]),
+    "ptm_safetensors_find": (i32, [vp, C.c_char_p, C.POINTER(StTensor)]),
+    "ptm_model_load": (i32, [C.c_char_p, i32, i32, i32, C.POINTER(vp)]),
     "ptm_model_decoder": (vp, [vp]),
     "ptm_model_config": (i32, [vp, C.POINTER(DecodeConfig)]),
     "ptm_model_layer": (i32, [vp, i32, C.POINTER(Layer)]),

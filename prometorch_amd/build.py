@@ -8,7 +8,7 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libptm_hip.so")
-SOURCES = ["glue.hip", "q4k_gemv.hip", "q6k_gemv.hip", "flash_decode.hip", "mixed_gemv.hip", "qgemm.hip", "decode.hip", "dispatch.hip", "other_gemv.hip", "gguf.hip", "prefill.hip", "sampler.hip", "tokenizer.hip", "plain_ops.hip"]
+SOURCES = ["glue.hip", "q4k_gemv.hip", "q6k_gemv.hip", "flash_decode.hip", "mixed_gemv.hip", "qgemm.hip", "decode.hip", "dispatch.hip", "other_gemv.hip", "gguf.hip", "prefill.hip", "sampler.hip", "tokenizer.hip", "plain_ops.hip", "dense_gemv.hip", "dense_gemm.hip", "mixer_attention.hip", "blocks.hip", "model_folder.hip"]
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off",
@@ -35,10 +35,23 @@ def build(verbose: bool = True, jobs: int = 8) -> str:
         if len(procs) >= jobs:
             _drain(procs)
     _drain(procs)
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB]
+    tmp = LIB + ".tmp"
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", tmp]
     if verbose:
         print(" ".join(cmd), flush=True)
     subprocess.check_call(cmd)
+    os.replace(tmp, LIB)  # a reader sees the whole library or none
+    return LIB
+
+
+def ensure() -> str:
+    """The library, built first if it is not there; processes that start together build it once."""
+    import fcntl
+    if not os.path.exists(LIB):
+        with open(LIB + ".lock", "w") as lock:
+            fcntl.flock(lock, fcntl.LOCK_EX)
+            if not os.path.exists(LIB):
+                build(verbose=False, jobs=min(16, max(4, len(os.sched_getaffinity(0)))))
     return LIB
 
 

@@ -1,0 +1,796 @@
+// Layers of a block decoder: the token step and the prompt rows over a list of blocks with a mixer each, a loop of blocks
+// with shared weights, and a per-layer token input.  The residual, the norms, rotations, scores and softmax are fp32.
+//
+// Token step, launches per layer (the post-norm and residual add of a branch wait in `pend` for the next projection's
+// prologue, which also takes in what a loop pass adds):
+//   attention  [post-norm + norm1 + q|k|v]  [qk-norm + rotation + append + split attention]  [merge]  [out]
+//   latent     [post-norm + norm1 + q|c]    [W_uk onto q + rotation + latent norm + append]  [split attention]  [merge + W_uv]  [out]
+//   both       [post-norm + norm2 + up + relu^2]  [down]  [post-norm + gate + gelu * e]  [proj]
+// Prompt rows: the same with one GEMM per projection (activation and token input in its epilogue) and one row launch per norm.
+#include "blocks.h"
+
+#include <cmath>
+#include <new>
+#include <vector>
+
+namespace ptm {
+
+// ---- row kernels ------------------------------------------------------------------------------
+// grid rows: out[r][:] = table row of tokens[r], columns past `hidden` zero
+__global__ __launch_bounds__(256) void embed_bf16_rows_kernel(const uint16_t* __restrict__ table, int64_t ld, const int* __restrict__ tokens,
+                                                              int hidden, int wp, float* __restrict__ out, float* __restrict__ out2) {
+    const int64_t src = (int64_t)tokens[blockIdx.x] * ld, dst = (int64_t)blockIdx.x * wp;
+    for (int i = threadIdx.x; i < wp; i += 256) {
+        const float v = i < hidden ? bf16_f(table[src + i]) : 0.0f;
+        out[dst + i] = v;
+        if (out2) out2[dst + i] = v;
+    }
+}
+
+// grid rows: x += RMS(h) * hw + add0 + add1 (each optional), then xn = RMS(x) * gamma (gamma NULL: xn = x; xn NULL: nothing)
+template <bool F32>
+__global__ __launch_bounds__(256) void residual_norm_rows_kernel(float* __restrict__ x, const float* __restrict__ h,
+                                                                 const float* __restrict__ hw, const float* __restrict__ add0,
+                                                                 const float* __restrict__ add1, const float* __restrict__ gamma,
+                                                                 void* __restrict__ xn, int hidden, int wp, float eps) {
+    __shared__ float red[4];
+    const int64_t base = (int64_t)blockIdx.x * wp;
+    float4* x4 = reinterpret_cast<float4*>(x + base);
+    const float4* h4 = reinterpret_cast<const float4*>(h + base);
+    const float4* a4 = reinterpret_cast<const float4*>(add0 + base);
+    const int n4 = wp / 4;
+    constexpr int NS = 8;  // slots kept in registers: rows of up to 8192 values are read once
+    float4 xv[NS], hv[NS];
+    float rh = 0.0f;
+    if (h) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int u = 0; u < NS; ++u) {
+            const int i = threadIdx.x + 256 * u;
+            hv[u] = i < n4 ? h4[i] : make_float4(0.f, 0.f, 0.f, 0.f);
+            ss = fmaf(hv[u].x, hv[u].x, fmaf(hv[u].y, hv[u].y, fmaf(hv[u].z, hv[u].z, fmaf(hv[u].w, hv[u].w, ss))));
+        }
+        for (int i = threadIdx.x + 256 * NS; i < n4; i += 256) {
+            const float4 v = h4[i];
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+        }
+        rh = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)hidden + eps);
+    }
+    const float4* w4 = reinterpret_cast<const float4*>(hw);
+    const float4* b4 = reinterpret_cast<const float4*>(add1);
+    auto combine = [&](int i, float4 v, float4 hh) {
+        if (h) {
+            const float4 w = w4[i];
+            v = make_float4(v.x + hh.x * rh * w.x, v.y + hh.y * rh * w.y, v.z + hh.z * rh * w.z, v.w + hh.w * rh * w.w);
+        }
+        if (add0) { const float4 a = a4[i]; v = make_float4(v.x + a.x, v.y + a.y, v.z + a.z, v.w + a.w); }
+        if (add1) { const float4 a = b4[i]; v = make_float4(v.x + a.x, v.y + a.y, v.z + a.z, v.w + a.w); }
+        return v;
+    };
+    const bool changed = h || add0 || add1;
+    float ss = 0.0f;
+#pragma unroll
+    for (int u = 0; u < NS; ++u) {
+        const int i = threadIdx.x + 256 * u;
+        xv[u] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (i < n4) {
+            xv[u] = combine(i, x4[i], hv[u]);
+            if (changed) x4[i] = xv[u];
+        }
+        ss = fmaf(xv[u].x, xv[u].x, fmaf(xv[u].y, xv[u].y, fmaf(xv[u].z, xv[u].z, fmaf(xv[u].w, xv[u].w, ss))));
+    }
+    for (int i = threadIdx.x + 256 * NS; i < n4; i += 256) {
+        const float4 v = combine(i, x4[i], h ? h4[i] : make_float4(0.f, 0.f, 0.f, 0.f));
+        if (changed) x4[i] = v;
+        ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+    }
+    if (!xn) return;
+    float r = 1.0f;
+    if (gamma) r = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)hidden + eps);
+    const float4* g4 = reinterpret_cast<const float4*>(gamma);
+    auto emit = [&](int i, float4 v) {
+        if (gamma) {
+            const float4 g = g4[i];
+            v = make_float4(v.x * r * g.x, v.y * r * g.y, v.z * r * g.z, v.w * r * g.w);
+        }
+        if constexpr (F32) {
+            *reinterpret_cast<float4*>(static_cast<float*>(xn) + base + 4 * i) = v;
+        } else {
+            *reinterpret_cast<uint2*>(static_cast<uint16_t*>(xn) + base + 4 * i) =
+                make_uint2((uint32_t)f_bf16(v.x) | ((uint32_t)f_bf16(v.y) << 16), (uint32_t)f_bf16(v.z) | ((uint32_t)f_bf16(v.w) << 16));
+        }
+    };
+#pragma unroll
+    for (int u = 0; u < NS; ++u) {
+        const int i = threadIdx.x + 256 * u;
+        if (i < n4) emit(i, xv[u]);
+    }
+    for (int i = threadIdx.x + 256 * NS; i < n4; i += 256) emit(i, x4[i]);  // a thread reads back what it stored itself
+}
+
+// grid rows: compact copy of the residual rows
+__global__ __launch_bounds__(256) void copy_rows_kernel(const float* __restrict__ x, int wp, int hidden, float* __restrict__ out) {
+    for (int i = threadIdx.x; i < hidden; i += 256) out[(int64_t)blockIdx.x * hidden + i] = x[(int64_t)blockIdx.x * wp + i];
+}
+
+struct MixRows {
+    const float* raw;   // [rows][ld] projections
+    int64_t ld;
+    int heads, kv_heads, dim, vdim, rot_dim, rot_dims, kv_rank;
+    const float *q_norm, *k_norm, *rope;
+    float eps;
+    int64_t pos0;
+    const int64_t* d_past;  // position of row 0 instead of pos0, if given
+    void* q;            // [rows][q_row]
+    int64_t q_row;
+    void *k, *v;        // caches
+    int64_t k_row, v_row;
+};
+
+// element c of a head that starts at p, scaled by r and the norm weights w (NULL: none), rotated if c < rot_dims
+__device__ __forceinline__ float rotated(const float* p, const float* w, float r, int c, int rot_dims, const float* cs) {
+    const float v = w ? p[c] * r * w[c] : p[c];
+    if (c >= rot_dims) return v;
+    const float o = w ? p[c ^ 1] * r * w[c ^ 1] : p[c ^ 1], co = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
+    return (c & 1) ? v * co + o * sn : v * co - o * sn;
+}
+
+// grid rows: q and k normed over the whole projection and rotated, k and v appended; heads padded to multiples of 8 with zeros
+template <bool F32, bool Q32>
+__global__ __launch_bounds__(256) void attention_prep_rows_kernel(const MixRows a) {
+    __shared__ float red[4];
+    const int tid = threadIdx.x;
+    const int64_t pos = (a.d_past ? *a.d_past : a.pos0) + blockIdx.x;
+    const float *q = a.raw + blockIdx.x * a.ld, *k = q + a.heads * a.dim, *v = k + a.kv_heads * a.dim;
+    const float* cs = a.rope + pos * a.rot_dims;
+    const int nq = a.heads * a.dim, nk = a.kv_heads * a.dim, d8 = (a.dim + 7) & ~7, v8 = (a.vdim + 7) & ~7;
+    float sq = 0.0f, sk = 0.0f;
+    for (int i = tid; i < nq; i += 256) sq = fmaf(q[i], q[i], sq);
+    for (int i = tid; i < nk; i += 256) sk = fmaf(k[i], k[i], sk);
+    const float rq = 1.0f / sqrtf(block_sum<4>(sq, red) / (float)nq + a.eps);
+    const float rk = 1.0f / sqrtf(block_sum<4>(sk, red) / (float)nk + a.eps);
+    for (int i = tid; i < a.heads * d8; i += 256) {
+        const int h = i / d8, c = i % d8;
+        put_elem<Q32>(a.q, blockIdx.x * a.q_row + i, c < a.dim ? rotated(q + h * a.dim, a.q_norm + h * a.dim, rq, c, a.rot_dims, cs) : 0.0f);
+    }
+    for (int i = tid; i < a.kv_heads * d8; i += 256) {
+        const int h = i / d8, c = i % d8;
+        put_elem<F32>(a.k, pos * a.k_row + i, c < a.dim ? rotated(k + h * a.dim, a.k_norm + h * a.dim, rk, c, a.rot_dims, cs) : 0.0f);
+    }
+    for (int i = tid; i < a.kv_heads * v8; i += 256) {
+        const int h = i / v8, c = i % v8;
+        put_elem<F32>(a.v, pos * a.v_row + i, c < a.vdim ? v[h * a.vdim + c] : 0.0f);
+    }
+}
+
+// grid rows: latent normed and appended with the rotated key part; q per head [dim, 8-padded | rotated part, 8-padded]
+template <bool F32>
+__global__ __launch_bounds__(256) void latent_prep_rows_kernel(const MixRows a) {
+    __shared__ float red[4];
+    const int tid = threadIdx.x;
+    const int64_t pos = a.pos0 + blockIdx.x;
+    const int qd = a.dim + a.rot_dim, d8 = (a.dim + 7) & ~7, r8 = (a.rot_dim + 7) & ~7, rank8 = (a.kv_rank + 7) & ~7;
+    const float *q = a.raw + blockIdx.x * a.ld, *c = q + a.heads * qd, *kr = c + a.kv_rank;
+    const float* cs = a.rope + pos * a.rot_dims;
+    float ss = 0.0f;
+    for (int i = tid; i < a.kv_rank; i += 256) ss = fmaf(c[i], c[i], ss);
+    const float r = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.kv_rank + a.eps);
+    for (int i = tid; i < rank8 + r8; i += 256) {
+        float v = 0.0f;
+        if (i < rank8) { if (i < a.kv_rank) v = c[i] * r * a.k_norm[i]; }
+        else if (i - rank8 < a.rot_dim) v = rotated(kr, nullptr, 1.0f, i - rank8, a.rot_dims, cs);
+        put_elem<F32>(a.k, pos * a.k_row + i, v);
+    }
+    for (int i = tid; i < a.heads * (d8 + r8); i += 256) {
+        const int h = i / (d8 + r8), e = i % (d8 + r8);
+        const float* qh = q + h * qd;
+        float v = 0.0f;
+        if (e < d8) { if (e < a.dim) v = qh[e]; }
+        else if (e - d8 < a.rot_dim) v = rotated(qh + a.dim, nullptr, 1.0f, e - d8, a.rot_dims, cs);
+        put_elem<F32>(a.q, blockIdx.x * a.q_row + i, v);
+    }
+}
+
+// ---- the stack -----------------------------------------------------------------------------------
+struct LayerRun {
+    int block;
+    int enters_pass;      // first block of a loop pass: its number, else -1
+    void *k = nullptr, *v = nullptr;
+};
+
+struct BlockStack {
+    ptm_block_config cfg{};
+    std::vector<ptm_block> blocks;
+    std::vector<const float*> rope;  // per block
+    std::vector<LayerRun> runs;
+    std::vector<void*> allocs;
+    int wp = 0;           // padded width
+    bool f32 = false;
+    // token step
+    float *emb = nullptr, *xa = nullptr, *xb = nullptr, *hb = nullptr, *proj = nullptr, *q = nullptr, *attn = nullptr,
+          *act = nullptr, *gate = nullptr, *pO = nullptr, *pM = nullptr, *pL = nullptr;
+    // what the last branch left: the residual, and the branch output that still has to be normed and added
+    const float *x = nullptr, *pend_h = nullptr, *pend_w = nullptr;
+    // prompt rows
+    int rows = 0;
+    void* slab = nullptr;
+    int* r_tokens = nullptr;
+    float *r_x = nullptr, *r_emb = nullptr, *r_h = nullptr, *r_proj = nullptr;
+    void *r_xn = nullptr, *r_q = nullptr, *r_attn = nullptr, *r_act = nullptr, *r_gate = nullptr, *r_kv = nullptr;
+    const float *r_pend_h = nullptr, *r_pend_w = nullptr;
+};
+
+static int dev_alloc(BlockStack* b, size_t bytes, void** out) {
+    int rc = hip_status(hipMalloc(out, bytes));
+    if (rc != PTM_OK) return rc;
+    b->allocs.push_back(*out);
+    return hip_status(hipMemset(*out, 0, bytes));
+}
+
+static bool latent(const ptm_block& L) { return L.mixer == PTM_MIX_LATENT; }
+static int qkv_rows(const ptm_block& L) {
+    return latent(L) ? L.heads * (L.dim + L.rot_dim) + L.kv_rank + L.rot_dim : (L.heads + L.kv_heads) * L.dim + L.kv_heads * L.vdim;
+}
+static int attn_cols(const ptm_block& L) { return L.heads * up8(L.vdim); }
+static int q_cols(const ptm_block& L) { return L.heads * (up8(L.dim) + (latent(L) ? up8(L.rot_dim) : 0)); }
+static int64_t k_row(const ptm_block& L) { return latent(L) ? up8(L.kv_rank) + up8(L.rot_dim) : L.kv_heads * up8(L.dim); }
+static int64_t v_row(const ptm_block& L) { return latent(L) ? 0 : L.kv_heads * up8(L.vdim); }
+static int expand_rows(const ptm_block& L) { return L.heads * (up8(L.dim) + up8(L.vdim)); }
+
+static int matrix_check(const ptm_qweight& w, int rows, int cols) {
+    if (!w.data) return PTM_E_NULL;
+    if (w.ggml_type != PTM_TYPE_BF16) return PTM_E_UNSUPPORTED;
+    if (w.rows != rows || w.cols != cols || w.row_stride_bytes < 2 * (int64_t)up64(cols) || (w.row_stride_bytes & 15)) return PTM_E_SHAPE;
+    if (!aligned16(w.data)) return PTM_E_ALIGN;
+    return PTM_OK;
+}
+
+static int block_check(const ptm_block& L, int hidden, int side_dim) {
+    if (L.mixer != PTM_MIX_ATTENTION && L.mixer != PTM_MIX_LATENT) return PTM_E_UNSUPPORTED;
+    if (L.heads <= 0 || L.dim <= 0 || L.vdim <= 0 || L.window < 0 || L.keep_first < 0 || L.softcap < 0.0f) return PTM_E_SHAPE;
+    if (L.rot.dims < 0 || (L.rot.dims & 1)) return PTM_E_SHAPE;
+    int rc;
+    if (latent(L)) {
+        if (L.rot_dim <= 0 || L.kv_rank <= 0 || L.rot.dims > L.rot_dim) return PTM_E_SHAPE;
+        if (L.keep_first || L.softcap != 0.0f) return PTM_E_UNSUPPORTED;
+        if (!L.k_norm) return PTM_E_NULL;
+        if ((rc = matrix_check(L.expand, expand_rows(L), L.kv_rank))) return rc;
+    } else {
+        if (L.kv_heads <= 0 || L.heads % L.kv_heads || L.rot.dims > L.dim) return PTM_E_SHAPE;
+        if (!L.q_norm || !L.k_norm) return PTM_E_NULL;
+    }
+    if (!L.norm1 || !L.norm1b) return PTM_E_NULL;
+    if ((rc = matrix_check(L.in, qkv_rows(L), hidden)) || (rc = matrix_check(L.out, hidden, attn_cols(L)))) return rc;
+    if (L.ff < 0) return PTM_E_SHAPE;
+    if (L.ff > 0) {
+        if (!L.norm2 || !L.norm2b) return PTM_E_NULL;
+        if ((rc = matrix_check(L.up, L.ff, hidden)) || (rc = matrix_check(L.down, hidden, L.ff))) return rc;
+    }
+    if (L.side_gate.data) {
+        if (side_dim <= 0 || L.side_offset < 0) return PTM_E_SHAPE;
+        if (!L.side_norm) return PTM_E_NULL;
+        if ((rc = matrix_check(L.side_gate, side_dim, hidden)) || (rc = matrix_check(L.side_proj, hidden, side_dim))) return rc;
+    }
+    return PTM_OK;
+}
+
+// attention of the block's decode step, without pointers into the caches when run is NULL
+static ptm_attention_args decode_args(const BlockStack* b, const ptm_block& L, const LayerRun* run) {
+    ptm_attention_args a{};
+    const int es = b->f32 ? 4 : 2;
+    a.rows = 1;
+    a.heads = L.heads;
+    a.window = L.window;
+    a.keep_first = L.keep_first;
+    a.scale = L.scale;
+    a.softcap = L.softcap;
+    a.fp32 = b->f32;
+    a.Q = b->q;
+    if (latent(L)) {
+        a.kv_heads = 1;
+        a.dim1 = a.vdim = up8(L.kv_rank);
+        a.dim2 = up8(L.rot_dim);
+        a.k1_row = a.k2_row = a.v_row = k_row(L);
+        if (run) {
+            a.K1 = a.V = run->k;
+            a.K2 = static_cast<uint8_t*>(run->k) + (size_t)a.dim1 * es;
+        }
+    } else {
+        a.kv_heads = L.kv_heads;
+        a.dim1 = a.k1_head = up8(L.dim);
+        a.vdim = a.v_head = up8(L.vdim);
+        a.k1_row = k_row(L);
+        a.v_row = v_row(L);
+        if (run) { a.K1 = run->k; a.V = run->v; }
+    }
+    a.q_row = L.heads * (a.dim1 + a.dim2);
+    a.o_row = L.heads * a.vdim;
+    return a;
+}
+
+int blocks_create(const ptm_block_config& c, BlockStack** out) {
+    *out = nullptr;
+    if (!c.blocks || !c.out_norm) return PTM_E_NULL;
+    if (c.vocab <= 0 || c.hidden <= 0 || c.n_blocks <= 0 || c.max_seq <= 0) return PTM_E_SHAPE;
+    if (c.precision != PTM_PRECISION_16 && c.precision != PTM_PRECISION_32) return PTM_E_UNSUPPORTED;
+    if (c.loop_times < 0 || (c.loop_times > 0 && (c.loop_start < 0 || c.loop_start >= c.loop_stop || c.loop_stop > c.n_blocks))) return PTM_E_SHAPE;
+    if (c.loop_times > 0 && !c.loop_step) return PTM_E_NULL;
+    int rc;
+    if ((rc = matrix_check(c.lm_head, c.vocab, c.hidden)) || (rc = matrix_check(c.embedding, c.vocab, c.hidden))) return rc;
+    if (c.side_table.data && ((rc = matrix_check(c.side_table, c.vocab, c.side_table.cols)))) return rc;
+    for (int i = 0; i < c.n_blocks; ++i) {
+        if ((rc = block_check(c.blocks[i], c.hidden, c.side_dim))) return rc;
+        if (c.blocks[i].side_gate.data && (!c.side_table.data || c.blocks[i].side_offset + c.side_dim > c.side_table.cols)) return PTM_E_SHAPE;
+    }
+    BlockStack* b = new (std::nothrow) BlockStack();
+    if (!b) return PTM_E_STATE;
+    b->cfg = c;
+    b->blocks.assign(c.blocks, c.blocks + c.n_blocks);
+    b->cfg.blocks = b->blocks.data();
+    b->wp = up64(c.hidden);
+    b->f32 = c.precision == PTM_PRECISION_32;
+    for (int i = 0; i < c.n_blocks; ++i) {
+        if (c.loop_times > 0 && i == c.loop_start) {
+            for (int t = 0; t < c.loop_times; ++t)
+                for (int k = c.loop_start; k < c.loop_stop; ++k) b->runs.push_back({k, k == c.loop_start ? t : -1});
+            i = c.loop_stop - 1;
+        } else {
+            b->runs.push_back({i, -1});
+        }
+    }
+    const int es = b->f32 ? 4 : 2;
+    size_t proj = 0, q = 0, attn = 0, act = 64, pO = 0, pM = 0;
+    rc = PTM_OK;
+    for (int i = 0; rc == PTM_OK && i < c.n_blocks; ++i) {
+        const ptm_block& L = b->blocks[(size_t)i];
+        auto grow = [](size_t& v, size_t n) { v = v > n ? v : n; };
+        const ptm_attention_args a = decode_args(b, L, nullptr);
+        const size_t splits = (size_t)decode_attention_splits(a, c.max_seq);
+        grow(proj, (size_t)up64(qkv_rows(L)));
+        grow(q, (size_t)a.q_row);
+        grow(attn, (size_t)up64(attn_cols(L)));
+        grow(act, (size_t)up64(L.ff));
+        grow(pO, splits * (size_t)a.o_row);
+        grow(pM, splits * (size_t)L.heads);
+        // rotation table, shared with an earlier block that rotates alike
+        const float* table = nullptr;
+        for (int k = 0; k < i && !table; ++k) {
+            const ptm_rotation &r = b->blocks[(size_t)k].rot, &n = L.rot;
+            if (r.dims == n.dims && r.base == n.base && r.factor == n.factor && r.original == n.original && r.fast == n.fast && r.slow == n.slow)
+                table = b->rope[(size_t)k];
+        }
+        if (!table) {
+            std::vector<float> host((size_t)c.max_seq * (size_t)(L.rot.dims > 0 ? L.rot.dims : 2), 0.0f);
+            if (L.rot.dims > 0) rc = ptm_rope_pairs_host(host.data(), c.max_seq, &L.rot);
+            void* dev = nullptr;
+            if (rc == PTM_OK) rc = dev_alloc(b, host.size() * 4, &dev);
+            if (rc == PTM_OK) rc = hip_status(hipMemcpy(dev, host.data(), host.size() * 4, hipMemcpyHostToDevice));
+            table = static_cast<const float*>(dev);
+        }
+        b->rope.push_back(table);
+    }
+    for (size_t i = 0; rc == PTM_OK && i < b->runs.size(); ++i) {
+        const ptm_block& L = b->blocks[(size_t)b->runs[i].block];
+        // 64 values behind the last row: a GEMM over latents reads whole steps of 64 columns
+        rc = dev_alloc(b, ((size_t)c.max_seq * (size_t)k_row(L) + 64) * es, &b->runs[i].k);
+        if (rc == PTM_OK && !latent(L)) rc = dev_alloc(b, ((size_t)c.max_seq * (size_t)v_row(L) + 64) * es, &b->runs[i].v);
+    }
+    auto vec = [&](float*& p, size_t n) { if (rc == PTM_OK) rc = dev_alloc(b, (n + 64) * 4, reinterpret_cast<void**>(&p)); };
+    vec(b->emb, (size_t)b->wp);
+    vec(b->xa, (size_t)b->wp);
+    vec(b->xb, (size_t)b->wp);
+    vec(b->hb, (size_t)b->wp);
+    vec(b->proj, proj);
+    vec(b->q, q);
+    vec(b->attn, attn > q ? attn : q);
+    vec(b->act, act);
+    vec(b->gate, (size_t)up64(c.side_dim > 0 ? c.side_dim : 1));
+    vec(b->pO, pO);
+    vec(b->pM, pM);
+    vec(b->pL, pM);
+    if (rc != PTM_OK) { blocks_destroy(b); return rc; }
+    dense_gemv_init();
+    *out = b;
+    return PTM_OK;
+}
+
+void blocks_destroy(BlockStack* b) {
+    if (!b) return;
+    for (void* p : b->allocs) (void)hipFree(p);
+    if (b->slab) (void)hipFree(b->slab);
+    delete b;
+}
+
+int blocks_runs(const BlockStack* b) { return (int)b->runs.size(); }
+
+#define PTM_TRY(call) do { rc = (call); if (rc != PTM_OK) return rc; } while (0)
+
+static MixRows mix_rows(const BlockStack* b, const ptm_block& L, int block, const LayerRun& run) {
+    MixRows m{};
+    m.heads = L.heads;
+    m.kv_heads = L.kv_heads;
+    m.dim = L.dim;
+    m.vdim = L.vdim;
+    m.rot_dim = L.rot_dim;
+    m.rot_dims = L.rot.dims;
+    m.kv_rank = L.kv_rank;
+    m.q_norm = L.q_norm;
+    m.k_norm = L.k_norm;
+    m.rope = b->rope[(size_t)block];
+    m.eps = b->cfg.eps;
+    m.k = run.k;
+    m.v = run.v;
+    m.k_row = k_row(L);
+    m.v_row = v_row(L);
+    return m;
+}
+
+static int add_pending(BlockStack* b, hipStream_t s) {  // in place, for traced steps
+    if (!b->pend_h) return PTM_OK;
+    if (b->x == b->emb) {  // a loop adds the embedding output again: it stays as it is
+        const int rc = ptm_copy(b->emb, b->xa, b->wp, s);
+        if (rc != PTM_OK) return rc;
+        b->x = b->xa;
+    }
+    hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(1), dim3(256), 0, s, const_cast<float*>(b->x), b->pend_h, b->pend_w,
+                       (const float*)nullptr, (const float*)nullptr, (const float*)nullptr, (void*)nullptr, b->cfg.hidden, b->wp, b->cfg.eps);
+    b->pend_h = b->pend_w = nullptr;
+    return launch_status();
+}
+
+int blocks_token(BlockStack* b, const int* d_token, const int64_t* d_past, float* trace, hipStream_t s) {
+    const ptm_block_config& c = b->cfg;
+    int rc;
+    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(1), dim3(256), 0, s, static_cast<const uint16_t*>(c.embedding.data),
+                       c.embedding.row_stride_bytes / 2, d_token, c.hidden, b->wp, b->emb, (float*)nullptr);
+    PTM_TRY(launch_status());
+    b->x = b->emb;
+    b->pend_h = b->pend_w = nullptr;
+    const float *add0 = nullptr, *add1 = nullptr;
+    auto weight = [](DenseGemv& g, const ptm_qweight& w, float* y) {
+        g.W = static_cast<const uint16_t*>(w.data);
+        g.ld = w.row_stride_bytes / 2;
+        g.N = w.rows;
+        g.K = w.cols;
+        g.y = y;
+    };
+    // a projection of the residual: takes in whatever is pending and leaves the sum in the other residual buffer
+    auto from_x = [&](DenseGemv& g) {
+        g.x = b->x;
+        g.eps = c.eps;
+        g.h = b->pend_h;
+        g.hw = b->pend_w;
+        g.add0 = add0;
+        g.add1 = add1;
+        if (g.h || add0 || add1) {
+            g.xout = b->x == b->xa ? b->xb : b->xa;
+            b->x = g.xout;
+        }
+        b->pend_h = b->pend_w = add0 = add1 = nullptr;
+        return dense_gemv(g, s);
+    };
+    auto branch_out = [&](const ptm_qweight& w, const float* x, const float* post) {
+        DenseGemv g;
+        weight(g, w, b->hb);
+        g.x = x;
+        b->pend_h = b->hb;
+        b->pend_w = post;
+        return dense_gemv(g, s);
+    };
+    for (size_t ri = 0; ri < b->runs.size(); ++ri) {
+        const LayerRun& run = b->runs[ri];
+        const ptm_block& L = b->blocks[(size_t)run.block];
+        if (run.enters_pass >= 0) {
+            add0 = run.enters_pass > 0 ? b->emb : nullptr;
+            add1 = c.loop_step + (int64_t)run.enters_pass * b->wp;
+        }
+        {
+            DenseGemv g;
+            weight(g, L.in, b->proj);
+            g.gamma = L.norm1;
+            PTM_TRY(from_x(g));
+        }
+        DecodeAttention d{};
+        d.a = decode_args(b, L, &run);
+        d.d_past = d_past;
+        d.max_seq = c.max_seq;
+        d.pO = b->pO;
+        d.pM = b->pM;
+        d.pL = b->pL;
+        const bool tiled = decode_attention_tiled(d.a);
+        const int splits = decode_attention_splits(d.a, c.max_seq);
+        if (latent(L)) {
+            const LatentStep ls{b->proj, L.k_norm, b->rope[(size_t)run.block], static_cast<const uint16_t*>(L.expand.data),
+                                L.expand.row_stride_bytes / 2, L.heads, L.dim, L.rot_dim, L.rot.dims, L.kv_rank, L.vdim, c.eps, d_past,
+                                b->q, run.k, b->f32};
+            PTM_TRY(latent_absorb(ls, s));
+            if (tiled) {
+                PTM_TRY(decode_attention(d, s));
+                PTM_TRY(latent_out(ls, b->pO, b->pM, b->pL, splits, d.a.vdim, b->attn, s));
+            } else {
+                d.a.O = b->pO;
+                PTM_TRY(attention_rows(d.a, d_past, true, s));
+                PTM_TRY(latent_out(ls, b->pO, nullptr, nullptr, 1, d.a.vdim, b->attn, s));
+            }
+        } else if (tiled) {
+            d.raw = b->proj;
+            d.q_norm = L.q_norm;
+            d.k_norm = L.k_norm;
+            d.rope = b->rope[(size_t)run.block];
+            d.dim = L.dim;
+            d.vdim_true = L.vdim;
+            d.rot_dims = L.rot.dims;
+            d.eps = c.eps;
+            d.k_cache = run.k;
+            d.v_cache = run.v;
+            PTM_TRY(decode_attention(d, s));
+            PTM_TRY(decode_attention_merge(b->pO, b->pM, b->pL, splits, L.heads, d.a.vdim, b->attn, s));
+        } else {
+            MixRows m = mix_rows(b, L, run.block, run);
+            m.raw = b->proj;
+            m.d_past = d_past;
+            m.q = b->q;
+            m.q_row = d.a.q_row;
+            if (b->f32) hipLaunchKernelGGL((attention_prep_rows_kernel<true, true>), dim3(1), dim3(256), 0, s, m);
+            else hipLaunchKernelGGL((attention_prep_rows_kernel<false, true>), dim3(1), dim3(256), 0, s, m);
+            PTM_TRY(launch_status());
+            d.a.O = b->attn;
+            PTM_TRY(attention_rows(d.a, d_past, true, s));
+        }
+        PTM_TRY(branch_out(L.out, b->attn, L.norm1b));
+        if (trace) {
+            PTM_TRY(add_pending(b, s));
+            PTM_TRY(ptm_copy(b->x, trace + (2 * ri) * (size_t)c.hidden, c.hidden, s));
+        }
+        if (L.ff > 0) {
+            DenseGemv g;
+            weight(g, L.up, b->act);
+            g.gamma = L.norm2;
+            g.epilogue = GEMV_RELU2;
+            PTM_TRY(from_x(g));
+            PTM_TRY(branch_out(L.down, b->act, L.norm2b));
+        }
+        if (L.side_gate.data) {
+            DenseGemv g;
+            weight(g, L.side_gate, b->gate);
+            g.epilogue = GEMV_SIDE;
+            g.side = static_cast<const uint16_t*>(c.side_table.data);
+            g.side_ld = c.side_table.row_stride_bytes / 2;
+            g.side_off = L.side_offset;
+            g.d_token = d_token;
+            PTM_TRY(from_x(g));
+            PTM_TRY(branch_out(L.side_proj, b->gate, L.side_norm));
+        }
+        if (trace) {
+            PTM_TRY(add_pending(b, s));
+            PTM_TRY(ptm_copy(b->x, trace + (2 * ri + 1) * (size_t)c.hidden, c.hidden, s));
+        }
+    }
+    return PTM_OK;
+}
+
+int blocks_head(BlockStack* b, int row, float* logits, float* xn, int64_t* d_next, void* argmax_ws, const ArgmaxAdvance* adv,
+                hipStream_t s) {
+    const ptm_block_config& c = b->cfg;
+    DenseGemv g;
+    g.W = static_cast<const uint16_t*>(c.lm_head.data);
+    g.ld = c.lm_head.row_stride_bytes / 2;
+    g.N = c.vocab;
+    g.K = c.hidden;
+    g.x = row < 0 ? b->x : b->r_x + (int64_t)row * b->wp;
+    g.h = row < 0 ? b->pend_h : b->r_pend_h ? b->r_pend_h + (int64_t)row * b->wp : nullptr;
+    g.hw = row < 0 ? b->pend_w : b->r_pend_w;
+    g.gamma = c.out_norm;
+    g.eps = c.eps;
+    g.xn_out = xn;
+    g.y = logits;
+    if (!adv) return dense_gemv(g, s);
+    const int wgs = dense_gemv_workgroups(g);
+    g.epilogue = GEMV_ARGMAX;
+    g.part_val = static_cast<float*>(argmax_ws);
+    g.part_idx = reinterpret_cast<int*>(g.part_val + wgs);
+    const int rc = dense_gemv(g, s);
+    return rc != PTM_OK ? rc : argmax_finish(g.part_val, g.part_idx, wgs, d_next, *adv, s);
+}
+
+// ---- prompt rows -----------------------------------------------------------------------------------
+// positions a chunk of `rows` rows may have to expand latents for
+static size_t expand_positions(const BlockStack* b, const ptm_block& L, int rows) {
+    const size_t all = (size_t)b->cfg.max_seq, n = (size_t)rows + (size_t)L.window;
+    return L.window > 0 && n < all ? n : all;
+}
+
+int blocks_reserve(BlockStack* b, int rows) {
+    if (b->rows >= rows) return PTM_OK;
+    if (b->slab) { (void)hipFree(b->slab); b->slab = nullptr; b->rows = 0; }
+    const ptm_block_config& c = b->cfg;
+    const size_t R = (size_t)rows, es = b->f32 ? 4 : 2, W = (size_t)b->wp;
+    size_t proj = 0, q = 0, attn = 0, act = 64, kv = 0;
+    for (const ptm_block& L : b->blocks) {
+        auto grow = [](size_t& v, size_t n) { v = v > n ? v : n; };
+        grow(proj, (size_t)up64(qkv_rows(L)));
+        grow(q, (size_t)q_cols(L));
+        grow(attn, (size_t)up64(attn_cols(L)));
+        grow(act, (size_t)up64(L.ff));
+        if (latent(L)) grow(kv, expand_positions(b, L, rows) * (size_t)expand_rows(L));
+    }
+    size_t off = 0;
+    auto take = [&](size_t bytes) { const size_t o = off; off += (bytes + 511) & ~(size_t)255; return o; };
+    const size_t o_tok = take(4 * R), o_x = take(4 * R * W), o_e = take(4 * R * W), o_h = take(4 * R * W), o_p = take(4 * R * proj),
+                 o_xn = take(es * R * W), o_q = take(es * R * q), o_at = take(es * R * attn), o_ac = take(es * R * act),
+                 o_g = take(es * R * (size_t)up64(c.side_dim > 0 ? c.side_dim : 1)), o_kv = take(es * kv);
+    int rc = hip_status(hipMalloc(&b->slab, off));
+    if (rc != PTM_OK) return rc;
+    if ((rc = hip_status(hipMemset(b->slab, 0, off))) != PTM_OK) return rc;
+    uint8_t* p = static_cast<uint8_t*>(b->slab);
+    b->r_tokens = (int*)(p + o_tok);
+    b->r_x = (float*)(p + o_x);
+    b->r_emb = (float*)(p + o_e);
+    b->r_h = (float*)(p + o_h);
+    b->r_proj = (float*)(p + o_p);
+    b->r_xn = p + o_xn;
+    b->r_q = p + o_q;
+    b->r_attn = p + o_at;
+    b->r_act = p + o_ac;
+    b->r_gate = p + o_g;
+    b->r_kv = p + o_kv;
+    b->rows = rows;
+    return PTM_OK;
+}
+
+int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, float* trace, hipStream_t s) {
+    const ptm_block_config& c = b->cfg;
+    const bool f32 = b->f32;
+    const int es = f32 ? 4 : 2;
+    int rc;
+    if (M <= 0 || M > b->rows) return PTM_E_STATE;
+    PTM_TRY(hip_status(hipMemcpyAsync(b->r_tokens, tokens_host, 4 * (size_t)M, hipMemcpyHostToDevice, s)));
+    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(M), dim3(256), 0, s, static_cast<const uint16_t*>(c.embedding.data),
+                       c.embedding.row_stride_bytes / 2, b->r_tokens, c.hidden, b->wp, b->r_x, b->r_emb);
+    PTM_TRY(launch_status());
+    b->r_pend_h = b->r_pend_w = nullptr;
+    const float *add0 = nullptr, *add1 = nullptr;
+    // the residual rows take in what is pending; their norm (or, gamma NULL, a copy) goes to r_xn unless `only_add`
+    auto norm = [&](const float* gamma, bool only_add = false) {
+        void* xn = only_add ? nullptr : b->r_xn;
+        if (f32) hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
+        else hipLaunchKernelGGL(residual_norm_rows_kernel<false>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
+        b->r_pend_h = b->r_pend_w = add0 = add1 = nullptr;
+        return launch_status();
+    };
+    auto product = [&](const ptm_qweight& w, const void* A, int64_t lda, int rows, int epilogue, void* C, int64_t ldc) {
+        DenseGemm g;
+        g.A = A;
+        g.a_fp32 = f32;
+        g.lda = lda;
+        g.W = static_cast<const uint16_t*>(w.data);
+        g.ldw = w.row_stride_bytes / 2;
+        g.M = rows;
+        g.N = w.rows;
+        g.K = w.cols;
+        g.epilogue = epilogue;
+        g.C = C;
+        g.ldc = ldc;
+        return g;
+    };
+    auto branch_out = [&](const ptm_qweight& w, const void* A, const float* post) {
+        b->r_pend_h = b->r_h;
+        b->r_pend_w = post;
+        return dense_gemm(product(w, A, up64(w.cols), M, GEMM_F32, b->r_h, b->wp), s);
+    };
+    for (size_t ri = 0; ri < b->runs.size(); ++ri) {
+        const LayerRun& run = b->runs[ri];
+        const ptm_block& L = b->blocks[(size_t)run.block];
+        if (run.enters_pass >= 0) {
+            add0 = run.enters_pass > 0 ? b->r_emb : nullptr;
+            add1 = c.loop_step + (int64_t)run.enters_pass * b->wp;
+        }
+        PTM_TRY(norm(L.norm1));
+        const int ldp = up64(qkv_rows(L));
+        PTM_TRY(dense_gemm(product(L.in, b->r_xn, b->wp, M, GEMM_F32, b->r_proj, ldp), s));
+        MixRows m = mix_rows(b, L, run.block, run);
+        m.raw = b->r_proj;
+        m.ld = ldp;
+        m.pos0 = pos0;
+        m.q = b->r_q;
+        m.q_row = q_cols(L);
+        ptm_attention_args a{};
+        a.Q = b->r_q;
+        a.O = b->r_attn;
+        a.q_row = m.q_row;
+        a.o_row = up64(attn_cols(L));
+        a.rows = M;
+        a.heads = L.heads;
+        a.dim1 = up8(L.dim);
+        a.vdim = up8(L.vdim);
+        a.window = L.window;
+        a.keep_first = L.keep_first;
+        a.pos0 = pos0;
+        a.scale = L.scale;
+        a.softcap = L.softcap;
+        a.fp32 = f32;
+        if (latent(L)) {
+            if (f32) hipLaunchKernelGGL(latent_prep_rows_kernel<true>, dim3(M), dim3(256), 0, s, m);
+            else hipLaunchKernelGGL(latent_prep_rows_kernel<false>, dim3(M), dim3(256), 0, s, m);
+            PTM_TRY(launch_status());
+            // keys and values of every position some row of the chunk sees
+            const int64_t lo = L.window > 0 && pos0 - L.window + 1 > 0 ? pos0 - L.window + 1 : 0, row = k_row(L), er = expand_rows(L);
+            const uint8_t* cache = static_cast<const uint8_t*>(run.k);
+            PTM_TRY(dense_gemm(product(L.expand, cache + lo * row * es, row, (int)(pos0 + M - lo), GEMM_ELEM, b->r_kv, er), s));
+            a.kv_heads = L.heads;
+            a.K1 = b->r_kv;
+            a.k1_row = er;
+            a.k1_head = a.dim1;
+            a.V = static_cast<uint8_t*>(b->r_kv) + (size_t)L.heads * a.dim1 * es;
+            a.v_row = er;
+            a.v_head = a.vdim;
+            a.dim2 = up8(L.rot_dim);
+            a.K2 = cache + (lo * row + up8(L.kv_rank)) * es;
+            a.k2_row = row;
+            a.kv_pos0 = lo;
+        } else {
+            if (f32) hipLaunchKernelGGL((attention_prep_rows_kernel<true, true>), dim3(M), dim3(256), 0, s, m);
+            else hipLaunchKernelGGL((attention_prep_rows_kernel<false, false>), dim3(M), dim3(256), 0, s, m);
+            PTM_TRY(launch_status());
+            a.kv_heads = L.kv_heads;
+            a.K1 = run.k;
+            a.k1_row = m.k_row;
+            a.k1_head = a.dim1;
+            a.V = run.v;
+            a.v_row = m.v_row;
+            a.v_head = a.vdim;
+        }
+        PTM_TRY(attention_rows(a, nullptr, false, s));
+        PTM_TRY(branch_out(L.out, b->r_attn, L.norm1b));
+        if (L.ff > 0) {
+            PTM_TRY(norm(L.norm2));
+            PTM_TRY(dense_gemm(product(L.up, b->r_xn, b->wp, M, GEMM_RELU2, b->r_act, up64(L.ff)), s));
+            PTM_TRY(branch_out(L.down, b->r_act, L.norm2b));
+        }
+        if (L.side_gate.data) {
+            PTM_TRY(norm(nullptr));
+            DenseGemm g = product(L.side_gate, b->r_xn, b->wp, M, GEMM_SIDE, b->r_gate, up64(c.side_dim));
+            g.side = static_cast<const uint16_t*>(c.side_table.data);
+            g.side_ld = c.side_table.row_stride_bytes / 2;
+            g.side_off = L.side_offset;
+            g.tokens = b->r_tokens;
+            PTM_TRY(dense_gemm(g, s));
+            PTM_TRY(branch_out(L.side_proj, b->r_gate, L.side_norm));
+        }
+        if (trace) {
+            PTM_TRY(norm(nullptr, true));
+            hipLaunchKernelGGL(copy_rows_kernel, dim3(M), dim3(256), 0, s, b->r_x, b->wp, c.hidden, trace + ri * (size_t)M * (size_t)c.hidden);
+            PTM_TRY(launch_status());
+        }
+    }
+    return PTM_OK;
+}
+#undef PTM_TRY
+
+}  // namespace ptm
+
+extern "C" int ptm_rope_pairs_host(float* table, int max_seq, const ptm_rotation* rot) {
+    if (!table || !rot) return PTM_E_NULL;
+    if (max_seq <= 0 || rot->dims <= 0 || (rot->dims & 1) || !(rot->base > 0.0)) return PTM_E_SHAPE;
+    const int half = rot->dims / 2;
+    std::vector<double> f((size_t)half);
+    double amp = 1.0;
+    for (int i = 0; i < half; ++i) f[(size_t)i] = std::pow(rot->base, -2.0 * i / rot->dims);
+    if (rot->factor > 0.0) {
+        const double two_pi = 6.283185307179586476925;
+        auto turns = [&](double t) { return rot->dims * std::log(rot->original / (two_pi * t)) / (2.0 * std::log(rot->base)); };
+        const double lo = std::fmax(std::floor(turns(rot->fast)), 0.0), hi = std::fmin(std::ceil(turns(rot->slow)), rot->dims - 1.0);
+        for (int i = 0; i < half; ++i) {
+            const double ramp = std::fmin(std::fmax((i - lo) / std::fmax(hi - lo, 0.001), 0.0), 1.0);
+            f[(size_t)i] = f[(size_t)i] / rot->factor * ramp + f[(size_t)i] * (1.0 - ramp);
+        }
+        amp = 0.1 * std::log(rot->factor) + 1.0;
+    }
+    for (int p = 0; p < max_seq; ++p)
+        for (int i = 0; i < half; ++i) {
+            const double a = p * f[(size_t)i];
+            table[((size_t)p * half + i) * 2] = (float)(std::cos(a) * amp);
+            table[((size_t)p * half + i) * 2 + 1] = (float)(std::sin(a) * amp);
+        }
+    return PTM_OK;
+}

@@ -11,7 +11,10 @@
 //   o-proj GEMV accumulating into the residual
 //   rmsnorm + gate + up + SiLU*up in one launch
 //   down-proj GEMV accumulating into the residual
-#include "ptm_common.h"
+//
+// A decoder made by ptm_decode_create_blocks runs the layers of a block list (blocks.hip) in place of this fixed shape; steps,
+// graphs, prompts in chunks, sampling and everything else here is shared.
+#include "blocks.h"
 
 #include <cstring>
 #include <new>
@@ -148,6 +151,7 @@ struct ptm_decoder {
     float* pf_split = nullptr;  // K-split partial sums of the GEMMs
     size_t pf_split_bytes = 0;
     int* pf_tokens = nullptr;
+    BlockStack* blocks = nullptr;  // the layers of a block decoder; NULL: cfg.layers
 };
 
 static bool tuned_type(uint32_t t) { return t == PTM_TYPE_Q4_K || t == PTM_TYPE_Q6_K; }
@@ -191,6 +195,14 @@ static int enqueue_step(ptm_decoder* d, bool sample = false, float* trace = null
     const int H = c.hidden, hd = c.head_dim;
     int rc;
 #define PTM_TRY(call) do { rc = (call); if (rc != PTM_OK) return rc; } while (0)
+    if (d->blocks) {
+        PTM_TRY(blocks_token(d->blocks, d->d_token, d->d_past, trace, s));
+        const ArgmaxAdvance adv{d->d_token, d->d_past, d->d_step, d->d_tokens, c.max_seq};
+        PTM_TRY(blocks_head(d->blocks, -1, d->logits, d->xn, d->d_next, d->amax_ws, sample ? nullptr : &adv, s));
+        if (!sample) return PTM_OK;
+        return sampler_enqueue(d->logits, c.vocab, d->d_counts, d->sampling, d->d_sampling, d->d_uniforms, d->d_step, d->sampler_ws,
+                               d->d_next, d->d_counts, adv, true, s);
+    }
     if (c.embedding_f32) PTM_TRY(ptm_embedding_row(c.embedding_f32, d->x, d->d_token, H, s));
     else PTM_TRY(ptm_embedding_row_q6k(c.lm_head.data, d->x, d->d_token, H, c.lm_head.row_stride_bytes, s));
     if (c.scale_embeddings) PTM_TRY(ptm_scale(d->x, sqrtf((float)H), H, s));
@@ -327,6 +339,7 @@ static int enqueue_step(ptm_decoder* d, bool sample = false, float* trace = null
 // ---- prefill: M prompt rows through the layers at once (reference: GGUFModel::forward with use_cache,
 // torch/io/gguf_model.h:2510-2571 and transformer_layer :7300-7460) -------------------------------------------
 static int prefill_alloc(ptm_decoder* d, int rows) {
+    if (d->blocks) return blocks_reserve(d->blocks, rows);
     if (d->pf_rows >= rows) return PTM_OK;
     if (d->pf_slab) { (void)hipFree(d->pf_slab); d->pf_slab = nullptr; d->pf_rows = 0; }
     const ptm_decode_config& c = d->cfg;
@@ -378,7 +391,8 @@ static int prefill_alloc(ptm_decoder* d, int rows) {
 }
 
 // rows [0, M) of one chunk at positions pos0 .. pos0 + M - 1; leaves the residual rows in pf_x
-static int prefill_chunk(ptm_decoder* d, const int* tokens_host, int M, int64_t pos0) {
+static int prefill_chunk(ptm_decoder* d, const int* tokens_host, int M, int64_t pos0, float* trace = nullptr) {
+    if (d->blocks) return blocks_rows(d->blocks, tokens_host, M, pos0, trace, d->stream);
     const ptm_decode_config& c = d->cfg;
     hipStream_t s = d->stream;
     const int H = c.hidden, hd = c.head_dim, qd = c.n_heads * hd, kvd = c.n_kv_heads * hd, I = c.inter;
@@ -485,6 +499,65 @@ static int prefill_chunk(ptm_decoder* d, const int* tokens_host, int M, int64_t 
 #undef PTM_TRY
 }
 
+// scratch, device scalars, stream and tables of a decoder whose cfg (and blocks) are set
+static int decoder_init(ptm_decoder* d) {
+    const ptm_decode_config& c = d->cfg;
+    const int H = c.hidden, qd = c.n_heads * c.head_dim, kvd = c.n_kv_heads * c.head_dim;
+    const int S = ptm_flash_decode_num_splits(c.max_seq);
+    auto up16 = [](size_t b) { return (b + 255) & ~(size_t)255; };
+    size_t off = 0;
+    auto take = [&](size_t bytes) { const size_t o = off; off += up16(bytes); return o; };
+    const size_t o_x = take(4 * (size_t)H), o_xn = take(4 * (size_t)up64(H)), o_q = take(4 * (size_t)qd),
+                 o_k = take(4 * (size_t)kvd), o_v = take(4 * (size_t)kvd), o_attn = take(4 * (size_t)qd),
+                 o_act = take(4 * (size_t)c.inter), o_gate = take(4 * (size_t)c.inter),
+                 o_up = take(4 * (size_t)c.inter), o_logits = take(4 * (size_t)c.vocab),
+                 o_pO = take(4 * (size_t)S * c.n_heads * c.head_dim), o_pL = take(4 * (size_t)S * c.n_heads),
+                 o_pM = take(4 * (size_t)S * c.n_heads), o_rope = take(4 * (size_t)c.max_seq * c.head_dim),
+                 o_hb = take(4 * (size_t)H), o_x2 = take(4 * (size_t)H), o_rope_swa = take(c.swa_window > 0 ? 4 * (size_t)c.max_seq * c.head_dim : 0),
+                 o_xq8 = take((size_t)ptm_q8_bytes(qd > (H > c.inter ? H : c.inter) ? qd : (H > c.inter ? H : c.inter))),
+                 o_ws = take((size_t)ptm_argmax_workspace_bytes(c.vocab)), o_tok = take(256), o_past = take(256),
+                 o_next = take(256), o_step = take(256),
+                 o_samp = take(256), o_counts = take(4 * (size_t)c.vocab), o_unif = take(4 * (size_t)c.max_seq),
+                 o_sws = take((size_t)ptm_sampler_workspace_bytes());
+    int rc;
+    if ((rc = hip_status(hipMalloc(&d->slab, off))) != PTM_OK) return rc;
+    uint8_t* base = static_cast<uint8_t*>(d->slab);
+    d->x = (float*)(base + o_x); d->xn = (float*)(base + o_xn); d->q = (float*)(base + o_q);
+    d->k = (float*)(base + o_k); d->v = (float*)(base + o_v); d->attn = (float*)(base + o_attn);
+    d->act = (float*)(base + o_act); d->gate = (float*)(base + o_gate); d->up = (float*)(base + o_up);
+    d->logits = (float*)(base + o_logits); d->pO = (float*)(base + o_pO); d->pL = (float*)(base + o_pL);
+    d->pM = (float*)(base + o_pM); d->rope = (float*)(base + o_rope); d->xq8 = base + o_xq8;
+    d->hb = (float*)(base + o_hb); d->x2 = (float*)(base + o_x2); d->rope_swa = c.swa_window > 0 ? (float*)(base + o_rope_swa) : d->rope;
+    d->amax_ws = base + o_ws; d->d_token = (int*)(base + o_tok); d->d_past = (int64_t*)(base + o_past);
+    d->d_next = (int64_t*)(base + o_next); d->d_step = (int*)(base + o_step);
+    d->d_sampling = (ptm_sampling*)(base + o_samp); d->d_counts = (int32_t*)(base + o_counts);
+    d->d_uniforms = (float*)(base + o_unif); d->sampler_ws = base + o_sws;
+    if ((rc = hip_status(hipMemset(d->sampler_ws, 0, (size_t)ptm_sampler_workspace_bytes()))) != PTM_OK) return rc;
+    q6k_init_attributes();  // one-time kernel attributes, before anything can be captured
+
+    if ((rc = hip_status(hipStreamCreateWithFlags(&d->stream, hipStreamNonBlocking))) != PTM_OK) return rc;
+    if ((rc = hip_status(hipHostMalloc((void**)&d->h_pinned, 8 * (size_t)c.max_seq, hipHostMallocDefault))) != PTM_OK) return rc;
+    // token ids go from the step's last kernel straight to pinned host memory (an 8-byte store per token): no copy launch
+    // between the step and the host's read
+    if ((rc = hip_status(hipHostGetDevicePointer((void**)&d->d_tokens, d->h_pinned, 0))) != PTM_OK) return rc;
+    if ((rc = hip_status(hipHostMalloc((void**)&d->h_uniforms, 4 * (size_t)c.max_seq, hipHostMallocDefault))) != PTM_OK) return rc;
+    if (!d->blocks) {  // a block decoder's rotations are its layers' own
+        std::vector<float> tab((size_t)c.max_seq * c.head_dim);
+        ptm_rope_table_host_factors(tab.data(), c.max_seq, c.head_dim, c.rope_freq_base, c.rope_scale, c.rope_factors_short,
+                                    c.rope_factors_long, c.rope_orig_ctx, c.rope_attn_factor);
+        if ((rc = hip_status(hipMemcpy(d->rope, tab.data(), tab.size() * 4, hipMemcpyHostToDevice))) != PTM_OK) return rc;
+        if (c.swa_window > 0) {  // ModelConfig::layer_rope_freq_base / layer_rope_scale, gguf_model.h:297-302
+            ptm_rope_table_host_factors(tab.data(), c.max_seq, c.head_dim, c.rope_swa_freq_base, 1.0f, c.rope_factors_short,
+                                        c.rope_factors_long, c.rope_orig_ctx, c.rope_attn_factor);
+            if ((rc = hip_status(hipMemcpy(d->rope_swa, tab.data(), tab.size() * 4, hipMemcpyHostToDevice))) != PTM_OK) return rc;
+        }
+    }
+    hipLaunchKernelGGL(set_scalars_kernel, dim3(1), dim3(1), 0, d->stream, d->d_token, 0, d->d_past, (int64_t)0, d->d_step);
+    if ((rc = hip_status(hipStreamSynchronize(d->stream))) != PTM_OK) return rc;
+    return PTM_OK;
+}
+
+
 extern "C" {
 
 int ptm_decode_create(const ptm_decode_config* cfg, ptm_decoder** out) {
@@ -528,59 +601,33 @@ int ptm_decode_create(const ptm_decode_config* cfg, ptm_decoder** out) {
         for (const ptm_qweight* w : {&L.q, &L.k, &L.v, &L.o, &L.gate, &L.up, &L.down})
             if (!tuned_type(w->ggml_type)) d->untuned_types = true;
 
-    const int S = ptm_flash_decode_num_splits(c.max_seq);
-    auto up16 = [](size_t b) { return (b + 255) & ~(size_t)255; };
-    size_t off = 0;
-    auto take = [&](size_t bytes) { const size_t o = off; off += up16(bytes); return o; };
-    const size_t o_x = take(4 * (size_t)H), o_xn = take(4 * (size_t)H), o_q = take(4 * (size_t)qd),
-                 o_k = take(4 * (size_t)kvd), o_v = take(4 * (size_t)kvd), o_attn = take(4 * (size_t)qd),
-                 o_act = take(4 * (size_t)c.inter), o_gate = take(4 * (size_t)c.inter),
-                 o_up = take(4 * (size_t)c.inter), o_logits = take(4 * (size_t)c.vocab),
-                 o_pO = take(4 * (size_t)S * c.n_heads * c.head_dim), o_pL = take(4 * (size_t)S * c.n_heads),
-                 o_pM = take(4 * (size_t)S * c.n_heads), o_rope = take(4 * (size_t)c.max_seq * c.head_dim),
-                 o_hb = take(4 * (size_t)H), o_x2 = take(4 * (size_t)H), o_rope_swa = take(c.swa_window > 0 ? 4 * (size_t)c.max_seq * c.head_dim : 0),
-                 o_xq8 = take((size_t)ptm_q8_bytes(qd > (H > c.inter ? H : c.inter) ? qd : (H > c.inter ? H : c.inter))),
-                 o_ws = take((size_t)ptm_argmax_workspace_bytes(c.vocab)), o_tok = take(256), o_past = take(256),
-                 o_next = take(256), o_step = take(256),
-                 o_samp = take(256), o_counts = take(4 * (size_t)c.vocab), o_unif = take(4 * (size_t)c.max_seq),
-                 o_sws = take((size_t)ptm_sampler_workspace_bytes());
-    if ((rc = hip_status(hipMalloc(&d->slab, off))) != PTM_OK) { delete d; return rc; }
-    uint8_t* base = static_cast<uint8_t*>(d->slab);
-    d->x = (float*)(base + o_x); d->xn = (float*)(base + o_xn); d->q = (float*)(base + o_q);
-    d->k = (float*)(base + o_k); d->v = (float*)(base + o_v); d->attn = (float*)(base + o_attn);
-    d->act = (float*)(base + o_act); d->gate = (float*)(base + o_gate); d->up = (float*)(base + o_up);
-    d->logits = (float*)(base + o_logits); d->pO = (float*)(base + o_pO); d->pL = (float*)(base + o_pL);
-    d->pM = (float*)(base + o_pM); d->rope = (float*)(base + o_rope); d->xq8 = base + o_xq8;
-    d->hb = (float*)(base + o_hb); d->x2 = (float*)(base + o_x2); d->rope_swa = c.swa_window > 0 ? (float*)(base + o_rope_swa) : d->rope;
-    d->amax_ws = base + o_ws; d->d_token = (int*)(base + o_tok); d->d_past = (int64_t*)(base + o_past);
-    d->d_next = (int64_t*)(base + o_next); d->d_step = (int*)(base + o_step);
-    d->d_sampling = (ptm_sampling*)(base + o_samp); d->d_counts = (int32_t*)(base + o_counts);
-    d->d_uniforms = (float*)(base + o_unif); d->sampler_ws = base + o_sws;
-    if ((rc = hip_status(hipMemset(d->sampler_ws, 0, (size_t)ptm_sampler_workspace_bytes()))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-    q6k_init_attributes();  // one-time kernel attributes, before anything can be captured
-
-    if ((rc = hip_status(hipStreamCreateWithFlags(&d->stream, hipStreamNonBlocking))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-    if ((rc = hip_status(hipHostMalloc((void**)&d->h_pinned, 8 * (size_t)c.max_seq, hipHostMallocDefault))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-    // token ids go from the step's last kernel straight to pinned host memory (an 8-byte store per token): no copy launch
-    // between the step and the host's read
-    if ((rc = hip_status(hipHostGetDevicePointer((void**)&d->d_tokens, d->h_pinned, 0))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-    if ((rc = hip_status(hipHostMalloc((void**)&d->h_uniforms, 4 * (size_t)c.max_seq, hipHostMallocDefault))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-    {
-        std::vector<float> tab((size_t)c.max_seq * c.head_dim);
-        ptm_rope_table_host_factors(tab.data(), c.max_seq, c.head_dim, c.rope_freq_base, c.rope_scale, c.rope_factors_short,
-                                    c.rope_factors_long, c.rope_orig_ctx, c.rope_attn_factor);
-        if ((rc = hip_status(hipMemcpy(d->rope, tab.data(), tab.size() * 4, hipMemcpyHostToDevice))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-        if (c.swa_window > 0) {  // ModelConfig::layer_rope_freq_base / layer_rope_scale, gguf_model.h:297-302
-            ptm_rope_table_host_factors(tab.data(), c.max_seq, c.head_dim, c.rope_swa_freq_base, 1.0f, c.rope_factors_short,
-                                        c.rope_factors_long, c.rope_orig_ctx, c.rope_attn_factor);
-            if ((rc = hip_status(hipMemcpy(d->rope_swa, tab.data(), tab.size() * 4, hipMemcpyHostToDevice))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
-        }
-    }
-    hipLaunchKernelGGL(set_scalars_kernel, dim3(1), dim3(1), 0, d->stream, d->d_token, 0, d->d_past, (int64_t)0, d->d_step);
-    if ((rc = hip_status(hipStreamSynchronize(d->stream))) != PTM_OK) { ptm_decode_destroy(d); return rc; }
+    if ((rc = decoder_init(d)) != PTM_OK) { ptm_decode_destroy(d); return rc; }
     *out = d;
     return PTM_OK;
 }
+
+int ptm_decode_create_blocks(const ptm_block_config* cfg, ptm_decoder** out) {
+    if (!cfg || !out) return PTM_E_NULL;
+    *out = nullptr;
+    ptm_decoder* d = new (std::nothrow) ptm_decoder();
+    if (!d) return PTM_E_STATE;
+    int rc = blocks_create(*cfg, &d->blocks);
+    if (rc != PTM_OK) { delete d; return rc; }
+    ptm_decode_config& c = d->cfg;
+    c.vocab = cfg->vocab;
+    c.hidden = cfg->hidden;
+    c.n_layers = blocks_runs(d->blocks);
+    c.max_seq = cfg->max_seq;
+    c.rms_eps = cfg->eps;
+    c.use_graph = cfg->use_graph;
+    c.lm_head = cfg->lm_head;
+    c.out_norm = cfg->out_norm;
+    if ((rc = decoder_init(d)) != PTM_OK) { ptm_decode_destroy(d); return rc; }
+    *out = d;
+    return PTM_OK;
+}
+
+int ptm_decode_layer_runs(const ptm_decoder* d) { return d ? d->cfg.n_layers : 0; }
 
 void ptm_decode_destroy(ptm_decoder* d) {
     if (!d) return;
@@ -593,6 +640,7 @@ void ptm_decode_destroy(ptm_decoder* d) {
     if (d->h_uniforms) (void)hipHostFree(d->h_uniforms);
     if (d->pf_slab) (void)hipFree(d->pf_slab);
     if (d->slab) (void)hipFree(d->slab);
+    blocks_destroy(d->blocks);
     if (d->stream) (void)hipStreamDestroy(d->stream);
     delete d;
 }
@@ -771,18 +819,50 @@ int ptm_decode_reserve_prefill(ptm_decoder* d, int rows) {
     return prefill_alloc(d, rows);
 }
 
-int ptm_decode_prefill(ptm_decoder* d, const int32_t* tokens, int n, int chunk_rows, int64_t* next_token) {
-    if (!d || !tokens || !next_token) return PTM_E_NULL;
+// Final norm, logits and argmax of prompt row `row` of the last chunk; adv NULL: no step bookkeeping.
+static int row_head(ptm_decoder* d, int row, const ArgmaxAdvance& adv) {
+    const ptm_decode_config& c = d->cfg;
+    hipStream_t s = d->stream;
+    if (d->blocks) return blocks_head(d->blocks, row, d->logits, d->xn, d->d_next, d->amax_ws, &adv, s);
+    int rc = hip_status(hipMemcpyAsync(d->x, d->pf_x + (size_t)row * c.hidden, 4 * (size_t)c.hidden, hipMemcpyDeviceToDevice, s));
+    if (rc != PTM_OK) return rc;
+    if (c.lm_head.ggml_type == PTM_TYPE_Q6_K)
+        return q6k_gemv_argmax_impl(c.lm_head.data, d->x, c.out_norm, c.rms_eps, 0, d->xn, d->logits, c.hidden, c.vocab,
+                                    c.lm_head.row_stride_bytes, d->d_next, d->amax_ws, adv, s);
+    rc = ptm_rms_norm(d->x, c.out_norm, d->xn, 1, c.hidden, c.rms_eps, 0, nullptr, s);
+    if (rc == PTM_OK) rc = gemv_any(c.lm_head, d->xn, d->logits, false, s);
+    if (rc == PTM_OK) rc = ptm_argmax(d->logits, d->d_next, c.vocab, s);
+    if (rc == PTM_OK && adv.d_token) {
+        hipLaunchKernelGGL(advance_kernel, dim3(1), dim3(1), 0, s, d->d_next, d->d_token, d->d_past, d->d_step, d->d_tokens, c.max_seq);
+        rc = launch_status();
+    }
+    return rc;
+}
+
+// The prompt in chunks; logits of the places `want` (ascending) go to logits_host.  trace: one chunk, block decoders.
+static int prefill_any(ptm_decoder* d, const int32_t* tokens, int n, int chunk_rows, const int32_t* want, int n_want,
+                       float* logits_host, int64_t* next_token, float* trace) {
+    if (!d || !tokens || !next_token || (n_want > 0 && (!want || !logits_host))) return PTM_E_NULL;
     if (d->status != PTM_OK) return PTM_E_STATE;
-    if (n <= 0) return PTM_E_SHAPE;
+    if (n <= 0 || n_want < 0) return PTM_E_SHAPE;
     if (d->past_len + n > d->cfg.max_seq) return PTM_E_RANGE;  // KV cache would overflow
     for (int i = 0; i < n; ++i)
         if (tokens[i] < 0 || tokens[i] >= d->cfg.vocab) return PTM_E_RANGE;
+    for (int i = 0; i < n_want; ++i)
+        if (want[i] < 0 || want[i] >= n || (i > 0 && want[i] <= want[i - 1])) return PTM_E_RANGE;
     const ptm_decode_config& c = d->cfg;
+    hipStream_t s = d->stream;
+    int rc = PTM_OK, wi = 0;
+    auto copy_logits = [&]() {
+        return hip_status(hipMemcpyAsync(logits_host + (size_t)wi++ * c.vocab, d->logits, 4 * (size_t)c.vocab, hipMemcpyDeviceToHost, s));
+    };
     if (d->untuned_types) {
         // no row-batched GEMM for these types: the prompt is stepped, each step a full decode step whose token is dropped
-        int rc = PTM_OK;
-        for (int i = 0; i < n && rc == PTM_OK; ++i) rc = run_steps(d, tokens[i], 1);
+        for (int i = 0; i < n && rc == PTM_OK; ++i) {
+            rc = run_steps(d, tokens[i], 1);
+            if (rc == PTM_OK && wi < n_want && want[wi] == i) rc = copy_logits();
+        }
+        if (rc == PTM_OK) rc = hip_status(hipStreamSynchronize(s));
         if (rc == PTM_OK) *next_token = d->h_pinned[d->out_base];
         return rc;
     }
@@ -790,40 +870,58 @@ int ptm_decode_prefill(ptm_decoder* d, const int32_t* tokens, int n, int chunk_r
     if (chunk_rows <= 0) chunk_rows = 2048;  // measured: 2048-row chunks run a 4096-token prompt 1.4x faster than 512-row ones
     if (chunk_rows > 2048) chunk_rows = 2048;  // bounds the row scratch (and the launch grids) whatever the prompt length
     if (chunk_rows > n) chunk_rows = n;
-    int rc = prefill_alloc(d, chunk_rows);
-    if (rc != PTM_OK) return rc;
-    hipStream_t s = d->stream;
+    if (trace && chunk_rows < n) return PTM_E_SHAPE;
+    if ((rc = prefill_alloc(d, chunk_rows)) != PTM_OK) return rc;
     int last_rows = 0;
     for (int done = 0; done < n; done += last_rows) {
         last_rows = n - done < chunk_rows ? n - done : chunk_rows;
-        if ((rc = prefill_chunk(d, tokens + done, last_rows, d->past_len + done)) != PTM_OK) return d->status = rc;
+        if ((rc = prefill_chunk(d, tokens + done, last_rows, d->past_len + done, trace)) != PTM_OK) return d->status = rc;
+        for (; wi < n_want && want[wi] < done + last_rows && want[wi] < n - 1;) {
+            if ((rc = row_head(d, want[wi] - done, ArgmaxAdvance{nullptr, nullptr, nullptr, nullptr, 0})) != PTM_OK) return d->status = rc;
+            if ((rc = copy_logits()) != PTM_OK) return d->status = rc;
+        }
     }
-    // only the last row is projected to logits (gguf_model.h:2551-2559): hand it to the decode tail, with the device-side
-    // position set so that the tail's bookkeeping leaves it at past_len + n
-    if ((rc = hip_status(hipMemcpyAsync(d->x, d->pf_x + (size_t)(last_rows - 1) * c.hidden, 4 * (size_t)c.hidden,
-                                        hipMemcpyDeviceToDevice, s))) != PTM_OK) return d->status = rc;
+    // the last row is handed to the decode tail (without `want`, the only one projected to logits: gguf_model.h:2551-2559), with
+    // the device-side position set so that the tail's bookkeeping leaves it at past_len + n
     hipLaunchKernelGGL(set_scalars_kernel, dim3(1), dim3(1), 0, s, d->d_token, (int)tokens[n - 1], d->d_past,
                        d->past_len + n - 1, d->d_step);
     if ((rc = launch_status()) != PTM_OK) return d->status = rc;
-    if (c.lm_head.ggml_type == PTM_TYPE_Q6_K) {
-        rc = q6k_gemv_argmax_impl(c.lm_head.data, d->x, c.out_norm, c.rms_eps, 0, d->xn, d->logits, c.hidden, c.vocab,
-                                  c.lm_head.row_stride_bytes, d->d_next, d->amax_ws,
-                                  ArgmaxAdvance{d->d_token, d->d_past, d->d_step, d->d_tokens, c.max_seq}, s);
-    } else {
-        rc = ptm_rms_norm(d->x, c.out_norm, d->xn, 1, c.hidden, c.rms_eps, 0, nullptr, s);
-        if (rc == PTM_OK) rc = gemv_any(c.lm_head, d->xn, d->logits, false, s);
-        if (rc == PTM_OK) rc = ptm_argmax(d->logits, d->d_next, c.vocab, s);
-        if (rc == PTM_OK) {
-            hipLaunchKernelGGL(advance_kernel, dim3(1), dim3(1), 0, s, d->d_next, d->d_token, d->d_past, d->d_step,
-                               d->d_tokens, c.max_seq);
-            rc = launch_status();
-        }
-    }
+    rc = row_head(d, last_rows - 1, ArgmaxAdvance{d->d_token, d->d_past, d->d_step, d->d_tokens, c.max_seq});
+    if (rc == PTM_OK && wi < n_want) rc = copy_logits();
     if (rc != PTM_OK) return d->status = rc;
     if ((rc = hip_status(hipStreamSynchronize(s))) != PTM_OK) return d->status = rc;
     d->past_len += n;
     *next_token = d->h_pinned[0];
     return PTM_OK;
+}
+
+int ptm_decode_prefill(ptm_decoder* d, const int32_t* tokens, int n, int chunk_rows, int64_t* next_token) {
+    return prefill_any(d, tokens, n, chunk_rows, nullptr, 0, nullptr, next_token, nullptr);
+}
+
+int ptm_decode_prefill_logits(ptm_decoder* d, const int32_t* tokens, int n, int chunk_rows, const int32_t* want, int n_want,
+                              float* logits_host, int64_t* next_token) {
+    return prefill_any(d, tokens, n, chunk_rows, want, n_want, logits_host, next_token, nullptr);
+}
+
+int ptm_decode_prefill_trace(ptm_decoder* d, const int32_t* tokens, int n, int64_t* next_token, float* trace_host) {
+    if (!d || !trace_host) return PTM_E_NULL;
+    if (!d->blocks) return PTM_E_UNSUPPORTED;
+    if (n <= 0) return PTM_E_SHAPE;
+    const size_t bytes = 4 * (size_t)d->cfg.n_layers * (size_t)n * (size_t)d->cfg.hidden;
+    void* buf = nullptr;
+    int rc = hip_status(hipMalloc(&buf, bytes));
+    if (rc != PTM_OK) return rc;
+    rc = prefill_any(d, tokens, n, n, nullptr, 0, nullptr, next_token, static_cast<float*>(buf));
+    if (rc == PTM_OK) rc = hip_status(hipMemcpy(trace_host, buf, bytes, hipMemcpyDeviceToHost));
+    (void)hipFree(buf);
+    return rc;
+}
+
+int ptm_decode_read_logits(ptm_decoder* d, float* logits_host) {
+    if (!d || !logits_host) return PTM_E_NULL;
+    const int rc = hip_status(hipStreamSynchronize(d->stream));
+    return rc != PTM_OK ? rc : hip_status(hipMemcpy(logits_host, d->logits, 4 * (size_t)d->cfg.vocab, hipMemcpyDeviceToHost));
 }
 
 int ptm_decode_step(ptm_decoder* d, int token_id, int64_t* next_token) {

@@ -10,7 +10,7 @@
 //   n_tensors x { string name | u32 n_dims | u64 dims[n_dims] | u32 ggml_type | u64 offset }
 //   padding to general.alignment (default 32) | tensor data (offsets relative to here)
 // dims[0] is the contiguous dimension (K, columns), dims[1] the rows (N).
-#include "ptm_common.h"
+#include "model.h"
 
 #include <fcntl.h>
 #include <sys/mman.h>
@@ -151,13 +151,18 @@ struct ptm_gguf {
     std::map<std::string, size_t> index;
 };
 
-struct ptm_model {
-    ptm_gguf* file = nullptr;
-    std::vector<void*> device_allocs;
-    std::vector<ptm_layer> layers;
-    ptm_decode_config cfg{};
-    ptm_decoder* dec = nullptr;
-};
+namespace ptm {
+int model_upload(ptm_model* m, const void* src, size_t bytes, void** dev) {
+    void* d = nullptr;
+    int rc = hip_status(hipMalloc(&d, bytes));
+    if (rc != PTM_OK) return rc;
+    m->device_allocs.push_back(d);
+    if (src) rc = hip_status(hipMemcpy(d, src, bytes, hipMemcpyHostToDevice));
+    else rc = hip_status(hipMemset(d, 0, bytes));
+    *dev = d;
+    return rc;
+}
+}  // namespace ptm
 
 extern "C" {
 
@@ -322,16 +327,7 @@ void ptm_model_free(ptm_model* m) {
     delete m;
 }
 
-static int upload(ptm_model* m, const void* src, size_t bytes, void** dev) {
-    void* d = nullptr;
-    int rc = hip_status(hipMalloc(&d, bytes));
-    if (rc != PTM_OK) return rc;
-    m->device_allocs.push_back(d);
-    if (src) rc = hip_status(hipMemcpy(d, src, bytes, hipMemcpyHostToDevice));
-    else rc = hip_status(hipMemset(d, 0, bytes));
-    *dev = d;
-    return rc;
-}
+static int upload(ptm_model* m, const void* src, size_t bytes, void** dev) { return model_upload(m, src, bytes, dev); }
 
 // a [rows x cols] Q4_K / Q6_K matrix: uploaded verbatim
 static int load_matrix(ptm_model* m, const std::string& name, int64_t rows, int64_t cols, ptm_qweight* w) {

@@ -249,6 +249,11 @@ __global__ __launch_bounds__(1024) void argmax_partials_kernel(const float* pv, 
     }
 }
 
+int argmax_finish(const float* part_val, const int* part_idx, int n, int64_t* out_index, const ArgmaxAdvance adv, hipStream_t s) {
+    hipLaunchKernelGGL(argmax_partials_kernel, dim3(1), dim3(1024), 0, s, part_val, part_idx, n, out_index, adv);
+    return launch_status();
+}
+
 static int q6k_check(const void* W, const void* x, int K, int N, int64_t stride) {
     if (!W || !x) return PTM_E_NULL;
     if (K <= 0 || N <= 0 || (K % 256) != 0) return PTM_E_SHAPE;
@@ -381,8 +386,7 @@ int q6k_gemv_argmax_impl(const void* W, const float* x, const float* gamma, floa
               reinterpret_cast<int*>(static_cast<float*>(workspace) + grid), gamma, eps, add_one, xn_out};
     const int rc2 = gamma ? q6k_launch<false, true, true>(a, s) : q6k_launch<false, true, false>(a, s);
     if (rc2 != PTM_OK) return rc2;
-    hipLaunchKernelGGL(argmax_partials_kernel, dim3(1), dim3(1024), 0, s, a.part_val, a.part_idx, grid, out_index, adv);
-    return launch_status();
+    return argmax_finish(a.part_val, a.part_idx, grid, out_index, adv, s);
 }
 
 }  // namespace ptm

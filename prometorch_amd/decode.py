@@ -12,6 +12,7 @@ import torch
 
 from . import _lib
 from ._lib import DecodeConfig, Layer, QWeight, check
+from .model import Stepper
 
 _NAMES = ("q", "k", "v", "o", "gate", "up", "down")
 
@@ -20,7 +21,7 @@ def _upload_bytes(a: np.ndarray) -> torch.Tensor:
     return torch.from_numpy(np.ascontiguousarray(a, dtype=np.uint8)).cuda()
 
 
-class Decoder:
+class Decoder(Stepper):
     """Greedy batch-1 decoder over caller-provided quantised weights.
 
     layers: list of dicts with (qtype, uint8[rows, stride]) per projection name and fp32 norm
@@ -114,11 +115,6 @@ class Decoder:
         torch.cuda.synchronize()
         check(self.L.ptm_decode_set_past_len(self.h, n), "decode_set_past_len")
 
-    def step(self, token: int) -> int:
-        out = C.c_int64()
-        check(self.L.ptm_decode_step(self.h, token, C.byref(out)), "decode_step")
-        return out.value
-
     def step_trace(self, token: int):
         """One step as plain launches that also returns the residual stream after every layer's attention branch and after
         its feed-forward branch: (token, trace[n_layers, 2, hidden])."""
@@ -127,57 +123,11 @@ class Decoder:
         check(self.L.ptm_decode_step_trace(self.h, token, C.byref(out), trace.data_ptr()), "decode_step_trace")
         return out.value, trace.cpu().numpy()
 
-    def prefill(self, tokens, chunk_rows: int = 0) -> int:
-        """Run the prompt through the model in row batches, appending its K/V rows; returns the greedy next token
-        (GGUFModel::forward with use_cache, gguf_model.h:2510-2571)."""
-        n = len(tokens)
-        buf = (C.c_int32 * n)(*[int(t) for t in tokens])
-        out = C.c_int64()
-        check(self.L.ptm_decode_prefill(self.h, buf, n, chunk_rows, C.byref(out)), "decode_prefill")
-        return out.value
-
-    def generate(self, prompt, uniforms, temperature: float, top_k: int, top_p: float, repeat_penalty: float = 1.0,
-                 stop_ids=()) -> list:
-        """Prompt, then up to len(uniforms) sampled tokens, ending before the first stop token (the serving loop of
-        promeserve/api_handlers.h:848-923 with everything but the token ids kept on the device)."""
-        from ._lib import Sampling
-        n, m, ns = len(prompt), len(uniforms), len(stop_ids)
-        pa = (C.c_int32 * n)(*[int(t) for t in prompt])
-        ua = (C.c_float * m)(*[float(u) for u in uniforms])
-        sa = (C.c_int32 * max(1, ns))(*[int(t) for t in stop_ids])
-        out = (C.c_int64 * m)()
-        n_out = C.c_int()
-        check(self.L.ptm_decode_generate(self.h, pa, n, Sampling(temperature, top_k, top_p, repeat_penalty), ua, m, sa, ns, out,
-                                         C.byref(n_out)), "decode_generate")
-        return list(out[:n_out.value])
-
-    def sampling_begin(self, temperature: float, top_k: int, top_p: float, repeat_penalty: float = 1.0) -> None:
-        """Start a sampled generation: store the parameters, forget previously generated tokens."""
-        from ._lib import Sampling
-        check(self.L.ptm_decode_sampling_begin(self.h, Sampling(temperature, top_k, top_p, repeat_penalty)),
-              "decode_sampling_begin")
-
-    def sample(self, token: int, uniforms) -> list:
-        """len(uniforms) chained sampled steps from `token`, one uniform draw per step."""
-        n = len(uniforms)
-        u = (C.c_float * n)(*[float(x) for x in uniforms])
-        buf = (C.c_int64 * n)()
-        check(self.L.ptm_decode_sample(self.h, token, n, u, buf), "decode_sample")
-        return list(buf)
-
-    def greedy(self, first_token: int, n: int) -> list:
-        buf = (C.c_int64 * n)()
-        check(self.L.ptm_decode_greedy(self.h, first_token, n, buf), "decode_greedy")
-        return list(buf)
-
     def _view(self, ptr: int, n: int) -> np.ndarray:
         out = torch.empty(n, dtype=torch.float32, device="cuda")
         _lib.check(self.L.ptm_copy(ptr, out.data_ptr(), n, None), "copy")
         torch.cuda.synchronize()
         return out.cpu().numpy()
-
-    def logits(self) -> np.ndarray:
-        return self._view(self.L.ptm_decode_logits(self.h), self.cfg["vocab"])
 
     def hidden(self) -> np.ndarray:
         return self._view(self.L.ptm_decode_hidden(self.h), self.cfg["hidden"])

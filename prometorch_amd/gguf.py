@@ -8,7 +8,8 @@ import ctypes as C
 import numpy as np
 
 from . import _lib
-from ._lib import DecodeConfig, GgufTensor, Layer, check
+from ._lib import GgufTensor, Layer, check
+from .model import LoadedModel
 
 F32, F16, Q4_K, Q6_K = 0, 1, 12, 14
 _T_U32, _T_I32, _T_F32, _T_BOOL, _T_STR, _T_ARR, _T_U64 = 4, 5, 6, 7, 8, 9, 10
@@ -106,7 +107,7 @@ class GGUFFile:
 # ---------------------------------------------------------------------------------------------
 # model loader
 # ---------------------------------------------------------------------------------------------
-class GGUFModel:
+class GGUFModel(LoadedModel):
     """A decoder created straight from a .gguf file; same stepping interface as decode.Decoder."""
 
     def __init__(self, path: str, max_seq: int, kv_fp16: bool = True, use_graph: bool = True):
@@ -114,11 +115,7 @@ class GGUFModel:
         m = C.c_void_p()
         check(self.L.ptm_model_load_gguf(path.encode(), max_seq, int(kv_fp16), int(use_graph), C.byref(m)),
               f"model_load_gguf({path})")
-        self.m = m
-        self._path = path
-        self.h = self.L.ptm_model_decoder(m)
-        c = DecodeConfig()
-        check(self.L.ptm_model_config(m, C.byref(c)), "model_config")
+        c = self._adopt(m, path)
         self.cfg = {k: getattr(c, k) for k in ("vocab", "hidden", "n_layers", "n_heads", "n_kv_heads", "head_dim", "inter", "max_seq")}
         self.cfg.update(rope_base=c.rope_freq_base, eps=c.rms_eps, kv_fp16=bool(c.kv_fp16), tied=not bool(c.embedding_f32),
                         rope_interleaved=bool(c.rope_interleaved), rope_scale=c.rope_scale,
@@ -140,36 +137,6 @@ class GGUFModel:
             n4 = nbytes // 4  # rows are multiples of 4 bytes: reuse the fp32 copy kernel for the raw bytes
             check(self.L.ptm_copy(t.data_ptr(), ptr, n4, None), "copy")
         torch.cuda.synchronize()
-
-    def set_past_len(self, n: int) -> None:
-        check(self.L.ptm_decode_set_past_len(self.h, n), "decode_set_past_len")
-
-    def step(self, token: int) -> int:
-        out = C.c_int64()
-        check(self.L.ptm_decode_step(self.h, token, C.byref(out)), "decode_step")
-        return out.value
-
-    def prefill(self, tokens, chunk_rows: int = 0) -> int:
-        n = len(tokens)
-        buf = (C.c_int32 * n)(*[int(t) for t in tokens])
-        out = C.c_int64()
-        check(self.L.ptm_decode_prefill(self.h, buf, n, chunk_rows, C.byref(out)), "decode_prefill")
-        return out.value
-
-    def generate(self, prompt, uniforms, temperature: float, top_k: int, top_p: float, repeat_penalty: float = 1.0,
-                 stop_ids=()) -> list:
-        """Prompt, then up to len(uniforms) sampled tokens, ending before the first stop token (the serving loop of
-        promeserve/api_handlers.h:848-923 with everything but the token ids kept on the device)."""
-        from ._lib import Sampling
-        n, m, ns = len(prompt), len(uniforms), len(stop_ids)
-        pa = (C.c_int32 * n)(*[int(t) for t in prompt])
-        ua = (C.c_float * m)(*[float(u) for u in uniforms])
-        sa = (C.c_int32 * max(1, ns))(*[int(t) for t in stop_ids])
-        out = (C.c_int64 * m)()
-        n_out = C.c_int()
-        check(self.L.ptm_decode_generate(self.h, pa, n, Sampling(temperature, top_k, top_p, repeat_penalty), ua, m, sa, ns, out,
-                                         C.byref(n_out)), "decode_generate")
-        return list(out[:n_out.value])
 
     # the reference's stop strings besides the file's eos id (GGUFModel::is_stop_token, gguf_model.h:5132-5139)
     STOP_TOKENS = ("<|im_end|>", "<|endoftext|>", "<end_of_turn>", "<|eot_id|>", "</s>", "<|end|>")
@@ -200,44 +167,9 @@ class GGUFModel:
                             repeat_penalty, stop_ids=self._stops)
         return self._tok.decode(out).decode("utf-8", errors="replace")
 
-    def sampling_begin(self, temperature: float, top_k: int, top_p: float, repeat_penalty: float = 1.0) -> None:
-        """Start a sampled generation: store the parameters, forget previously generated tokens."""
-        from ._lib import Sampling
-        check(self.L.ptm_decode_sampling_begin(self.h, Sampling(temperature, top_k, top_p, repeat_penalty)),
-              "decode_sampling_begin")
-
-    def sample(self, token: int, uniforms) -> list:
-        """len(uniforms) chained sampled steps from `token`, one uniform draw per step."""
-        n = len(uniforms)
-        u = (C.c_float * n)(*[float(x) for x in uniforms])
-        buf = (C.c_int64 * n)()
-        check(self.L.ptm_decode_sample(self.h, token, n, u, buf), "decode_sample")
-        return list(buf)
-
-    def greedy(self, first_token: int, n: int) -> list:
-        buf = (C.c_int64 * n)()
-        check(self.L.ptm_decode_greedy(self.h, first_token, n, buf), "decode_greedy")
-        return list(buf)
-
-    def logits(self) -> np.ndarray:
-        import torch
-        out = torch.empty(self.cfg["vocab"], dtype=torch.float32, device="cuda")
-        check(self.L.ptm_copy(self.L.ptm_decode_logits(self.h), out.data_ptr(), self.cfg["vocab"], None), "copy")
-        torch.cuda.synchronize()
-        return out.cpu().numpy()
-
     def close(self) -> None:
         if getattr(self, "_tok", None) is not None:
             self._tok.close()
             self._file.close()
             self._tok = self._file = None
-        if getattr(self, "m", None):
-            self.L.ptm_model_free(self.m)
-            self.m = None
-            self.h = None
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
+        super().close()
