@@ -133,6 +133,110 @@ def only_kernel(which, torch, ops, synth):
     return out
 
 
+# Tovasun layers at the sizes of the models above: [latent, attention] pairs, bfloat16 weights.  `like`: the closest existing
+# model (GQA, two norms a layer, gated feed-forward, Q4_K_M weights) with as many layers of the same width, heads and inter size.
+BLOCK_SHAPES = {
+    "width_2560": dict(width=2560, heads=32, kv_heads=8, dim=128, ff=9728, rank=512, rot=64, window=1024, long_window=4096, side=256),
+    "width_4096": dict(width=4096, heads=32, kv_heads=8, dim=128, ff=14336, rank=512, rot=64, window=1024, long_window=4096, side=256),
+}
+BLOCK_LAYERS, BLOCK_VOCAB = 8, 32768
+
+
+def block_model_config(s):
+    lat = {"heads": s["heads"], "dim": s["dim"], "rot_dim": s["rot"], "kv_rank": s["rank"], "vdim": s["dim"],
+           "scale": (s["dim"] + s["rot"]) ** -0.5, "mask": {"size": s["window"]},
+           "rot": {"base": 10000.0, "dims": s["rot"], "scaling": {"factor": 4.0, "fast": 32.0, "slow": 1.0, "original": 4096}}}
+    att = {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5, "softcap": 30.0,
+           "mask": {"size": s["long_window"], "keep_first": 4}, "rot": {"base": 10000.0, "dims": s["dim"] // 2}}
+    layers = [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}}
+              for _ in range(BLOCK_LAYERS // 2) for t, m in (("latent_attention", lat), ("attention", att))]
+    return {"architecture": "Tovasun", "layers": layers, "norm": {"eps": 1e-6}, "vocab": BLOCK_VOCAB, "width": s["width"],
+            "token_side": {"dim": s["side"]}}
+
+
+def blocks_main(steps, warmup, only=None):
+    """Decode and prompt throughput of Tovasun models beside the closest existing model of the same size."""
+    import shutil
+    import tempfile
+    import torch
+    from prometorch_amd import _lib, model as registry
+    from prometorch_amd.decode import Decoder
+    from prometorch_amd.testing import folder_writer as fw, synth
+    _lib.load()
+    torch.cuda.set_device(0)
+    pool = fw.to_bf16(np.random.default_rng(SEED).standard_normal(1 << 24, np.float32) * 0.02)
+
+    def measure(m):
+        tokens = [int(t) for t in synth.rng_for(SEED, 77).integers(0, BLOCK_VOCAB, 2048)]
+        r = {}
+        for n in (512, 2048):
+            m.set_past_len(0)
+            m.prefill(tokens[:n])
+            ts = []
+            for _ in range(3):
+                m.set_past_len(0)
+                t0 = time.perf_counter()
+                m.prefill(tokens[:n])
+                ts.append(time.perf_counter() - t0)
+            r["prefill_%d_ms" % n] = sorted(ts)[1] * 1e3
+            r["prefill_%d_tok_s" % n] = n / sorted(ts)[1]
+        tok = 1
+        for _ in range(warmup):
+            tok = m.step(tok)
+        t0 = time.perf_counter()
+        for _ in range(steps):
+            tok = m.step(tok)
+        r["decode_ms_per_token"] = (time.perf_counter() - t0) / steps * 1e3
+        r["decode_tok_s"] = 1e3 / r["decode_ms_per_token"]
+        return r
+
+    out = {"workload": "tovasun", "layers": BLOCK_LAYERS, "vocab": BLOCK_VOCAB, "past": 2048, "steps": steps, "data": "synthetic, random weights"}
+    for name, s in BLOCK_SHAPES.items():
+        if only and name != only:
+            continue
+        cfg = block_model_config(s)
+        shapes = fw.tensor_shapes(cfg)
+        folder = tempfile.mkdtemp(prefix="tovasun_bench_")
+        try:
+            json.dump(cfg, open(os.path.join(folder, "config.json"), "w"))
+            one = fw.to_bf16(np.ones(1, np.float32))[0]
+            arrays = {n: np.full(sh, one) if len(sh) == 1 else np.resize(pool, sh) for n, sh in shapes.items()}
+            fw.write_safetensors(os.path.join(folder, "model.safetensors"), arrays)
+            del arrays
+            t0 = time.time()
+            m = registry.load(folder, max_seq=4096)
+            log("%s: loaded in %.1fs" % (name, time.time() - t0))
+        finally:
+            shutil.rmtree(folder)
+        mine = measure(m)
+        m.close()
+        read = sum(2 * int(np.prod(sh)) for n, sh in shapes.items() if n not in ("embed", "side.embed"))
+        kv = BLOCK_LAYERS // 2 * (s["window"] * (s["rank"] + s["rot"]) + 2048 * 2 * s["kv_heads"] * s["dim"]) * 2
+        mine["decode_bytes"] = read + kv
+        mine["decode_hbm_frac"] = (read + kv) / mine["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBS
+        mats = sum(int(np.prod(sh)) for n, sh in shapes.items() if len(sh) == 2 and n not in ("embed", "side.embed", "head"))
+        mine["prefill_2048_matrix_tflops"] = 2 * mats * 2048 / mine["prefill_2048_ms"] / 1e9
+        lcfg = dict(synth.QWEN3_4B, hidden=s["width"], n_layers=BLOCK_LAYERS, n_heads=s["heads"], n_kv_heads=s["kv_heads"],
+                    head_dim=s["dim"], inter=s["ff"], vocab=BLOCK_VOCAB)
+        layers = [synth.make_layer(SEED, i, lcfg) for i in range(BLOCK_LAYERS)]
+        head = synth.make_head(SEED, lcfg)
+        d = Decoder(lcfg, layers, head, max_seq=4096)
+        like = measure(d)
+        d.close()
+        read = sum(W.nbytes for L in layers for W in (L[k][1] for k in ("q", "k", "v", "o", "gate", "up", "down"))) + head["lm_head"].nbytes
+        kv = BLOCK_LAYERS * 2048 * 2 * s["kv_heads"] * s["dim"] * 2
+        like["decode_bytes"] = read + kv
+        like["decode_hbm_frac"] = (read + kv) / like["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBS
+        H, q = s["width"], s["heads"] * s["dim"]
+        mats = BLOCK_LAYERS * (2 * H * q + 2 * H * s["kv_heads"] * s["dim"] + 3 * H * s["ff"])
+        like["prefill_2048_matrix_tflops"] = 2 * mats * 2048 / like["prefill_2048_ms"] / 1e9
+        out[name] = {"tovasun_bf16": mine, "qwen3_like_q4_k_m": like}
+        for k, v in out[name].items():
+            log(name, k, {a: round(b, 3) for a, b in v.items()})
+        torch.cuda.empty_cache()
+    return out
+
+
 def main():
     # stdout carries exactly one line, the JSON result: anything a native library prints to file descriptor 1 in the
     # meantime (the compiled reference reports its scratch allocation there) is sent to stderr instead
@@ -156,7 +260,14 @@ def main():
     ap.add_argument("--only", choices=["prefill_gemm", "prefill_attention"], default=None,
                     help="launch just this prompt-pass kernel a few times and print its time: the target of the counter "
                          "passes behind the figures quoted for it (rocprofv3 --pmc ... -- python3 bench.py --only ...)")
+    ap.add_argument("--tovasun", nargs="?", const="all", choices=["all"] + sorted(BLOCK_SHAPES),
+                    help="instead of the default workload: Tovasun models (latent and grouped-query attention layers, bfloat16 weights) "
+                         "beside the closest existing model at equal sizes")
     args = ap.parse_args()
+    if args.tovasun:
+        result = blocks_main(args.steps, args.warmup, None if args.tovasun == "all" else args.tovasun)
+        os.write(json_fd, (json.dumps(result) + "\n").encode())
+        return
     if args.cpu_child > 0:
         os.dup2(json_fd, 1)
         cpu_child_main(args.cpu_child)

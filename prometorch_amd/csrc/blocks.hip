@@ -388,6 +388,8 @@ int blocks_create(const ptm_block_config& c, BlockStack** out) {
     vec(b->pO, pO);
     vec(b->pM, pM);
     vec(b->pL, pM);
+    // the clears above run on the null stream, which the decoder's own stream does not wait for
+    if (rc == PTM_OK) rc = hip_status(hipStreamSynchronize(nullptr));
     if (rc != PTM_OK) { blocks_destroy(b); return rc; }
     dense_gemv_init();
     *out = b;
@@ -622,6 +624,7 @@ int blocks_reserve(BlockStack* b, int rows) {
     int rc = hip_status(hipMalloc(&b->slab, off));
     if (rc != PTM_OK) return rc;
     if ((rc = hip_status(hipMemset(b->slab, 0, off))) != PTM_OK) return rc;
+    if ((rc = hip_status(hipStreamSynchronize(nullptr))) != PTM_OK) return rc;  // before the decoder's stream writes there
     uint8_t* p = static_cast<uint8_t*>(b->slab);
     b->r_tokens = (int*)(p + o_tok);
     b->r_x = (float*)(p + o_x);

@@ -553,6 +553,7 @@ static int decoder_init(ptm_decoder* d) {
         }
     }
     hipLaunchKernelGGL(set_scalars_kernel, dim3(1), dim3(1), 0, d->stream, d->d_token, 0, d->d_past, (int64_t)0, d->d_step);
+    if ((rc = hip_status(hipStreamSynchronize(nullptr))) != PTM_OK) return rc;  // the clears ran there
     if ((rc = hip_status(hipStreamSynchronize(d->stream))) != PTM_OK) return rc;
     return PTM_OK;
 }
