@@ -16,10 +16,10 @@ FLAGS = [
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     "-Wall", "-Wno-unused-function", "-Wno-unknown-warning-option", "-Wno-unused-command-line-argument",
 ]
-# Per-file additions.  prefill.hip: its matrix-core attention rescales the output accumulators between MFMAs with vector
+# Per-file additions.  prefill.hip, mixer_attention.hip: their matrix-core attention rescales the output accumulators between MFMAs with vector
 # arithmetic, which cannot touch accumulation registers; with the accumulators there the compiler copies all 64 of them
 # out and back on every tile.  One wave per SIMD leaves room for them in ordinary registers.
-FILE_FLAGS = {"prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}
+FILE_FLAGS = {name: ["-mllvm", "-amdgpu-mfma-vgpr-form"] for name in ("prefill.hip", "mixer_attention.hip")}
 
 
 def build(verbose: bool = True, jobs: int = 8) -> str:

@@ -16,29 +16,44 @@
 namespace ptm {
 
 // ---- row kernels ------------------------------------------------------------------------------
-// grid rows: out[r][:] = table row of tokens[r], columns past `hidden` zero
-__global__ __launch_bounds__(256) void embed_bf16_rows_kernel(const uint16_t* __restrict__ table, int64_t ld, const int* __restrict__ tokens,
-                                                              int hidden, int wp, float* __restrict__ out, float* __restrict__ out2) {
-    const int64_t src = (int64_t)tokens[blockIdx.x] * ld, dst = (int64_t)blockIdx.x * wp;
-    for (int i = threadIdx.x; i < wp; i += 256) {
-        const float v = i < hidden ? bf16_f(table[src + i]) : 0.0f;
-        out[dst + i] = v;
-        if (out2) out2[dst + i] = v;
-    }
+// grid (rows, wp / 512): out[r][:] = table row of tokens[r] (the table's rows are padded like the output's)
+__global__ __launch_bounds__(128) void embed_bf16_rows_kernel(const uint16_t* __restrict__ table, int64_t ld, const int* __restrict__ tokens,
+                                                              int wp, float* __restrict__ out, float* __restrict__ out2) {
+    const int i = (blockIdx.y * 128 + threadIdx.x) * 4;
+    if (i >= wp) return;
+    const uint2 u = *reinterpret_cast<const uint2*>(table + (int64_t)tokens[blockIdx.x] * ld + i);
+    const float4 v = make_float4(bf16_lo(u.x), bf16_hi(u.x), bf16_lo(u.y), bf16_hi(u.y));
+    *reinterpret_cast<float4*>(out + (int64_t)blockIdx.x * wp + i) = v;
+    if (out2) *reinterpret_cast<float4*>(out2 + (int64_t)blockIdx.x * wp + i) = v;
 }
 
-// grid rows: x += RMS(h) * hw + add0 + add1 (each optional), then xn = RMS(x) * gamma (gamma NULL: xn = x; xn NULL: nothing)
+// grid rows: x += RMS(h) * hw + add0 + add1 (each optional), then xn = RMS(x) * gamma (gamma NULL: xn = x; xn NULL: nothing).
+// h may still be `slabs` partial sums, `slab` floats apart.
 template <bool F32>
 __global__ __launch_bounds__(256) void residual_norm_rows_kernel(float* __restrict__ x, const float* __restrict__ h,
-                                                                 const float* __restrict__ hw, const float* __restrict__ add0,
-                                                                 const float* __restrict__ add1, const float* __restrict__ gamma,
-                                                                 void* __restrict__ xn, int hidden, int wp, float eps) {
+                                                                 int slabs, int64_t slab, const float* __restrict__ hw,
+                                                                 const float* __restrict__ add0, const float* __restrict__ add1,
+                                                                 const float* __restrict__ gamma, void* __restrict__ xn, int hidden, int wp, float eps) {
     __shared__ float red[4];
     const int64_t base = (int64_t)blockIdx.x * wp;
     float4* x4 = reinterpret_cast<float4*>(x + base);
     const float4* h4 = reinterpret_cast<const float4*>(h + base);
     const float4* a4 = reinterpret_cast<const float4*>(add0 + base);
     const int n4 = wp / 4;
+    auto h_at = [&](int i) {
+        float4 v = h4[i];
+        for (int z = 1; z < slabs; ++z) {
+            const float4 p = *reinterpret_cast<const float4*>(h + base + z * slab + 4 * i);
+            v = make_float4(v.x + p.x, v.y + p.y, v.z + p.z, v.w + p.w);
+        }
+        if (4 * i + 3 >= hidden) {  // the slabs' padding is not kept clear
+            if (4 * i >= hidden) v.x = 0.0f;
+            if (4 * i + 1 >= hidden) v.y = 0.0f;
+            if (4 * i + 2 >= hidden) v.z = 0.0f;
+            v.w = 4 * i + 3 >= hidden ? 0.0f : v.w;
+        }
+        return v;
+    };
     constexpr int NS = 8;  // slots kept in registers: rows of up to 8192 values are read once
     float4 xv[NS], hv[NS];
     float rh = 0.0f;
@@ -47,11 +62,11 @@ __global__ __launch_bounds__(256) void residual_norm_rows_kernel(float* __restri
 #pragma unroll
         for (int u = 0; u < NS; ++u) {
             const int i = threadIdx.x + 256 * u;
-            hv[u] = i < n4 ? h4[i] : make_float4(0.f, 0.f, 0.f, 0.f);
+            hv[u] = i < n4 ? h_at(i) : make_float4(0.f, 0.f, 0.f, 0.f);
             ss = fmaf(hv[u].x, hv[u].x, fmaf(hv[u].y, hv[u].y, fmaf(hv[u].z, hv[u].z, fmaf(hv[u].w, hv[u].w, ss))));
         }
         for (int i = threadIdx.x + 256 * NS; i < n4; i += 256) {
-            const float4 v = h4[i];
+            const float4 v = h_at(i);
             ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
         }
         rh = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)hidden + eps);
@@ -80,7 +95,7 @@ __global__ __launch_bounds__(256) void residual_norm_rows_kernel(float* __restri
         ss = fmaf(xv[u].x, xv[u].x, fmaf(xv[u].y, xv[u].y, fmaf(xv[u].z, xv[u].z, fmaf(xv[u].w, xv[u].w, ss))));
     }
     for (int i = threadIdx.x + 256 * NS; i < n4; i += 256) {
-        const float4 v = combine(i, x4[i], h ? h4[i] : make_float4(0.f, 0.f, 0.f, 0.f));
+        const float4 v = combine(i, x4[i], h ? h_at(i) : make_float4(0.f, 0.f, 0.f, 0.f));
         if (changed) x4[i] = v;
         ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
     }
@@ -113,6 +128,28 @@ __global__ __launch_bounds__(256) void copy_rows_kernel(const float* __restrict_
     for (int i = threadIdx.x; i < hidden; i += 256) out[(int64_t)blockIdx.x * hidden + i] = x[(int64_t)blockIdx.x * wp + i];
 }
 
+struct SideRows {
+    const float* g;     // [slabs][rows][ld] partial sums of W_gate x
+    int slabs;
+    int64_t slab, ld;
+    const uint16_t* table;
+    int64_t table_ld;
+    int offset, dim;
+    const int* tokens;
+    void* out;          // [rows][ld]
+};
+// grid rows: out = gelu_tanh(g) * e, e the token's row of the side table from column `offset`
+template <bool F32>
+__global__ __launch_bounds__(256) void side_rows_kernel(const SideRows a) {
+    const uint16_t* e = a.table + (int64_t)a.tokens[blockIdx.x] * a.table_ld + a.offset;
+    const int64_t base = blockIdx.x * a.ld;
+    for (int i = threadIdx.x; i < a.dim; i += 256) {
+        float v = 0.0f;
+        for (int z = 0; z < a.slabs; ++z) v += a.g[base + z * a.slab + i];
+        put_elem<F32>(a.out, base + i, gelu_tanh(v) * bf16_f(e[i]));
+    }
+}
+
 struct MixRows {
     const float* raw;   // [rows][ld] projections
     int64_t ld;
@@ -127,12 +164,37 @@ struct MixRows {
     int64_t k_row, v_row;
 };
 
-// element c of a head that starts at p, scaled by r and the norm weights w (NULL: none), rotated if c < rot_dims
-__device__ __forceinline__ float rotated(const float* p, const float* w, float r, int c, int rot_dims, const float* cs) {
-    const float v = w ? p[c] * r * w[c] : p[c];
-    if (c >= rot_dims) return v;
-    const float o = w ? p[c ^ 1] * r * w[c ^ 1] : p[c ^ 1], co = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
-    return (c & 1) ? v * co + o * sn : v * co - o * sn;
+// Elements c, c + 1 (c even) of a head of n values that starts at p, scaled by r and the norm weights w (NULL: none), rotated
+// if c < rot_dims; zero past n.
+__device__ __forceinline__ float2 rotated2(const float* p, const float* w, float r, int c, int n, int rot_dims, const float* cs) {
+    float2 v = make_float2(0.0f, 0.0f);
+    if (c >= n) return v;
+    v.x = w ? p[c] * r * w[c] : p[c];
+    if (c + 1 >= n) return v;
+    v.y = w ? p[c + 1] * r * w[c + 1] : p[c + 1];
+    if (c < rot_dims) {
+        const float2 t = *reinterpret_cast<const float2*>(cs + c);
+        v = make_float2(v.x * t.x - v.y * t.y, v.y * t.x + v.x * t.y);
+    }
+    return v;
+}
+template <bool F32>
+__device__ __forceinline__ void put2(void* p, int64_t i, float2 v) {
+    if constexpr (F32) *reinterpret_cast<float2*>(static_cast<float*>(p) + i) = v;
+    else *reinterpret_cast<uint32_t*>(static_cast<uint16_t*>(p) + i) = (uint32_t)f_bf16(v.x) | ((uint32_t)f_bf16(v.y) << 16);
+}
+__device__ __forceinline__ float sumsq256(const float* p, int n) {  // this thread's share
+    float s = 0.0f;
+    if (((n | (int)(reinterpret_cast<uintptr_t>(p) >> 2)) & 3) == 0) {
+#pragma unroll 4
+        for (int i = threadIdx.x; i < n / 4; i += 256) {
+            const float4 v = reinterpret_cast<const float4*>(p)[i];
+            s = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, s))));
+        }
+    } else {
+        for (int i = threadIdx.x; i < n; i += 256) s = fmaf(p[i], p[i], s);
+    }
+    return s;
 }
 
 // grid rows: q and k normed over the whole projection and rotated, k and v appended; heads padded to multiples of 8 with zeros
@@ -144,22 +206,23 @@ __global__ __launch_bounds__(256) void attention_prep_rows_kernel(const MixRows 
     const float *q = a.raw + blockIdx.x * a.ld, *k = q + a.heads * a.dim, *v = k + a.kv_heads * a.dim;
     const float* cs = a.rope + pos * a.rot_dims;
     const int nq = a.heads * a.dim, nk = a.kv_heads * a.dim, d8 = (a.dim + 7) & ~7, v8 = (a.vdim + 7) & ~7;
-    float sq = 0.0f, sk = 0.0f;
-    for (int i = tid; i < nq; i += 256) sq = fmaf(q[i], q[i], sq);
-    for (int i = tid; i < nk; i += 256) sk = fmaf(k[i], k[i], sk);
+    const float sq = sumsq256(q, nq), sk = sumsq256(k, nk);
     const float rq = 1.0f / sqrtf(block_sum<4>(sq, red) / (float)nq + a.eps);
     const float rk = 1.0f / sqrtf(block_sum<4>(sk, red) / (float)nk + a.eps);
-    for (int i = tid; i < a.heads * d8; i += 256) {
+#pragma unroll 4
+    for (int i = 2 * tid; i < a.heads * d8; i += 512) {
         const int h = i / d8, c = i % d8;
-        put_elem<Q32>(a.q, blockIdx.x * a.q_row + i, c < a.dim ? rotated(q + h * a.dim, a.q_norm + h * a.dim, rq, c, a.rot_dims, cs) : 0.0f);
+        put2<Q32>(a.q, blockIdx.x * a.q_row + i, rotated2(q + h * a.dim, a.q_norm + h * a.dim, rq, c, a.dim, a.rot_dims, cs));
     }
-    for (int i = tid; i < a.kv_heads * d8; i += 256) {
+#pragma unroll 2
+    for (int i = 2 * tid; i < a.kv_heads * d8; i += 512) {
         const int h = i / d8, c = i % d8;
-        put_elem<F32>(a.k, pos * a.k_row + i, c < a.dim ? rotated(k + h * a.dim, a.k_norm + h * a.dim, rk, c, a.rot_dims, cs) : 0.0f);
+        put2<F32>(a.k, pos * a.k_row + i, rotated2(k + h * a.dim, a.k_norm + h * a.dim, rk, c, a.dim, a.rot_dims, cs));
     }
-    for (int i = tid; i < a.kv_heads * v8; i += 256) {
+#pragma unroll 2
+    for (int i = 2 * tid; i < a.kv_heads * v8; i += 512) {
         const int h = i / v8, c = i % v8;
-        put_elem<F32>(a.v, pos * a.v_row + i, c < a.vdim ? v[h * a.vdim + c] : 0.0f);
+        put2<F32>(a.v, pos * a.v_row + i, rotated2(v + h * a.vdim, nullptr, 1.0f, c, a.vdim, 0, nullptr));
     }
 }
 
@@ -172,22 +235,16 @@ __global__ __launch_bounds__(256) void latent_prep_rows_kernel(const MixRows a) 
     const int qd = a.dim + a.rot_dim, d8 = (a.dim + 7) & ~7, r8 = (a.rot_dim + 7) & ~7, rank8 = (a.kv_rank + 7) & ~7;
     const float *q = a.raw + blockIdx.x * a.ld, *c = q + a.heads * qd, *kr = c + a.kv_rank;
     const float* cs = a.rope + pos * a.rot_dims;
-    float ss = 0.0f;
-    for (int i = tid; i < a.kv_rank; i += 256) ss = fmaf(c[i], c[i], ss);
-    const float r = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.kv_rank + a.eps);
-    for (int i = tid; i < rank8 + r8; i += 256) {
-        float v = 0.0f;
-        if (i < rank8) { if (i < a.kv_rank) v = c[i] * r * a.k_norm[i]; }
-        else if (i - rank8 < a.rot_dim) v = rotated(kr, nullptr, 1.0f, i - rank8, a.rot_dims, cs);
-        put_elem<F32>(a.k, pos * a.k_row + i, v);
-    }
-    for (int i = tid; i < a.heads * (d8 + r8); i += 256) {
+    const float r = 1.0f / sqrtf(block_sum<4>(sumsq256(c, a.kv_rank), red) / (float)a.kv_rank + a.eps);
+    for (int i = 2 * tid; i < rank8 + r8; i += 512)
+        put2<F32>(a.k, pos * a.k_row + i,
+                  i < rank8 ? rotated2(c, a.k_norm, r, i, a.kv_rank, 0, nullptr) : rotated2(kr, nullptr, 1.0f, i - rank8, a.rot_dim, a.rot_dims, cs));
+#pragma unroll 4
+    for (int i = 2 * tid; i < a.heads * (d8 + r8); i += 512) {
         const int h = i / (d8 + r8), e = i % (d8 + r8);
         const float* qh = q + h * qd;
-        float v = 0.0f;
-        if (e < d8) { if (e < a.dim) v = qh[e]; }
-        else if (e - d8 < a.rot_dim) v = rotated(qh + a.dim, nullptr, 1.0f, e - d8, a.rot_dims, cs);
-        put_elem<F32>(a.q, blockIdx.x * a.q_row + i, v);
+        put2<F32>(a.q, blockIdx.x * a.q_row + i,
+                  e < d8 ? rotated2(qh, nullptr, 1.0f, e, a.dim, 0, nullptr) : rotated2(qh + a.dim, nullptr, 1.0f, e - d8, a.rot_dim, a.rot_dims, cs));
     }
 }
 
@@ -218,7 +275,11 @@ struct BlockStack {
     float *r_x = nullptr, *r_emb = nullptr, *r_h = nullptr, *r_proj = nullptr;
     void *r_xn = nullptr, *r_q = nullptr, *r_attn = nullptr, *r_act = nullptr, *r_gate = nullptr, *r_kv = nullptr;
     const float *r_pend_h = nullptr, *r_pend_w = nullptr;
+    int r_slabs = 1;      // r_pend_h is the sum of that many slabs of a K-split product
+    int64_t r_h_room = 0; // floats behind r_h
 };
+
+constexpr int64_t SPLIT_ROOM = (int64_t)8 << 20;  // floats for K-split partial sums beyond one set of rows
 
 static int dev_alloc(BlockStack* b, size_t bytes, void** out) {
     int rc = hip_status(hipMalloc(out, bytes));
@@ -434,7 +495,7 @@ static int add_pending(BlockStack* b, hipStream_t s) {  // in place, for traced 
         if (rc != PTM_OK) return rc;
         b->x = b->xa;
     }
-    hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(1), dim3(256), 0, s, const_cast<float*>(b->x), b->pend_h, b->pend_w,
+    hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(1), dim3(256), 0, s, const_cast<float*>(b->x), b->pend_h, 1, (int64_t)0, b->pend_w,
                        (const float*)nullptr, (const float*)nullptr, (const float*)nullptr, (void*)nullptr, b->cfg.hidden, b->wp, b->cfg.eps);
     b->pend_h = b->pend_w = nullptr;
     return launch_status();
@@ -443,8 +504,8 @@ static int add_pending(BlockStack* b, hipStream_t s) {  // in place, for traced 
 int blocks_token(BlockStack* b, const int* d_token, const int64_t* d_past, float* trace, hipStream_t s) {
     const ptm_block_config& c = b->cfg;
     int rc;
-    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(1), dim3(256), 0, s, static_cast<const uint16_t*>(c.embedding.data),
-                       c.embedding.row_stride_bytes / 2, d_token, c.hidden, b->wp, b->emb, (float*)nullptr);
+    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(1, (b->wp + 511) / 512), dim3(128), 0, s, static_cast<const uint16_t*>(c.embedding.data),
+                       c.embedding.row_stride_bytes / 2, d_token, b->wp, b->emb, (float*)nullptr);
     PTM_TRY(launch_status());
     b->x = b->emb;
     b->pend_h = b->pend_w = nullptr;
@@ -504,7 +565,7 @@ int blocks_token(BlockStack* b, const int* d_token, const int64_t* d_past, float
         if (latent(L)) {
             const LatentStep ls{b->proj, L.k_norm, b->rope[(size_t)run.block], static_cast<const uint16_t*>(L.expand.data),
                                 L.expand.row_stride_bytes / 2, L.heads, L.dim, L.rot_dim, L.rot.dims, L.kv_rank, L.vdim, c.eps, d_past,
-                                b->q, run.k, b->f32};
+                                b->q, tiled, run.k, b->f32};
             PTM_TRY(latent_absorb(ls, s));
             if (tiled) {
                 PTM_TRY(decode_attention(d, s));
@@ -618,7 +679,7 @@ int blocks_reserve(BlockStack* b, int rows) {
     }
     size_t off = 0;
     auto take = [&](size_t bytes) { const size_t o = off; off += (bytes + 511) & ~(size_t)255; return o; };
-    const size_t o_tok = take(4 * R), o_x = take(4 * R * W), o_e = take(4 * R * W), o_h = take(4 * R * W), o_p = take(4 * R * proj),
+    const size_t o_tok = take(4 * R), o_x = take(4 * R * W), o_e = take(4 * R * W), o_h = take(4 * (R * W + (size_t)SPLIT_ROOM)), o_p = take(4 * R * proj),
                  o_xn = take(es * R * W), o_q = take(es * R * q), o_at = take(es * R * attn), o_ac = take(es * R * act),
                  o_g = take(es * R * (size_t)up64(c.side_dim > 0 ? c.side_dim : 1)), o_kv = take(es * kv);
     int rc = hip_status(hipMalloc(&b->slab, off));
@@ -631,6 +692,7 @@ int blocks_reserve(BlockStack* b, int rows) {
     b->r_emb = (float*)(p + o_e);
     b->r_h = (float*)(p + o_h);
     b->r_proj = (float*)(p + o_p);
+    b->r_h_room = (int64_t)(R * W) + SPLIT_ROOM;
     b->r_xn = p + o_xn;
     b->r_q = p + o_q;
     b->r_attn = p + o_at;
@@ -648,17 +710,20 @@ int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, floa
     int rc;
     if (M <= 0 || M > b->rows) return PTM_E_STATE;
     PTM_TRY(hip_status(hipMemcpyAsync(b->r_tokens, tokens_host, 4 * (size_t)M, hipMemcpyHostToDevice, s)));
-    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(M), dim3(256), 0, s, static_cast<const uint16_t*>(c.embedding.data),
-                       c.embedding.row_stride_bytes / 2, b->r_tokens, c.hidden, b->wp, b->r_x, b->r_emb);
+    hipLaunchKernelGGL(embed_bf16_rows_kernel, dim3(M, (b->wp + 511) / 512), dim3(128), 0, s, static_cast<const uint16_t*>(c.embedding.data),
+                       c.embedding.row_stride_bytes / 2, b->r_tokens, b->wp, b->r_x, b->r_emb);
     PTM_TRY(launch_status());
     b->r_pend_h = b->r_pend_w = nullptr;
+    b->r_slabs = 1;
+    const int64_t slab = (int64_t)M * b->wp;
     const float *add0 = nullptr, *add1 = nullptr;
     // the residual rows take in what is pending; their norm (or, gamma NULL, a copy) goes to r_xn unless `only_add`
     auto norm = [&](const float* gamma, bool only_add = false) {
         void* xn = only_add ? nullptr : b->r_xn;
-        if (f32) hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
-        else hipLaunchKernelGGL(residual_norm_rows_kernel<false>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
+        if (f32) hipLaunchKernelGGL(residual_norm_rows_kernel<true>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_slabs, slab, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
+        else hipLaunchKernelGGL(residual_norm_rows_kernel<false>, dim3(M), dim3(256), 0, s, b->r_x, b->r_pend_h, b->r_slabs, slab, b->r_pend_w, add0, add1, gamma, xn, c.hidden, b->wp, c.eps);
         b->r_pend_h = b->r_pend_w = add0 = add1 = nullptr;
+        b->r_slabs = 1;
         return launch_status();
     };
     auto product = [&](const ptm_qweight& w, const void* A, int64_t lda, int rows, int epilogue, void* C, int64_t ldc) {
@@ -679,7 +744,10 @@ int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, floa
     auto branch_out = [&](const ptm_qweight& w, const void* A, const float* post) {
         b->r_pend_h = b->r_h;
         b->r_pend_w = post;
-        return dense_gemm(product(w, A, up64(w.cols), M, GEMM_F32, b->r_h, b->wp), s);
+        DenseGemm g = product(w, A, up64(w.cols), M, GEMM_F32, b->r_h, b->wp);
+        g.slab = slab;
+        g.slab_room = b->r_h_room;
+        return dense_gemm(g, s, &b->r_slabs);
     };
     for (size_t ri = 0; ri < b->runs.size(); ++ri) {
         const LayerRun& run = b->runs[ri];
@@ -752,12 +820,17 @@ int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, floa
         }
         if (L.side_gate.data) {
             PTM_TRY(norm(nullptr));
-            DenseGemm g = product(L.side_gate, b->r_xn, b->wp, M, GEMM_SIDE, b->r_gate, up64(c.side_dim));
-            g.side = static_cast<const uint16_t*>(c.side_table.data);
-            g.side_ld = c.side_table.row_stride_bytes / 2;
-            g.side_off = L.side_offset;
-            g.tokens = b->r_tokens;
-            PTM_TRY(dense_gemm(g, s));
+            // few columns: the product is split over K, its sums (in r_h, consumed by the norm above) get the epilogue here
+            DenseGemm g = product(L.side_gate, b->r_xn, b->wp, M, GEMM_F32, b->r_h, up64(c.side_dim));
+            g.slab = (int64_t)M * g.ldc;
+            g.slab_room = b->r_h_room;
+            int slabs = 1;
+            PTM_TRY(dense_gemm(g, s, &slabs));
+            const SideRows sr{b->r_h, slabs, g.slab, g.ldc, static_cast<const uint16_t*>(c.side_table.data), c.side_table.row_stride_bytes / 2,
+                              L.side_offset, c.side_dim, b->r_tokens, b->r_gate};
+            if (f32) hipLaunchKernelGGL(side_rows_kernel<true>, dim3(M), dim3(256), 0, s, sr);
+            else hipLaunchKernelGGL(side_rows_kernel<false>, dim3(M), dim3(256), 0, s, sr);
+            PTM_TRY(launch_status());
             PTM_TRY(branch_out(L.side_proj, b->r_gate, L.side_norm));
         }
         if (trace) {
@@ -766,6 +839,7 @@ int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, floa
             PTM_TRY(launch_status());
         }
     }
+    if (b->r_slabs > 1 || c.hidden != b->wp) PTM_TRY(norm(nullptr, true));  // the head reads finished rows with clear padding
     return PTM_OK;
 }
 #undef PTM_TRY

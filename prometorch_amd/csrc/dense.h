@@ -80,7 +80,8 @@ struct LatentStep {
     int heads, dim, rot_dim, rot_dims, kv_rank, vdim;
     float eps;
     const int64_t* d_past;
-    float* q;                 // [heads][up8(kv_rank) + up8(rot_dim)]
+    void* q;                  // [heads][up8(kv_rank) + up8(rot_dim)]: fp32, or two bfloat16 planes of that (tiled attention)
+    int q_planes;
     void* cache;              // [max_seq][up8(kv_rank) + up8(rot_dim)]
     int fp32;
 };
@@ -90,7 +91,7 @@ int latent_out(const LatentStep& a, const float* pO, const float* pM, const floa
                hipStream_t s);
 
 // C = epilogue(A . W^T): GEMM_F32 fp32 C; otherwise element type of the rows (bfloat16, or fp32 when a_fp32)
-enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2, GEMM_SIDE = 3 };
+enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2 };
 struct DenseGemm {
     const void* A = nullptr;
     int a_fp32 = 0;
@@ -101,17 +102,17 @@ struct DenseGemm {
     int epilogue = GEMM_F32;
     void* C = nullptr;
     int64_t ldc = 0;
-    const uint16_t* side = nullptr;
-    int64_t side_ld = 0;
-    int side_off = 0;
-    const int* tokens = nullptr;
+    // K split over workgroups where the output has too few tiles (GEMM_F32 only): split z leaves its partial sums at
+    // C + z * slab; slab_room floats are available for all of them
+    int64_t slab = 0, slab_room = 0;
+    int splits = 1;  // set by dense_gemm
 };
-int dense_gemm(const DenseGemm& g, hipStream_t s);
+int dense_gemm(DenseGemm g, hipStream_t s, int* splits = nullptr);
 
 // Attention of one decode token, position *d_past.  bfloat16 caches with tile classes the matrix-core kernel has: splits
 // partial results (decode_attention_splits); otherwise one finished result.
 struct DecodeAttention {
-    ptm_attention_args a;      // rows 1; Q is fp32 [heads][dim1 + dim2] unless raw is given
+    ptm_attention_args a;      // rows 1; Q (unless raw is given): two bfloat16 planes [2][heads][dim1 + dim2] that add up to q
     const int64_t* d_past;
     int max_seq;
     // attention mixer: un-normed projections, finished in the prologue, and the rows appended to the caches

@@ -25,21 +25,14 @@ __device__ __forceinline__ float relu2(float v) { return v > 0.0f ? v * v : 0.0f
 
 // four consecutive columns n .. n + 3 of row m
 template <bool F32>
-__device__ __forceinline__ void store4(const DenseGemm& g, int m, int n, float v0, float v1, float v2, float v3) {
+__device__ __forceinline__ void store4(const DenseGemm& g, int split, int m, int n, float v0, float v1, float v2, float v3) {
     if (g.epilogue == GEMM_RELU2) {
         v0 = relu2(v0);
         v1 = relu2(v1);
         v2 = relu2(v2);
         v3 = relu2(v3);
-    } else if (g.epilogue == GEMM_SIDE) {
-        const uint16_t* e = g.side + (int64_t)g.tokens[m] * g.side_ld + g.side_off + n;
-        const int left = g.N - n - 1;
-        v0 = gelu_tanh(v0) * bf16_f(e[0]);
-        v1 = gelu_tanh(v1) * bf16_f(e[min(1, left)]);
-        v2 = gelu_tanh(v2) * bf16_f(e[min(2, left)]);
-        v3 = gelu_tanh(v3) * bf16_f(e[min(3, left)]);
     }
-    const int64_t at = (int64_t)m * g.ldc + n;
+    const int64_t at = (int64_t)m * g.ldc + n + split * g.slab;
     if (F32 || g.epilogue == GEMM_F32) {
         float* c = static_cast<float*>(g.C) + at;
         if (n + 3 < g.N && (g.ldc & 3) == 0) {
@@ -72,10 +65,11 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int j = lane & 31, kh = lane >> 5;
     int tm, tn;
-    tile_of(blockIdx.x, (g.M + BM - 1) / BM, (g.N + BN - 1) / BN, tm, tn);
+    const int tiles_m = (g.M + BM - 1) / BM, tiles_n = (g.N + BN - 1) / BN, split = blockIdx.x / (tiles_m * tiles_n);
+    tile_of(blockIdx.x - split * tiles_m * tiles_n, tiles_m, tiles_n, tm, tn);
     const int m0 = tm * BM, n0 = tn * BN;
     const int wm = (wave % (BM / WM)) * WM, wn = (wave / (BM / WM)) * WN;
-    const int steps = (g.K + 63) / 64;
+    const int all = (g.K + 63) / 64, steps = all * (split + 1) / g.splits, first = all * split / g.splits;
     const uint16_t* A = static_cast<const uint16_t*>(g.A);
     const int pr = tid >> 3, pp = tid & 7;  // row and piece of this thread's first staged piece; the others 32 rows on
     const u32x4* pa[PA];
@@ -113,10 +107,10 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
         for (int b = 0; b < TN; ++b)
 #pragma unroll
             for (int r = 0; r < 16; ++r) acc[a][b][r] = 0.0f;
-    fetch(0);
-    stage(0);
+    fetch(first);
+    stage(first & 1);
     __syncthreads();
-    for (int st = 0; st < steps; ++st) {
+    for (int st = first; st < steps; ++st) {
         const int buf = st & 1;
         fetch(st + 1 < steps ? st + 1 : st);
 #pragma unroll
@@ -144,7 +138,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const int n = n0 + wn + 32 * b + 8 * q + 4 * kh;
-                if (n < g.N) store4<false>(g, m, n, acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]);
+                if (n < g.N) store4<false>(g, split, m, n, acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]);
             }
     }
 }
@@ -183,26 +177,45 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const DenseGemm g) 
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
         const int n = n0 + wn + 8 * q + 4 * kh;
-        if (n < g.N) store4<true>(g, m, n, acc[4 * q], acc[4 * q + 1], acc[4 * q + 2], acc[4 * q + 3]);
+        if (n < g.N) store4<true>(g, 0, m, n, acc[4 * q], acc[4 * q + 1], acc[4 * q + 2], acc[4 * q + 3]);
     }
 }
 
-int dense_gemm(const DenseGemm& g, hipStream_t s) {
+int dense_gemm(DenseGemm g, hipStream_t s, int* splits) {
     if (!g.A || !g.W || !g.C) return PTM_E_NULL;
     const int kp = up64(g.K);
     if (g.M <= 0 || g.N <= 0 || g.K <= 0 || g.lda <= 0 || g.ldw < kp || g.ldc < g.N) return PTM_E_SHAPE;
     if (!aligned16(g.A) || !aligned16(g.W) || !aligned16(g.C) || (g.lda & 7) || (g.ldw & 7)) return PTM_E_ALIGN;
     auto tiles = [&](int bm, int bn) { return ((int64_t)g.M + bm - 1) / bm * ((g.N + bn - 1) / bn); };
-    if (tiles(32, 64) > 0x7fffffff) return PTM_E_UNSUPPORTED;
+    if (tiles(32, 64) * 16 > 0x7fffffff) return PTM_E_UNSUPPORTED;
+    // splits that bring `t` tiles to about `target` workgroups, each with at least four steps of K
+    auto split = [&](int64_t t, int64_t target) {
+        g.splits = 1;
+        if (!splits || g.slab <= 0) return;
+        int64_t n = (target + t / 2) / t;
+        if (n > kp / 256) n = kp / 256;
+        if (n > 16) n = 16;
+        while (n > 1 && n * g.slab > g.slab_room) --n;
+        g.splits = n > 1 ? (int)n : 1;
+    };
     if (g.a_fp32) {
+        g.splits = 1;
         hipLaunchKernelGGL(dense_gemm_f32_kernel, dim3((unsigned)tiles(64, 64)), dim3(256), 0, s, g);
-    } else if (tiles(128, 128) >= 192) {
-        hipLaunchKernelGGL((dense_gemm_kernel<128, 128, 64, 64>), dim3((unsigned)tiles(128, 128)), dim3(256), 0, s, g);
-    } else if (g.M > 32) {
-        hipLaunchKernelGGL((dense_gemm_kernel<64, 64, 32, 32>), dim3((unsigned)tiles(64, 64)), dim3(256), 0, s, g);
+    } else if (g.M <= 32) {
+        split(tiles(32, 128), 512);
+        hipLaunchKernelGGL((dense_gemm_kernel<32, 128, 32, 32>), dim3((unsigned)(tiles(32, 128) * g.splits)), dim3(256), 0, s, g);
+    } else if (g.M <= 64) {
+        split(tiles(64, 64), 512);
+        hipLaunchKernelGGL((dense_gemm_kernel<64, 64, 32, 32>), dim3((unsigned)(tiles(64, 64) * g.splits)), dim3(256), 0, s, g);
     } else {
-        hipLaunchKernelGGL((dense_gemm_kernel<32, 128, 32, 32>), dim3((unsigned)tiles(32, 128)), dim3(256), 0, s, g);
+        const int64_t t = tiles(128, 128);
+        if (t < 192) split(t, 384);
+        if (t * g.splits >= 128)
+            hipLaunchKernelGGL((dense_gemm_kernel<128, 128, 64, 64>), dim3((unsigned)(t * g.splits)), dim3(256), 0, s, g);
+        else
+            hipLaunchKernelGGL((dense_gemm_kernel<64, 64, 32, 32>), dim3((unsigned)(tiles(64, 64) * g.splits)), dim3(256), 0, s, g);
     }
+    if (splits) *splits = g.splits;
     return launch_status();
 }
 

@@ -290,36 +290,49 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const LatentStep a) 
     const int dim8 = (a.dim + 7) & ~7;
     const int lr = tid & 15, dg = tid >> 4, rr = r0 + lr * 8;
     const float* q = a.proj + (int64_t)h * qd;
+    const uint16_t* w = a.expand + ((int64_t)h * dim8) * a.ld + (rr < a.kv_rank ? rr : 0);
+    u32x4 wr[8];  // the first 128 rows, requested before q is staged
+#pragma unroll
+    for (int u = 0; u < 8; ++u) wr[u] = *reinterpret_cast<const u32x4*>(w + (int64_t)min(dg + 16 * u, a.dim - 1) * a.ld);
     for (int i = tid; i < a.dim; i += 256) s_q[i] = q[i];
     __syncthreads();
     float acc[8];
 #pragma unroll
     for (int i = 0; i < 8; ++i) acc[i] = 0.0f;
+    auto add = [&](const u32x4& v, float x) {
+        acc[0] = fmaf(bf16_lo(v.x), x, acc[0]);
+        acc[1] = fmaf(bf16_hi(v.x), x, acc[1]);
+        acc[2] = fmaf(bf16_lo(v.y), x, acc[2]);
+        acc[3] = fmaf(bf16_hi(v.y), x, acc[3]);
+        acc[4] = fmaf(bf16_lo(v.z), x, acc[4]);
+        acc[5] = fmaf(bf16_hi(v.z), x, acc[5]);
+        acc[6] = fmaf(bf16_lo(v.w), x, acc[6]);
+        acc[7] = fmaf(bf16_hi(v.w), x, acc[7]);
+    };
     if (rr < a.kv_rank) {
-        const uint16_t* w = a.expand + ((int64_t)h * dim8) * a.ld + rr;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) add(wr[u], dg + 16 * u < a.dim ? s_q[dg + 16 * u] : 0.0f);
 #pragma unroll 4
-        for (int d = dg; d < a.dim; d += 16) {
-            const uint4 v = *reinterpret_cast<const uint4*>(w + (int64_t)d * a.ld);
-            const float x = s_q[d];
-            acc[0] = fmaf(bf16_lo(v.x), x, acc[0]);
-            acc[1] = fmaf(bf16_hi(v.x), x, acc[1]);
-            acc[2] = fmaf(bf16_lo(v.y), x, acc[2]);
-            acc[3] = fmaf(bf16_hi(v.y), x, acc[3]);
-            acc[4] = fmaf(bf16_lo(v.z), x, acc[4]);
-            acc[5] = fmaf(bf16_hi(v.z), x, acc[5]);
-            acc[6] = fmaf(bf16_lo(v.w), x, acc[6]);
-            acc[7] = fmaf(bf16_hi(v.w), x, acc[7]);
-        }
+        for (int d = dg + 128; d < a.dim; d += 16) add(*reinterpret_cast<const u32x4*>(w + (int64_t)d * a.ld), s_q[d]);
     }
 #pragma unroll
     for (int i = 0; i < 8; ++i) s_sum[dg][lr * 8 + i] = acc[i];
     __syncthreads();
-    float* dst = a.q + (int64_t)h * row;
+    auto put_q = [&](int i, float v) {
+        const int64_t at = (int64_t)h * row + i;
+        if (a.q_planes) {
+            const uint16_t hi = f_bf16(v);
+            static_cast<uint16_t*>(a.q)[at] = hi;
+            static_cast<uint16_t*>(a.q)[(int64_t)a.heads * row + at] = f_bf16(v - bf16_f(hi));
+        } else {
+            static_cast<float*>(a.q)[at] = v;
+        }
+    };
     if (tid < 128 && r0 + tid < rank8) {
         float v = 0.0f;
 #pragma unroll
         for (int k = 0; k < 16; ++k) v += s_sum[k][tid];
-        dst[r0 + tid] = v;  // columns past kv_rank hold zero weights
+        put_q(r0 + tid, v);  // columns past kv_rank hold zero weights
     }
     if (r0 == 0)
         for (int i = tid; i < rot8; i += 256) {
@@ -331,7 +344,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const LatentStep a) 
                     v = (i & 1) ? v * c + o * sn : v * c - o * sn;
                 }
             }
-            dst[rank8 + i] = v;
+            put_q(rank8 + i, v);
         }
 }
 
@@ -344,7 +357,7 @@ int latent_absorb(const LatentStep& a, hipStream_t s) {
 }
 
 // grid (heads, ceil(vdim / 32)).  The head's split results are merged into its latent (LDS), which 32 rows of W_uv take to
-// the head's output.
+// the head's output: 8 rows per wave, their first 512 columns requested before the merge.
 constexpr int LO_MAX_SPLITS = 256;
 __global__ __launch_bounds__(256) void latent_out_kernel(const uint16_t* __restrict__ w_uv, int64_t ld, int heads, int kv_rank,
                                                          int vdim, const float* __restrict__ pO, const float* __restrict__ pM,
@@ -354,6 +367,15 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const uint16_t* __restr
     __shared__ float s_w[LO_MAX_SPLITS];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int h = blockIdx.x, v8 = (vdim + 7) & ~7, kp = (kv_rank + 63) & ~63;
+    const int v0 = blockIdx.y * 32 + wave * 8;
+    const uint16_t* w = w_uv + (int64_t)h * v8 * ld;
+    u32x4 wr[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+        wr[i] = u32x4{0, 0, 0, 0};
+        if (lane * 8 < kp) wr[i] = *reinterpret_cast<const u32x4*>(w + (int64_t)min(v0 + i, vdim - 1) * ld + lane * 8);
+    }
+    issue_order_fence();
     if (pM) {
         if (wave == 0) {
             float m = -INFINITY;
@@ -372,35 +394,47 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const uint16_t* __restr
         s_w[0] = 1.0f;
     }
     __syncthreads();
-    for (int r = tid; r < kp; r += 256) {
-        float v = 0.0f;
+    for (int r = tid * 2; r < kp; r += 512) {
+        float a0 = 0.0f, a1 = 0.0f;
         if (r < kv_rank) {
+            const float* p = pO + (int64_t)h * o_row + r;
 #pragma unroll 8
-            for (int i = 0; i < splits; ++i)  // a split without a visible key has weight 0 and a zero result
-                v = fmaf(pO[((int64_t)i * heads + h) * o_row + r], s_w[i], v);
+            for (int i = 0; i < splits; ++i) {  // a share without a visible key has weight 0
+                const float2 v = *reinterpret_cast<const float2*>(p + (int64_t)i * heads * o_row);
+                a0 = fmaf(v.x, s_w[i], a0);
+                a1 = fmaf(v.y, s_w[i], a1);
+            }
         }
-        s_c[r] = v;
+        s_c[r] = a0;
+        s_c[r + 1] = r + 1 < kv_rank ? a1 : 0.0f;
     }
     __syncthreads();
-    for (int i = wave; i < 32; i += 4) {
-        const int v = blockIdx.y * 32 + i;
-        if (v >= vdim) break;
-        const uint16_t* w = w_uv + ((int64_t)h * v8 + v) * ld;
-        float acc = 0.0f;
-        for (int k = lane * 8; k < kp; k += 512) {
-            const uint4 u = *reinterpret_cast<const uint4*>(w + k);
-            const float4 x0 = *reinterpret_cast<const float4*>(s_c + k), x1 = *reinterpret_cast<const float4*>(s_c + k + 4);
-            acc = fmaf(bf16_lo(u.x), x0.x, acc);
-            acc = fmaf(bf16_hi(u.x), x0.y, acc);
-            acc = fmaf(bf16_lo(u.y), x0.z, acc);
-            acc = fmaf(bf16_hi(u.y), x0.w, acc);
-            acc = fmaf(bf16_lo(u.z), x1.x, acc);
-            acc = fmaf(bf16_hi(u.z), x1.y, acc);
-            acc = fmaf(bf16_lo(u.w), x1.z, acc);
-            acc = fmaf(bf16_hi(u.w), x1.w, acc);
+    float acc[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[i] = 0.0f;
+    for (int k = lane * 8; k < kp; k += 512) {
+        if (k >= 512)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) wr[i] = *reinterpret_cast<const u32x4*>(w + (int64_t)min(v0 + i, vdim - 1) * ld + k);
+        const float4 x0 = *reinterpret_cast<const float4*>(s_c + k), x1 = *reinterpret_cast<const float4*>(s_c + k + 4);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            float t = acc[i];
+            t = fmaf(bf16_lo(wr[i].x), x0.x, t);
+            t = fmaf(bf16_hi(wr[i].x), x0.y, t);
+            t = fmaf(bf16_lo(wr[i].y), x0.z, t);
+            t = fmaf(bf16_hi(wr[i].y), x0.w, t);
+            t = fmaf(bf16_lo(wr[i].z), x1.x, t);
+            t = fmaf(bf16_hi(wr[i].z), x1.y, t);
+            t = fmaf(bf16_lo(wr[i].w), x1.z, t);
+            t = fmaf(bf16_hi(wr[i].w), x1.w, t);
+            acc[i] = t;
         }
-        acc = sum64(acc);
-        if (lane == 0) out[(int64_t)h * v8 + v] = acc;
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+        const float s = sum64(acc[i]);
+        if (lane == 0 && v0 + i < vdim) out[(int64_t)h * v8 + v0 + i] = s;
     }
 }
 

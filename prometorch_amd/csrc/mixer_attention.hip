@@ -127,7 +127,7 @@ static int rows_launch(const ptm_attention_args& a, const int64_t* d_past, hipSt
 // holds in its S^T accumulator, in that order.
 template <int DQ, int DV>
 __global__ __launch_bounds__(256, DQ <= 192 && DV <= 128 ? 2 : 1) void attention_mfma_kernel(const ptm_attention_args a) {
-    constexpr int KS = DQ / 16, DT = DV / 32, KP = DQ * 2 + 16, VP = DV * 2 + 64, PK = DQ / 32, PV = DV / 32;
+    constexpr int KS = DQ / 16, DT = DV / 32, KP = DQ * 2 + 16, VP = DV * 2 + 64;
     __shared__ __align__(16) uint8_t s_k[64 * KP];
     __shared__ __align__(16) uint8_t s_v[64 * VP];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane & 31, kh = lane >> 5;
@@ -166,57 +166,71 @@ __global__ __launch_bounds__(256, DQ <= 192 && DV <= 128 ? 2 : 1) void attention
     const int ntiles = nk + (int)(p_max / 64) - wt0 + 1;
     auto tile_at = [&](int i) { return i < nk ? i : wt0 + i - nk; };
 
-    // staged pieces of 16 bytes: row of the tile, source column; pieces past the key or value size are zeros
-    const uint16_t* kp[PK];
-    const uint16_t* vp[PV];
-    int64_t kstr[PK];
-    uint32_t lk[PK], lv[PV];
-    int kr[PK], vr[PV];
+    // A thread stages 16-byte pieces of rows tid / 8 and tid / 8 + 32, columns 8 (tid % 8) + 64 g; pieces past the key or value
+    // size are zeros.
+    constexpr int GK = DQ / 64, GV = DV / 64;
+    const int r0 = tid >> 3, c0 = (tid & 7) * 8;
+    const uint16_t* kp[GK];
+    const uint16_t* vp[GV];
+    uint32_t kstr[GK];
 #pragma unroll
-    for (int i = 0; i < PK; ++i) {
-        const int q = tid + 256 * i, r = q / (DQ / 8), c = (q % (DQ / 8)) * 8;
-        kr[i] = r;
-        lk[i] = r * KP + c * 2;
+    for (int i = 0; i < GK; ++i) {
+        const int c = c0 + 64 * i;
         kp[i] = c < a.dim1 ? static_cast<const uint16_t*>(a.K1) + (int64_t)g * a.k1_head + c
                            : c < dq ? static_cast<const uint16_t*>(a.K2) + (c - a.dim1) : nullptr;
-        kstr[i] = c < a.dim1 ? a.k1_row : a.k2_row;
+        kstr[i] = (uint32_t)(c < a.dim1 ? a.k1_row : a.k2_row);
     }
 #pragma unroll
-    for (int i = 0; i < PV; ++i) {
-        const int q = tid + 256 * i, r = q / (DV / 8), c = (q % (DV / 8)) * 8;
-        vr[i] = r;
-        lv[i] = r * VP + c * 2;
+    for (int i = 0; i < GV; ++i) {
+        const int c = c0 + 64 * i;
         vp[i] = c < a.vdim ? static_cast<const uint16_t*>(a.V) + (int64_t)g * a.v_head + c : nullptr;
     }
-    u32x4 kreg[PK], vreg[PV];
-    auto fetch = [&](int tile) {  // keys past the last visible one repeat it, keys before the array its first; both are masked
-        const int64_t k0 = (int64_t)tile * 64;
+    u32x4 kreg[2 * GK], vreg[2 * GV];
+    const int key_last = (int)(p_max - a.kv_pos0);
+    // keys past the last visible one repeat it, keys before the array its first; both are masked
+    auto key_of = [&](int tile, int r) {
+        const int key = (int)((int64_t)tile * 64 - a.kv_pos0) + r;
+        return (uint32_t)max(min(key, key_last), 0);
+    };
+    auto fetch_k = [&](int tile) {
 #pragma unroll
-        for (int i = 0; i < PK; ++i) {
-            int64_t key = k0 + kr[i];
-            key = (key < p_max ? key : p_max) - a.kv_pos0;
-            kreg[i] = u32x4{0, 0, 0, 0};
-            if (kp[i]) kreg[i] = *reinterpret_cast<const u32x4*>(kp[i] + (key > 0 ? key : 0) * kstr[i]);
+        for (int u = 0; u < 2; ++u) {
+            const uint32_t key = key_of(tile, r0 + 32 * u);
+#pragma unroll
+            for (int i = 0; i < GK; ++i) {
+                kreg[GK * u + i] = u32x4{0, 0, 0, 0};
+                if (kp[i]) kreg[GK * u + i] = *reinterpret_cast<const u32x4*>(kp[i] + (uint64_t)key * kstr[i]);
+            }
         }
+    };
+    auto fetch_v = [&](int tile) {
 #pragma unroll
-        for (int i = 0; i < PV; ++i) {
-            int64_t key = k0 + vr[i];
-            key = (key < p_max ? key : p_max) - a.kv_pos0;
-            vreg[i] = u32x4{0, 0, 0, 0};
-            if (vp[i]) vreg[i] = *reinterpret_cast<const u32x4*>(vp[i] + (key > 0 ? key : 0) * a.v_row);
+        for (int u = 0; u < 2; ++u) {
+            const uint32_t key = key_of(tile, r0 + 32 * u);
+#pragma unroll
+            for (int i = 0; i < GV; ++i) {
+                vreg[GV * u + i] = u32x4{0, 0, 0, 0};
+                if (vp[i]) vreg[GV * u + i] = *reinterpret_cast<const u32x4*>(vp[i] + (uint64_t)key * (uint32_t)a.v_row);
+            }
         }
     };
     const float sc2 = a.scale * LOG2E, inv_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
-    fetch(tile_at(0));
+    fetch_k(tile_at(0));
+    fetch_v(tile_at(0));
     for (int it = 0; it < ntiles; ++it) {
         const int64_t k0 = (int64_t)tile_at(it) * 64;
         __syncthreads();  // every wave has finished reading the previous tile
 #pragma unroll
-        for (int i = 0; i < PK; ++i) *reinterpret_cast<u32x4*>(s_k + lk[i]) = kreg[i];
+        for (int u = 0; u < 2; ++u) {
 #pragma unroll
-        for (int i = 0; i < PV; ++i) *reinterpret_cast<u32x4*>(s_v + lv[i]) = vreg[i];
+            for (int i = 0; i < GK; ++i) *reinterpret_cast<u32x4*>(s_k + (r0 + 32 * u) * KP + (c0 + 64 * i) * 2) = kreg[GK * u + i];
+#pragma unroll
+            for (int i = 0; i < GV; ++i) *reinterpret_cast<u32x4*>(s_v + (r0 + 32 * u) * VP + (c0 + 64 * i) * 2) = vreg[GV * u + i];
+        }
         __syncthreads();
-        if (it + 1 < ntiles) fetch(tile_at(it + 1));
+        const int next = tile_at(it + 1 < ntiles ? it + 1 : it);
+        fetch_k(next);
+        issue_order_fence();
         at_f16 sc[2];
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
@@ -228,6 +242,9 @@ __global__ __launch_bounds__(256, DQ <= 192 && DV <= 128 ? 2 : 1) void attention
                 sc[u] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka, qf[ks], sc[u], 0, 0, 0);
             }
         }
+        issue_order_fence();
+        fetch_v(next);
+        issue_order_fence();
         if (a.softcap > 0.0f) {
 #pragma unroll
             for (int u = 0; u < 2; ++u)
@@ -344,6 +361,7 @@ int attention_rows(const ptm_attention_args& a, const int64_t* d_past, bool q_fp
     const int dq = a.dim1 + a.dim2;
     if (a.fp32) return rows_launch<true, true>(a, d_past, s);
     if (q_fp32_out_fp32) return rows_launch<false, true>(a, d_past, s);
+    if (a.pos0 + a.rows > 0x7fffffff || ((a.k1_row | a.k2_row | a.v_row) >> 31)) return PTM_E_UNSUPPORTED;
     if (d_past || dq > 256 || a.vdim > 256) return rows_launch<false, false>(a, d_past, s);
     if (dq <= 64 && a.vdim <= 64) return mfma_launch<64, 64>(a, s);
     if (dq <= 128 && a.vdim <= 64) return mfma_launch<128, 64>(a, s);
@@ -355,12 +373,28 @@ int attention_rows(const ptm_attention_args& a, const int64_t* d_past, bool q_fp
 // ---- one decode token on the matrix cores ---------------------------------------------------------
 // v_mfma_f32_16x16x32_bf16: A: lane l holds row l % 16, summation indices 8 (l / 16) + 0..7; B: column l % 16 alike; C: column
 // l % 16, rows 4 (l / 16) + r.  v_mfma_f32_16x16x16_bf16: summation indices 4 (l / 16) + 0..3 - the layout S^T leaves P^T in.
-// RAW: q, k, v arrive un-normed; every workgroup norms and rotates its heads' q, the one that holds the newest position also the
-// key, takes it (and the value) from LDS and appends both rows to the caches.
+// RAW: q, k, v arrive un-normed; every workgroup norms and rotates its heads' q (behind the requests for its first keys and
+// values), the one that holds the newest position also the key, takes it (and the value) from LDS and appends both rows to the
+// caches.  Otherwise q is ready as two bfloat16 planes [2][heads][dim1 + dim2] and its fragments come straight from memory.
+__device__ __forceinline__ float sumsq_part(const float* p, int n) {  // this thread's share of 256
+    float s = 0.0f;
+    if (((n | (int)(reinterpret_cast<uintptr_t>(p) >> 2)) & 3) == 0) {
+#pragma unroll 4
+        for (int i = threadIdx.x; i < n / 4; i += 256) {
+            const float4 v = reinterpret_cast<const float4*>(p)[i];
+            s = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, s))));
+        }
+    } else {
+#pragma unroll 4
+        for (int i = threadIdx.x; i < n; i += 256) s = fmaf(p[i], p[i], s);
+    }
+    return s;
+}
+
 template <int DQ, int DV, bool RAW, bool V_IS_K>
 __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttention d, int splits) {
-    constexpr int KS = DQ / 32, DT = DV / 16, QP = DQ * 2 + 16, VP = DV * 2 + 32, PV = DV / 32;
-    __shared__ __align__(16) uint8_t s_q[2][16 * QP];
+    constexpr int KS = DQ / 32, DT = DV / 16, QP = DQ * 2 + 16, VP = DV * 2 + 32, PV = V_IS_K ? 1 : DV / 32;
+    __shared__ __align__(16) uint8_t s_q[2][RAW ? 16 * QP : 16];
     __shared__ __align__(16) uint8_t s_v[4][16 * VP];     // wave-private V rows; afterwards the waves' results
     __shared__ __align__(16) uint16_t s_newk[RAW ? DQ : 8], s_newv[RAW ? DV : 8];
     __shared__ float s_m[4][16], s_l[4][16], red[4];
@@ -373,91 +407,28 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
     const int64_t lo = a.window > 0 && past - a.window + 1 > 0 ? past - a.window + 1 : 0;
     const int wc0 = (int)(lo / 64), kc = (a.keep_first + 63) / 64, nk = a.window > 0 ? (kc < wc0 ? kc : wc0) : 0;
     const int total = nk + (int)(past / 64) - wc0 + 1;
-    const bool newest = (total - 1) % splits == split;  // this workgroup's share holds the newest position
-    if (RAW || split < total) {
-        float rq = 0.0f, rk = 0.0f;
-        const float *rawk = nullptr, *cs = nullptr;
-        if constexpr (RAW) {
-            const int nq = a.heads * d.dim, nkv = a.kv_heads * d.dim;
-            rawk = d.raw + nq;
-            cs = d.rope + past * d.rot_dims;
-            float ss = 0.0f, sk = 0.0f;
-            for (int i = tid; i < nq; i += 256) ss = fmaf(d.raw[i], d.raw[i], ss);
-            if (newest)
-                for (int i = tid; i < nkv; i += 256) sk = fmaf(rawk[i], rawk[i], sk);
-            rq = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)nq + d.eps);
-            if (newest) rk = 1.0f / sqrtf(block_sum<4>(sk, red) / (float)nkv + d.eps);
+    if (split >= total) {  // nothing to do: the merge gives this share weight 0
+        if (tid < nh) {
+            d.pM[(int64_t)split * a.heads + h0 + tid] = -INFINITY;
+            d.pL[(int64_t)split * a.heads + h0 + tid] = 0.0f;
         }
-        for (int i = tid; i < 16 * DQ; i += 256) {
-            const int h = i / DQ, c = i % DQ;
-            float v = 0.0f;
-            if constexpr (RAW) {
-                if (h < nh && c < d.dim) {
-                    const int at = (h0 + h) * d.dim + c;
-                    v = d.raw[at] * rq * d.q_norm[at];
-                    if (c < d.rot_dims) {
-                        const int at2 = (h0 + h) * d.dim + (c ^ 1);
-                        const float o = d.raw[at2] * rq * d.q_norm[at2], cc = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
-                        v = (c & 1) ? v * cc + o * sn : v * cc - o * sn;
-                    }
-                }
-            } else {
-                if (h < nh && c < dq) v = static_cast<const float*>(a.Q)[(int64_t)(h0 + h) * dq + c];
-            }
-            const short hi = bf_bits(v);
-            *reinterpret_cast<short*>(s_q[0] + h * QP + c * 2) = hi;
-            *reinterpret_cast<short*>(s_q[1] + h * QP + c * 2) = bf_bits(v - bf_val(hi));
-        }
-        if constexpr (RAW) {
-            if (newest) {
-                const float* rawv = rawk + a.kv_heads * d.dim + g * d.vdim_true;
-                const bool writer = blockIdx.y % tiles == 0;
-                for (int c = tid; c < DQ; c += 256) {
-                    float v = 0.0f;
-                    if (c < d.dim) {
-                        const int at = g * d.dim + c;
-                        v = rawk[at] * rk * d.k_norm[at];
-                        if (c < d.rot_dims) {
-                            const int at2 = g * d.dim + (c ^ 1);
-                            const float o = rawk[at2] * rk * d.k_norm[at2], cc = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
-                            v = (c & 1) ? v * cc + o * sn : v * cc - o * sn;
-                        }
-                    }
-                    const uint16_t b = f_bf16(v);
-                    s_newk[c] = b;
-                    if (writer && c < a.dim1) static_cast<uint16_t*>(d.k_cache)[past * a.k1_row + (int64_t)g * a.k1_head + c] = b;
-                }
-                for (int c = tid; c < DV; c += 256) {
-                    const uint16_t b = f_bf16(c < d.vdim_true ? rawv[c] : 0.0f);
-                    s_newv[c] = b;
-                    if (writer && c < a.vdim) static_cast<uint16_t*>(d.v_cache)[past * a.v_row + (int64_t)g * a.v_head + c] = b;
-                }
-            }
-        }
+        return;
     }
-    __syncthreads();
-    at_f4 acc[DT];
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt) acc[dt] = at_f4{0.f, 0.f, 0.f, 0.f};
-    float m_run = -INFINITY, l_run = 0.0f;
-    const float sc2 = a.scale * LOG2E, inv_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
-    uint8_t* sv = s_v[wave];
-    for (int c = split; c < total; c += splits) {
-        const int64_t k0 = (int64_t)(c < nk ? c : wc0 + c - nk) * 64 + 16 * wave;
-        if (k0 > past) continue;  // wave-uniform
+    const bool newest = (total - 1) % splits == split;  // this workgroup's share holds the newest position
+    u32x4 ka[KS], vv[PV];
+    const int ntrips = (total - split + splits - 1) / splits;
+    auto first_key = [&](int c) { return (int64_t)(c < nk ? c : wc0 + c - nk) * 64 + 16 * wave; };
+    auto fetch = [&](int64_t k0) {  // positions past the newest repeat it and are masked
         const int64_t kpos = k0 + j < past ? k0 + j : past;
         const uint16_t* k1 = static_cast<const uint16_t*>(a.K1) + kpos * a.k1_row + (int64_t)g * a.k1_head;
         const uint16_t* k2 = static_cast<const uint16_t*>(a.K2) + kpos * a.k2_row - a.dim1;
-        u32x4 ka[KS];
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
             const int col = 32 * ks + 8 * rg;
             ka[ks] = u32x4{0, 0, 0, 0};
-            if (col < a.dim1) ka[ks] = *reinterpret_cast<const u32x4*>(k1 + col);
-            else if (col < dq) ka[ks] = *reinterpret_cast<const u32x4*>(k2 + col);
+            if (col < dq) ka[ks] = *reinterpret_cast<const u32x4*>((col < a.dim1 ? k1 : k2) + col);
         }
         if constexpr (!V_IS_K) {
-            u32x4 vv[PV];
 #pragma unroll
             for (int i = 0; i < PV; ++i) {
                 const int q = lane + 64 * i, r = q / (DV / 8), col = (q % (DV / 8)) * 8;
@@ -465,6 +436,73 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
                 vv[i] = u32x4{0, 0, 0, 0};
                 if (col < a.vdim) vv[i] = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.V) + vpos * a.v_row + (int64_t)g * a.v_head + col);
             }
+        }
+    };
+    fetch(first_key(split));
+    if constexpr (RAW) {
+        const int nq = a.heads * d.dim, nkv = a.kv_heads * d.dim;
+        const float *rawk = d.raw + nq, *cs = d.rope + past * d.rot_dims;
+        auto turned = [&](const float* p, const float* w, float r, int c) {
+            const float v = p[c] * r * w[c];
+            if (c >= d.rot_dims) return v;
+            const float o = p[c ^ 1] * r * w[c ^ 1], co = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
+            return (c & 1) ? v * co + o * sn : v * co - o * sn;
+        };
+        const float pq = sumsq_part(d.raw, nq), pk = newest ? sumsq_part(rawk, nkv) : 0.0f;
+        const float rq = 1.0f / sqrtf(block_sum<4>(pq, red) / (float)nq + d.eps);
+#pragma unroll 2
+        for (int i = tid; i < nh * DQ; i += 256) {
+            const int h = i / DQ, c = i % DQ;
+            const float v = c < d.dim ? turned(d.raw + (h0 + h) * d.dim, d.q_norm + (h0 + h) * d.dim, rq, c) : 0.0f;
+            const short hi = bf_bits(v);
+            *reinterpret_cast<short*>(s_q[0] + h * QP + c * 2) = hi;
+            *reinterpret_cast<short*>(s_q[1] + h * QP + c * 2) = bf_bits(v - bf_val(hi));
+        }
+        for (int i = tid; i < (16 - nh) * (DQ / 2); i += 256) {  // columns without a head
+            const int h = nh + i / (DQ / 2), c = i % (DQ / 2);
+            *reinterpret_cast<uint32_t*>(s_q[0] + h * QP + c * 4) = 0;
+            *reinterpret_cast<uint32_t*>(s_q[1] + h * QP + c * 4) = 0;
+        }
+        if (newest) {
+            const float rk = 1.0f / sqrtf(block_sum<4>(pk, red) / (float)nkv + d.eps);
+            const float* rawv = rawk + nkv + g * d.vdim_true;
+            const bool writer = blockIdx.y % tiles == 0;
+            for (int c = tid; c < DQ; c += 256) {
+                const uint16_t b = f_bf16(c < d.dim ? turned(rawk + g * d.dim, d.k_norm + g * d.dim, rk, c) : 0.0f);
+                s_newk[c] = b;
+                if (writer && c < a.dim1) static_cast<uint16_t*>(d.k_cache)[past * a.k1_row + (int64_t)g * a.k1_head + c] = b;
+            }
+            for (int c = tid; c < DV; c += 256) {
+                const uint16_t b = f_bf16(c < d.vdim_true ? rawv[c] : 0.0f);
+                s_newv[c] = b;
+                if (writer && c < a.vdim) static_cast<uint16_t*>(d.v_cache)[past * a.v_row + (int64_t)g * a.v_head + c] = b;
+            }
+        }
+        __syncthreads();
+    }
+    // the fragment of q's plane t for columns 32 ks + 8 rg .. of head j (columns past the key size meet zero keys)
+    const uint16_t* qp = static_cast<const uint16_t*>(a.Q) + (int64_t)(h0 + (j < nh ? j : nh - 1)) * dq;
+    auto q_frag = [&](int t, int ks) {
+        if constexpr (RAW) {
+            return *reinterpret_cast<const at_b8*>(s_q[t] + j * QP + (32 * ks + 8 * rg) * 2);
+        } else {
+            const int col = 32 * ks + 8 * rg;
+            return *reinterpret_cast<const at_b8*>(qp + (int64_t)t * a.heads * dq + (col < dq ? col : 0));
+        }
+    };
+    at_f4 acc[DT];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) acc[dt] = at_f4{0.f, 0.f, 0.f, 0.f};
+    float m_run = -INFINITY, l_run = 0.0f;
+    const float sc2 = a.scale * LOG2E, inv_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
+    uint8_t* sv = s_v[wave];
+    for (int trip = 0; trip < ntrips; ++trip) {
+        const int64_t k0 = first_key(split + trip * splits);
+        if (trip > 0) fetch(k0);
+        if constexpr (V_IS_K) {
+#pragma unroll
+            for (int ks = 0; ks < DV / 32; ++ks) *reinterpret_cast<u32x4*>(sv + j * VP + (32 * ks + 8 * rg) * 2) = ka[ks];
+        } else {
 #pragma unroll
             for (int i = 0; i < PV; ++i) {
                 const int q = lane + 64 * i, r = q / (DV / 8), col = (q % (DV / 8)) * 8;
@@ -475,23 +513,17 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
             }
         }
         if constexpr (RAW) {
-            if (kpos == past) {
+            if (k0 + j >= past) {
 #pragma unroll
                 for (int ks = 0; ks < KS; ++ks) ka[ks] = *reinterpret_cast<const u32x4*>(s_newk + 32 * ks + 8 * rg);
             }
-        }
-        if constexpr (V_IS_K) {
-#pragma unroll
-            for (int ks = 0; ks < DV / 32; ++ks) *reinterpret_cast<u32x4*>(sv + j * VP + (32 * ks + 8 * rg) * 2) = ka[ks];
         }
         at_f4 s1 = {0.f, 0.f, 0.f, 0.f}, s2 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
             const at_b8 k8 = __builtin_bit_cast(at_b8, ka[ks]);
-            const at_b8 qh = *reinterpret_cast<const at_b8*>(s_q[0] + j * QP + (32 * ks + 8 * rg) * 2);
-            const at_b8 ql = *reinterpret_cast<const at_b8*>(s_q[1] + j * QP + (32 * ks + 8 * rg) * 2);
-            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8, qh, s1, 0, 0, 0);
-            s2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8, ql, s2, 0, 0, 0);
+            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8, q_frag(0, ks), s1, 0, 0, 0);
+            s2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k8, q_frag(1, ks), s2, 0, 0, 0);
         }
         float sc[4], mx = -INFINITY;
 #pragma unroll
@@ -518,10 +550,13 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
         m_run = m_new;
         __builtin_amdgcn_wave_barrier();
         issue_order_fence();
+        if (trip > 0) {
+#pragma unroll
+            for (int dt = 0; dt < DT; ++dt) acc[dt] *= corr;
+        }
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) {
             const at_s4 v = lds_tr16(sv + (4 * rg + (j >> 2)) * VP + (16 * dt + 4 * (j & 3)) * 2);
-            acc[dt] *= corr;
             acc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(v, ph, acc[dt], 0, 0, 0);
             acc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(v, pl, acc[dt], 0, 0, 0);
         }
@@ -544,7 +579,8 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
     const float f = __builtin_amdgcn_exp2f(m_run - ms);
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc[dt] *= f;
-    // waves 2, 3 hand their sums to waves 0, 1, then wave 1 to wave 0
+    // Every wave sums a quarter of the value dimensions over the four waves: first waves 2, 3 hand over the tiles of waves 0, 1,
+    // then each pair exchanges halves.  Two waves' results fit the memory of the V rows.
     at_f4* s_o = reinterpret_cast<at_f4*>(s_v);
     static_assert(sizeof(s_v) >= sizeof(at_f4) * 2 * DT * 64, "two waves' results fit the V rows");
     if (wave >= 2)
@@ -555,23 +591,20 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) acc[dt] += s_o[(wave * DT + dt) * 64 + lane];
     __syncthreads();
-    if (wave == 1)
+    if (wave < 2)
 #pragma unroll
-        for (int dt = 0; dt < DT; ++dt) s_o[dt * 64 + lane] = acc[dt];
+        for (int dt = 0; dt < DT; ++dt) s_o[(wave * DT + dt) * 64 + lane] = acc[dt];
     __syncthreads();
-    if (wave != 0 || j >= nh) return;
-    const int64_t ph = (int64_t)split * a.heads + h0 + j;
-    if (rg == 0) {
-        d.pM[ph] = m_all * (1.0f / LOG2E);
-        d.pL[ph] = l_all;
+    if (j >= nh) return;
+    const int64_t at = (int64_t)split * a.heads + h0 + j;
+    if (wave == 0 && rg == 0) {
+        d.pM[at] = m_all * (1.0f / LOG2E);
+        d.pL[at] = l_all;
     }
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-        const int col = 16 * dt + 4 * rg;
-        if (col < a.vdim) {
-            const at_f4 v = acc[dt] + s_o[dt * 64 + lane];
-            *reinterpret_cast<at_f4*>(d.pO + ph * a.vdim + col) = v;
-        }
+    for (int i = 0; i < DT / 4; ++i) {
+        const int dt = wave * (DT / 4) + i, col = 16 * dt + 4 * rg;
+        if (col < a.vdim) *reinterpret_cast<at_f4*>(d.pO + at * a.vdim + col) = s_o[dt * 64 + lane] + s_o[(DT + dt) * 64 + lane];
     }
 }
 
