@@ -376,30 +376,54 @@ __global__ __launch_bounds__(256) void latent_out_kernel(const uint16_t* __restr
         if (lane * 8 < kp) wr[i] = *reinterpret_cast<const u32x4*>(w + (int64_t)min(v0 + i, vdim - 1) * ld + lane * 8);
     }
     issue_order_fence();
+    // the first 512 latent values of up to 24 splits are requested before the weights are known
+    float2 pre[24];
+    {
+        const float* p = pO + (int64_t)h * o_row + min(tid * 2, o_row - 2);
+#pragma unroll
+        for (int i = 0; i < 24; ++i) pre[i] = *reinterpret_cast<const float2*>(p + (int64_t)min(i, splits - 1) * heads * o_row);
+    }
+    issue_order_fence();
     if (pM) {
         if (wave == 0) {
-            float m = -INFINITY;
-            for (int i = lane; i < splits; i += 64) m = fmaxf(m, pM[(int64_t)i * heads + h]);
+            float mv[LO_MAX_SPLITS / 64], lv[LO_MAX_SPLITS / 64], m = -INFINITY;
+#pragma unroll
+            for (int u = 0; u < LO_MAX_SPLITS / 64; ++u) {
+                const int i = min(lane + 64 * u, splits - 1);
+                mv[u] = lane + 64 * u < splits ? pM[(int64_t)i * heads + h] : -INFINITY;
+                lv[u] = pL[(int64_t)i * heads + h];
+                m = fmaxf(m, mv[u]);
+            }
             m = max64(m);
             float l = 0.0f;
-            for (int i = lane; i < splits; i += 64) {
-                const float e = expf(pM[(int64_t)i * heads + h] - m);
-                s_w[i] = e;
-                l = fmaf(pL[(int64_t)i * heads + h], e, l);
+#pragma unroll
+            for (int u = 0; u < LO_MAX_SPLITS / 64; ++u) {
+                mv[u] = expf(mv[u] - m);
+                l = fmaf(lv[u], mv[u], l);
             }
             l = 1.0f / sum64(l);
-            for (int i = lane; i < splits; i += 64) s_w[i] *= l;
+#pragma unroll
+            for (int u = 0; u < LO_MAX_SPLITS / 64; ++u) s_w[lane + 64 * u] = mv[u] * l;  // 0 past the last split
         }
-    } else if (tid == 0) {
-        s_w[0] = 1.0f;
+    } else if (tid < 64) {
+        s_w[tid] = tid == 0 ? 1.0f : 0.0f;
     }
     __syncthreads();
     for (int r = tid * 2; r < kp; r += 512) {
         float a0 = 0.0f, a1 = 0.0f;
         if (r < kv_rank) {
             const float* p = pO + (int64_t)h * o_row + r;
+            int i = 0;
+            if (r < 512) {
+#pragma unroll
+                for (int k = 0; k < 24; ++k) {
+                    a0 = fmaf(pre[k].x, s_w[k], a0);
+                    a1 = fmaf(pre[k].y, s_w[k], a1);
+                }
+                i = 24;
+            }
 #pragma unroll 8
-            for (int i = 0; i < splits; ++i) {  // a share without a visible key has weight 0
+            for (; i < splits; ++i) {  // a share without a visible key has weight 0
                 const float2 v = *reinterpret_cast<const float2*>(p + (int64_t)i * heads * o_row);
                 a0 = fmaf(v.x, s_w[i], a0);
                 a1 = fmaf(v.y, s_w[i], a1);

@@ -372,7 +372,10 @@ int attention_rows(const ptm_attention_args& a, const int64_t* d_past, bool q_fp
 
 // ---- one decode token on the matrix cores ---------------------------------------------------------
 // v_mfma_f32_16x16x32_bf16: A: lane l holds row l % 16, summation indices 8 (l / 16) + 0..7; B: column l % 16 alike; C: column
-// l % 16, rows 4 (l / 16) + r.  v_mfma_f32_16x16x16_bf16: summation indices 4 (l / 16) + 0..3 - the layout S^T leaves P^T in.
+// l % 16, rows 4 (l / 16) + r.  A wave scores 16 of a chunk's 64 positions (S^T = K . Q^T); the weights, in the layout the
+// scores were left in, go to all waves through LDS and each sums a quarter of the value dimensions over the whole chunk
+// (O^T = V^T . P^T): two tiles of 16 positions make the 32 summation indices, each lane's eight being the positions
+// 4 (l / 16) + 0..3 of either tile.
 // RAW: q, k, v arrive un-normed; every workgroup norms and rotates its heads' q (behind the requests for its first keys and
 // values), the one that holds the newest position also the key, takes it (and the value) from LDS and appends both rows to the
 // caches.  Otherwise q is ready as two bfloat16 planes [2][heads][dim1 + dim2] and its fragments come straight from memory.
@@ -393,9 +396,10 @@ __device__ __forceinline__ float sumsq_part(const float* p, int n) {  // this th
 
 template <int DQ, int DV, bool RAW, bool V_IS_K>
 __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttention d, int splits) {
-    constexpr int KS = DQ / 32, DT = DV / 16, QP = DQ * 2 + 16, VP = DV * 2 + 32, PV = V_IS_K ? 1 : DV / 32;
+    constexpr int KS = DQ / 32, DW = DV / 64, QP = DQ * 2 + 16, VP = DV * 2 + 32, PV = V_IS_K ? 1 : DV / 32;
     __shared__ __align__(16) uint8_t s_q[2][RAW ? 16 * QP : 16];
-    __shared__ __align__(16) uint8_t s_v[4][16 * VP];     // wave-private V rows; afterwards the waves' results
+    __shared__ __align__(16) uint8_t s_v[64 * VP];
+    __shared__ __align__(16) at_s4 s_p[2][4][64];
     __shared__ __align__(16) uint16_t s_newk[RAW ? DQ : 8], s_newv[RAW ? DV : 8];
     __shared__ float s_m[4][16], s_l[4][16], red[4];
     const ptm_attention_args& a = d.a;
@@ -490,15 +494,18 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
             return *reinterpret_cast<const at_b8*>(qp + (int64_t)t * a.heads * dq + (col < dq ? col : 0));
         }
     };
-    at_f4 acc[DT];
+    at_f4 acc[DW];
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) acc[dt] = at_f4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < DW; ++i) acc[i] = at_f4{0.f, 0.f, 0.f, 0.f};
     float m_run = -INFINITY, l_run = 0.0f;
     const float sc2 = a.scale * LOG2E, inv_cap = a.softcap > 0.0f ? 1.0f / a.softcap : 0.0f;
-    uint8_t* sv = s_v[wave];
+    uint8_t* sv = s_v + 16 * wave * VP;
     for (int trip = 0; trip < ntrips; ++trip) {
         const int64_t k0 = first_key(split + trip * splits);
-        if (trip > 0) fetch(k0);
+        if (trip > 0) {
+            fetch(k0);
+            __syncthreads();  // every wave has finished with the previous chunk's values and weights
+        }
         if constexpr (V_IS_K) {
 #pragma unroll
             for (int ks = 0; ks < DV / 32; ++ks) *reinterpret_cast<u32x4*>(sv + j * VP + (32 * ks + 8 * rg) * 2) = ka[ks];
@@ -535,7 +542,10 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
         }
         mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
         mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-        const float m_new = fmaxf(m_run, mx), ms = m_new == -INFINITY ? 0.0f : m_new;
+        if (rg == 0) s_m[wave][j] = mx;
+        __syncthreads();
+        const float m_new = fmaxf(m_run, fmaxf(fmaxf(s_m[0][j], s_m[1][j]), fmaxf(s_m[2][j], s_m[3][j])));
+        const float ms = m_new == -INFINITY ? 0.0f : m_new;
         const float corr = __builtin_amdgcn_exp2f(m_run - ms);
         at_s4 ph, pl;
         float psum = 0.0f;
@@ -546,108 +556,88 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
             ph[r] = bf_bits(p);
             pl[r] = bf_bits(p - bf_val(ph[r]));
         }
-        l_run = fmaf(l_run, corr, psum);  // this lane's positions; the four lane groups are added at the end
+        s_p[0][wave][lane] = ph;
+        s_p[1][wave][lane] = pl;
+        l_run = fmaf(l_run, corr, psum);  // this lane's positions; lane groups and waves are added at the end
         m_run = m_new;
-        __builtin_amdgcn_wave_barrier();
-        issue_order_fence();
+        __syncthreads();
         if (trip > 0) {
 #pragma unroll
-            for (int dt = 0; dt < DT; ++dt) acc[dt] *= corr;
+            for (int i = 0; i < DW; ++i) acc[i] *= corr;
         }
+        typedef short s8 __attribute__((ext_vector_type(8)));
+        auto join = [](at_s4 x, at_s4 y) { return __builtin_bit_cast(at_b8, (s8){x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]}); };
 #pragma unroll
-        for (int dt = 0; dt < DT; ++dt) {
-            const at_s4 v = lds_tr16(sv + (4 * rg + (j >> 2)) * VP + (16 * dt + 4 * (j & 3)) * 2);
-            acc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(v, ph, acc[dt], 0, 0, 0);
-            acc[dt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(v, pl, acc[dt], 0, 0, 0);
+        for (int t = 0; t < 4; t += 2) {
+            const at_b8 hi = join(s_p[0][t][lane], s_p[0][t + 1][lane]), lw = join(s_p[1][t][lane], s_p[1][t + 1][lane]);
+#pragma unroll
+            for (int i = 0; i < DW; ++i) {
+                const uint8_t* vrow = s_v + (16 * t + 4 * rg + (j >> 2)) * VP + (16 * (wave * DW + i) + 4 * (j & 3)) * 2;
+                const at_b8 v = join(lds_tr16(vrow), lds_tr16(vrow + 16 * VP));
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, hi, acc[i], 0, 0, 0);
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, lw, acc[i], 0, 0, 0);
+            }
         }
-        issue_order_fence();
-        __builtin_amdgcn_wave_barrier();
     }
     l_run += __shfl_xor(l_run, 16, 64);
     l_run += __shfl_xor(l_run, 32, 64);
-    if (rg == 0) {
-        s_m[wave][j] = m_run;
-        s_l[wave][j] = l_run;
-    }
-    __syncthreads();  // also: every wave has finished with its V rows
-    float m_all = -INFINITY, l_all = 0.0f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) m_all = fmaxf(m_all, s_m[w][j]);
-    const float ms = m_all == -INFINITY ? 0.0f : m_all;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) l_all = fmaf(s_l[w][j], __builtin_amdgcn_exp2f(s_m[w][j] - ms), l_all);
-    const float f = __builtin_amdgcn_exp2f(m_run - ms);
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt) acc[dt] *= f;
-    // Every wave sums a quarter of the value dimensions over the four waves: first waves 2, 3 hand over the tiles of waves 0, 1,
-    // then each pair exchanges halves.  Two waves' results fit the memory of the V rows.
-    at_f4* s_o = reinterpret_cast<at_f4*>(s_v);
-    static_assert(sizeof(s_v) >= sizeof(at_f4) * 2 * DT * 64, "two waves' results fit the V rows");
-    if (wave >= 2)
-#pragma unroll
-        for (int dt = 0; dt < DT; ++dt) s_o[((wave - 2) * DT + dt) * 64 + lane] = acc[dt];
-    __syncthreads();
-    if (wave < 2)
-#pragma unroll
-        for (int dt = 0; dt < DT; ++dt) acc[dt] += s_o[(wave * DT + dt) * 64 + lane];
-    __syncthreads();
-    if (wave < 2)
-#pragma unroll
-        for (int dt = 0; dt < DT; ++dt) s_o[(wave * DT + dt) * 64 + lane] = acc[dt];
+    if (rg == 0) s_l[wave][j] = l_run;
     __syncthreads();
     if (j >= nh) return;
     const int64_t at = (int64_t)split * a.heads + h0 + j;
     if (wave == 0 && rg == 0) {
-        d.pM[at] = m_all * (1.0f / LOG2E);
-        d.pL[at] = l_all;
+        d.pM[at] = m_run * (1.0f / LOG2E);
+        d.pL[at] = (s_l[0][j] + s_l[1][j]) + (s_l[2][j] + s_l[3][j]);
     }
 #pragma unroll
-    for (int i = 0; i < DT / 4; ++i) {
-        const int dt = wave * (DT / 4) + i, col = 16 * dt + 4 * rg;
-        if (col < a.vdim) *reinterpret_cast<at_f4*>(d.pO + at * a.vdim + col) = s_o[dt * 64 + lane] + s_o[(DT + dt) * 64 + lane];
+    for (int i = 0; i < DW; ++i) {
+        const int col = 16 * (wave * DW + i) + 4 * rg;
+        if (col < a.vdim) *reinterpret_cast<at_f4*>(d.pO + at * a.vdim + col) = acc[i];
     }
 }
 
-// grid heads: out[h][v] = sum over the splits of their results, weighted by exp(m - max) / total
-__global__ __launch_bounds__(128) void decode_merge_kernel(const float* __restrict__ pO, const float* __restrict__ pM,
+// grid (heads, ceil(vdim / 64)): out[h][v] = sum over the splits of their results, weighted by exp(m - max) / total.  Four
+// waves take every fourth split of 64 values; the results are requested before the weights are known.
+__global__ __launch_bounds__(256) void decode_merge_kernel(const float* __restrict__ pO, const float* __restrict__ pM,
                                                            const float* __restrict__ pL, int splits, int heads, int vdim,
                                                            float* __restrict__ out) {
-    __shared__ float s_w[256];
-    const int tid = threadIdx.x, lane = tid & 63, h = blockIdx.x;
-    if (tid < 64) {
-        float mv[4], lv[4], m = -INFINITY;
+    __shared__ float s_sum[4][64];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.x, v = blockIdx.y * 64 + lane, vc = min(v, vdim - 1);
+    float o[16], mv[4], lv[4], m = -INFINITY;
 #pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            const int i = min(lane + 64 * u, splits - 1);
-            mv[u] = lane + 64 * u < splits ? pM[(int64_t)i * heads + h] : -INFINITY;
-            lv[u] = pL[(int64_t)i * heads + h];
-            m = fmaxf(m, mv[u]);
-        }
-        m = max64(m);
-        float l = 0.0f;
+    for (int u = 0; u < 16; ++u) o[u] = pO[((int64_t)min(wave + 4 * u, splits - 1) * heads + h) * vdim + vc];
 #pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            mv[u] = expf(mv[u] - m);
-            l = fmaf(lv[u], mv[u], l);
-        }
-        l = 1.0f / sum64(l);
-#pragma unroll
-        for (int u = 0; u < 4; ++u)
-            if (lane + 64 * u < splits) s_w[lane + 64 * u] = mv[u] * l;
+    for (int u = 0; u < 4; ++u) {
+        const int i = min(lane + 64 * u, splits - 1);
+        mv[u] = lane + 64 * u < splits ? pM[(int64_t)i * heads + h] : -INFINITY;
+        lv[u] = pL[(int64_t)i * heads + h];
+        m = fmaxf(m, mv[u]);
     }
+    m = max64(m);
+    float l = 0.0f;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+        mv[u] = expf(mv[u] - m);  // lane + 64 u: split's weight, 0 past the last
+        l = fmaf(lv[u], mv[u], l);
+    }
+    l = 1.0f / sum64(l);
+    auto weight = [&](int i) {
+        const float w = i < 64 ? mv[0] : i < 128 ? mv[1] : i < 192 ? mv[2] : mv[3];  // wave-uniform i
+        return __shfl(w, i & 63, 64);
+    };
+    float acc = 0.0f;
+#pragma unroll
+    for (int u = 0; u < 16; ++u) acc = fmaf(o[u], weight(wave + 4 * u), acc);
+    for (int i = wave + 64; i < splits; i += 4) acc = fmaf(pO[((int64_t)i * heads + h) * vdim + vc], weight(i), acc);
+    s_sum[wave][lane] = acc * l;
     __syncthreads();
-    for (int v = tid; v < vdim; v += 128) {
-        float acc = 0.0f;
-#pragma unroll 8
-        for (int i = 0; i < splits; ++i) acc = fmaf(pO[((int64_t)i * heads + h) * vdim + v], s_w[i], acc);
-        out[(int64_t)h * vdim + v] = acc;
-    }
+    if (wave == 0 && v < vdim) out[(int64_t)h * vdim + v] = (s_sum[0][lane] + s_sum[1][lane]) + (s_sum[2][lane] + s_sum[3][lane]);
 }
 
 int decode_attention_merge(const float* pO, const float* pM, const float* pL, int splits, int heads, int vdim, float* out,
                            hipStream_t s) {
     if (splits <= 0 || splits > 256) return PTM_E_UNSUPPORTED;
-    hipLaunchKernelGGL(decode_merge_kernel, dim3(heads), dim3(128), 0, s, pO, pM, pL, splits, heads, vdim, out);
+    hipLaunchKernelGGL(decode_merge_kernel, dim3(heads, (vdim + 63) / 64), dim3(256), 0, s, pO, pM, pL, splits, heads, vdim, out);
     return launch_status();
 }
 
