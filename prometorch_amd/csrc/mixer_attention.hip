@@ -378,7 +378,7 @@ int attention_rows(const ptm_attention_args& a, const int64_t* d_past, bool q_fp
 // 4 (l / 16) + 0..3 of either tile.
 // RAW: q, k, v arrive un-normed; every workgroup norms and rotates its heads' q (behind the requests for its first keys and
 // values), the one that holds the newest position also the key, takes it (and the value) from LDS and appends both rows to the
-// caches.  Otherwise q is ready as two bfloat16 planes [2][heads][dim1 + dim2] and its fragments come straight from memory.
+// caches.  Otherwise q is ready as two bfloat16 planes [2][heads][dim1 + dim2].
 __device__ __forceinline__ float sumsq_part(const float* p, int n) {  // this thread's share of 256
     float s = 0.0f;
     if (((n | (int)(reinterpret_cast<uintptr_t>(p) >> 2)) & 3) == 0) {
@@ -397,7 +397,7 @@ __device__ __forceinline__ float sumsq_part(const float* p, int n) {  // this th
 template <int DQ, int DV, bool RAW, bool V_IS_K>
 __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttention d, int splits) {
     constexpr int KS = DQ / 32, DW = DV / 64, QP = DQ * 2 + 16, VP = DV * 2 + 32, PV = V_IS_K ? 1 : DV / 32;
-    __shared__ __align__(16) uint8_t s_q[2][RAW ? 16 * QP : 16];
+    __shared__ __align__(16) uint8_t s_q[2][16 * QP];
     __shared__ __align__(16) uint8_t s_v[64 * VP];
     __shared__ __align__(16) at_s4 s_p[2][4][64];
     __shared__ __align__(16) uint16_t s_newk[RAW ? DQ : 8], s_newv[RAW ? DV : 8];
@@ -407,6 +407,17 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
     const int per = a.heads / a.kv_heads, tiles = (per + 15) / 16, dq = a.dim1 + a.dim2;
     const int split = blockIdx.x, g = blockIdx.y / tiles, h0 = g * per + 16 * (blockIdx.y % tiles);
     const int nh = min(16, (g + 1) * per - h0);
+    constexpr int QN = RAW ? 1 : 2 * 16 * DQ / 8 / 256;  // 16-byte pieces of the q planes per thread
+    u32x4 qr[QN];
+    if constexpr (!RAW) {  // requested first: they do not depend on the position
+#pragma unroll
+        for (int i = 0; i < QN; ++i) {
+            const int p = tid + 256 * i, t = p / (2 * DQ), h = p / (DQ / 8) % 16, c = p % (DQ / 8) * 8;
+            qr[i] = u32x4{0, 0, 0, 0};
+            if (h < nh && c < dq)
+                qr[i] = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.Q) + ((int64_t)t * a.heads + h0 + h) * dq + c);
+        }
+    }
     const int64_t past = *d.d_past;
     const int64_t lo = a.window > 0 && past - a.window + 1 > 0 ? past - a.window + 1 : 0;
     const int wc0 = (int)(lo / 64), kc = (a.keep_first + 63) / 64, nk = a.window > 0 ? (kc < wc0 ? kc : wc0) : 0;
@@ -482,18 +493,16 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
                 if (writer && c < a.vdim) static_cast<uint16_t*>(d.v_cache)[past * a.v_row + (int64_t)g * a.v_head + c] = b;
             }
         }
-        __syncthreads();
-    }
-    // the fragment of q's plane t for columns 32 ks + 8 rg .. of head j (columns past the key size meet zero keys)
-    const uint16_t* qp = static_cast<const uint16_t*>(a.Q) + (int64_t)(h0 + (j < nh ? j : nh - 1)) * dq;
-    auto q_frag = [&](int t, int ks) {
-        if constexpr (RAW) {
-            return *reinterpret_cast<const at_b8*>(s_q[t] + j * QP + (32 * ks + 8 * rg) * 2);
-        } else {
-            const int col = 32 * ks + 8 * rg;
-            return *reinterpret_cast<const at_b8*>(qp + (int64_t)t * a.heads * dq + (col < dq ? col : 0));
+    } else {
+#pragma unroll
+        for (int i = 0; i < QN; ++i) {
+            const int p = tid + 256 * i, t = p / (2 * DQ), h = p / (DQ / 8) % 16, c = p % (DQ / 8) * 8;
+            *reinterpret_cast<u32x4*>(s_q[t] + h * QP + c * 2) = qr[i];
         }
-    };
+    }
+    __syncthreads();
+    // the fragment of q's plane t for columns 32 ks + 8 rg .. of head j
+    auto q_frag = [&](int t, int ks) { return *reinterpret_cast<const at_b8*>(s_q[t] + j * QP + (32 * ks + 8 * rg) * 2); };
     at_f4 acc[DW];
 #pragma unroll
     for (int i = 0; i < DW; ++i) acc[i] = at_f4{0.f, 0.f, 0.f, 0.f};
