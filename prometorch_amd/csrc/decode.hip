@@ -597,12 +597,13 @@ int ptm_decode_create(const ptm_decode_config* cfg, ptm_decoder** out) {
     d->cfg = c;
     d->layers.assign(c.layers, c.layers + c.n_layers);
     d->cfg.layers = d->layers.data();
-    d->cfg.rope_factors_short = d->cfg.rope_factors_long = nullptr;  // host arrays of the caller: read below, not kept
     for (const ptm_layer& L : d->layers)
         for (const ptm_qweight* w : {&L.q, &L.k, &L.v, &L.o, &L.gate, &L.up, &L.down})
             if (!tuned_type(w->ggml_type)) d->untuned_types = true;
 
-    if ((rc = decoder_init(d)) != PTM_OK) { ptm_decode_destroy(d); return rc; }
+    rc = decoder_init(d);
+    d->cfg.rope_factors_short = d->cfg.rope_factors_long = nullptr;  // host arrays of the caller: read above, not kept
+    if (rc != PTM_OK) { ptm_decode_destroy(d); return rc; }
     *out = d;
     return PTM_OK;
 }
