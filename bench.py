@@ -169,7 +169,7 @@ def blocks_main(steps, warmup, only=None):
     def measure(m):
         tokens = [int(t) for t in synth.rng_for(SEED, 77).integers(0, BLOCK_VOCAB, 2048)]
         r = {}
-        for n in (512, 2048):
+        for n in (32, 512, 2048):
             m.set_past_len(0)
             m.prefill(tokens[:n])
             ts = []

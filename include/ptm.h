@@ -505,7 +505,7 @@ void* ptm_decode_stream(ptm_decoder* d);
  *   embedding table; x += RMSNorm(W_proj g, side_norm)
  * Mixers:
  *   PTM_MIX_ATTENTION  GQA; q and k RMS-normed over the whole projection, rotated, scores scale * q.k, optionally
- *                      softcap * tanh(score / softcap), sliding window with kept first positions
+ *                      softcap * tanh(score / softcap), sliding window with kept first positions (both mixers take these)
  *   PTM_MIX_LATENT     q per head [dim | rot_dim]; one latent c (RMS-normed) and one rotated key part per position are
  *                      cached; per head k = [W_uk c | rotated part], v = W_uv c.  A decode step never expands the cache:
  *                      W_uk moves onto the query and W_uv onto the attended latent.

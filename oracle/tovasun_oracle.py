@@ -102,7 +102,7 @@ def latent_attention(h, w, name, m, eps):
     v = (c @ w[name + "uv"].T).reshape(n, H, m["vdim"])
     full_q = np.concatenate([q[:, :, :d], q_rot], axis=2)
     full_k = np.concatenate([k, np.broadcast_to(k_rot, (n, H, rd))], axis=2)
-    o = softmax_attend(full_q, full_k, v, m["scale"], visible(n, m.get("mask")))
+    o = softmax_attend(full_q, full_k, v, m["scale"], visible(n, m.get("mask")), m.get("softcap"))
     return o.reshape(n, -1) @ w[name + "o"].T
 
 

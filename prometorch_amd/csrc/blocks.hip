@@ -313,13 +313,14 @@ static int block_check(const ptm_block& L, int hidden, int side_dim) {
     int rc;
     if (latent(L)) {
         if (L.rot_dim <= 0 || L.kv_rank <= 0 || L.rot.dims > L.rot_dim) return PTM_E_SHAPE;
-        if (L.keep_first || L.softcap != 0.0f) return PTM_E_UNSUPPORTED;
+        if (L.dim > 1024 || L.kv_rank > 2048 || L.kv_rank + L.rot_dim > 8000) return PTM_E_UNSUPPORTED;
         if (!L.k_norm) return PTM_E_NULL;
         if ((rc = matrix_check(L.expand, expand_rows(L), L.kv_rank))) return rc;
     } else {
         if (L.kv_heads <= 0 || L.heads % L.kv_heads || L.rot.dims > L.dim) return PTM_E_SHAPE;
         if (!L.q_norm || !L.k_norm) return PTM_E_NULL;
     }
+    if (L.vdim > 2048 || L.dim > 4000 || attn_cols(L) > 36864 || hidden > 36864 || L.ff > 36864) return PTM_E_UNSUPPORTED;
     if (!L.norm1 || !L.norm1b) return PTM_E_NULL;
     if ((rc = matrix_check(L.in, qkv_rows(L), hidden)) || (rc = matrix_check(L.out, hidden, attn_cols(L)))) return rc;
     if (L.ff < 0) return PTM_E_SHAPE;
@@ -657,10 +658,13 @@ int blocks_head(BlockStack* b, int row, float* logits, float* xn, int64_t* d_nex
 }
 
 // ---- prompt rows -----------------------------------------------------------------------------------
-// positions a chunk of `rows` rows may have to expand latents for
+// first position whose latents a chunk at pos0 expands, and how many positions a chunk of `rows` rows may expand at most
+static int64_t expand_from(const ptm_block& L, int64_t pos0) {
+    return L.window > 0 && !L.keep_first && pos0 - L.window + 1 > 0 ? pos0 - L.window + 1 : 0;
+}
 static size_t expand_positions(const BlockStack* b, const ptm_block& L, int rows) {
     const size_t all = (size_t)b->cfg.max_seq, n = (size_t)rows + (size_t)L.window;
-    return L.window > 0 && n < all ? n : all;
+    return L.window > 0 && !L.keep_first && n < all ? n : all;
 }
 
 int blocks_reserve(BlockStack* b, int rows) {
@@ -785,7 +789,7 @@ int blocks_rows(BlockStack* b, const int* tokens_host, int M, int64_t pos0, floa
             else hipLaunchKernelGGL(latent_prep_rows_kernel<false>, dim3(M), dim3(256), 0, s, m);
             PTM_TRY(launch_status());
             // keys and values of every position some row of the chunk sees
-            const int64_t lo = L.window > 0 && pos0 - L.window + 1 > 0 ? pos0 - L.window + 1 : 0, row = k_row(L), er = expand_rows(L);
+            const int64_t lo = expand_from(L, pos0), row = k_row(L), er = expand_rows(L);
             const uint8_t* cache = static_cast<const uint8_t*>(run.k);
             PTM_TRY(dense_gemm(product(L.expand, cache + lo * row * es, row, (int)(pos0 + M - lo), GEMM_ELEM, b->r_kv, er), s));
             a.kv_heads = L.heads;

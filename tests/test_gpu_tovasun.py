@@ -8,7 +8,7 @@ import pytest
 from oracle import tovasun_oracle as T
 from prometorch_amd import _lib, model as registry, ops
 from prometorch_amd.testing import folder_writer as fw, synth
-from tovasun_models import MODELS, attention, latent, layer, model, variant
+from tovasun_models import MODELS, attention, latent, layer, model, random_model, variant
 
 pytestmark = pytest.mark.gpu
 # rms error of a position's logits over their deviation: (worst, 97th percentile, mean).  bfloat16: where two keys of a sharp
@@ -68,6 +68,25 @@ def test_prompt_portions_and_decode(dev, built, name, precision):
     for sizes in ([len(tokens)], [2], [1], [7, 1, 1, 3, 2, 64, 5, 1, 31], [64], [66, 1]):
         assert_close(portions(m, tokens, sizes), want, precision, (name, sizes))
     m.close()
+
+
+@pytest.mark.parametrize("seed", range(24))
+def test_random_designs(dev, tmp_path, seed):
+    cfg = random_model(seed)
+    w = fw.random_weights(cfg, seed + 100)
+    tokens = np.random.default_rng(seed).integers(0, cfg["vocab"], 170).tolist()
+    want = T.logits(tokens, w, cfg)
+    path = fw.write_model_folder(str(tmp_path / "m"), cfg, w)
+    for precision in ("float32", "bfloat16"):
+        m = registry.load(path, max_seq=171, precision=precision)
+        for sizes in ([170], [97, 2, 1, 1, 1, 33, 1], [1]):
+            got = portions(m, tokens, sizes)
+            if precision == "float32":
+                assert_close(got, want, precision, (seed, sizes))
+            else:  # some of these softmaxes turn over on the last bit (single positions up to 0.7 in a rounded oracle too)
+                e = errors(got, want)
+                assert np.quantile(e, 0.9) < 0.1 and e.mean() < 0.05, (seed, sizes, e.mean(), np.quantile(e, 0.9))
+        m.close()
 
 
 @pytest.mark.parametrize("name", ["odd", "all_looped", "large_heads", "beyond_classes"])
@@ -225,6 +244,18 @@ def test_greedy_generation(dev, built, precision):
     if precision == "float32":
         assert gap.max() == 0.0
     m.close()
+
+
+def test_command_line(dev, built, capsys):
+    """Token ids in, the same greedy ids out as through the Python interface."""
+    from prometorch_amd.__main__ import main
+    path, cfg, w, tokens, _ = built("odd")
+    m = registry.load(path, max_seq=64)
+    want = m.generate(tokens[:9], [0.0] * 12, temperature=0.0, top_k=1, top_p=1.0)
+    m.close()
+    args = ["generate", "--model", path, "--tokens", ",".join(map(str, tokens[:9])), "--max-new", "12", "--temperature", "0"]
+    assert main(args) == 0
+    assert capsys.readouterr().out.split() == [str(t) for t in want]
 
 
 def test_sampled_generation(dev, built):

@@ -214,6 +214,21 @@ def test_trace_run_is_executable():
     assert r.returncode == 0 and "--max-tokens" in r.stdout
 
 
+def test_command_line_arguments(monkeypatch, capsys):
+    from prometorch_amd import __main__ as cli
+    fake = FakeModel()
+    fake.generate = lambda prompt, u, temperature, top_k, top_p, repeat_penalty, stop_ids: fake.calls.append(
+        (prompt, len(u), temperature, top_k, list(stop_ids))) or [4, 2]
+    opened = []
+    monkeypatch.setattr(cli.registry, "load", lambda path, max_seq, precision: opened.append((path, max_seq, precision)) or fake)
+    assert cli.main(["generate", "--model", "m", "--tokens", "3,1 2", "--max-new", "5", "--top-k", "7", "--stop", "9", "--dtype", "float32"]) == 0
+    assert capsys.readouterr().out.split() == ["4", "2"]
+    assert opened == [("m", 8, "float32")] and fake.calls == [([3, 1, 2], 5, 0.7, 7, [9]), "closed"]
+    for bad in (["generate", "--model", "m"], ["generate", "--model", "m", "--tokens", "a"], ["generate", "--model", "m", "--tokens", ""]):
+        with pytest.raises(SystemExit):
+            cli.main(bad)
+
+
 def test_planted_variants_differ():
     """The neighbours of a mask that the GPU tests compare against do change the oracle's logits."""
     cfg = MODELS["plain"]

@@ -63,6 +63,36 @@ MODELS = {
 }
 
 
+def random_model(seed):
+    """A design of any shape: sizes, heads, masks, layer order, loop and token input drawn at random."""
+    import random
+    r = random.Random(seed)
+    layers = []
+    for _ in range(r.randint(1, 5)):
+        window = r.choice([0, 1, 2, r.randint(3, 30), r.randint(40, 140)])
+        ff = r.choice([None, r.randint(9, 150), 8 * r.randint(2, 20)])
+        if r.random() < 0.5:
+            kv = r.choice([1, 2, 3])
+            dim = r.choice([r.randint(5, 40), 64, 32, r.randint(60, 130)])
+            mix = attention(kv * r.choice([1, 2, 3, 5, 8, 17]), kv, dim, r.choice([dim, r.randint(3, 90)]),
+                            rot=2 * r.randint(1, dim // 2), window=window, keep=r.choice([0, 1, r.randint(2, 12), 80]) if window else 0,
+                            softcap=r.choice([0.0, 6.0, 40.0]), base=r.choice([100.0, 1e4, 5e5]), sharp=r.choice([1.0, 2.0]))
+            if r.random() < 0.3:
+                mix["rot"]["scaling"] = dict(YARN)
+        else:
+            mix = latent(r.choice([1, 2, 5, 18]), r.randint(4, 70), 2 * r.randint(2, 20), r.choice([r.randint(8, 60), 64, r.randint(65, 300)]),
+                         r.randint(4, 70), window=window, yarn=r.choice([None, YARN, {"factor": 1.7, "fast": 20.0, "slow": 2.0, "original": 700}]),
+                         base=r.choice([300.0, 1e4]), sharp=r.choice([1.0, 2.0]))
+        layers.append(layer(mix, ff))
+    n = len(layers)
+    loop = None
+    if r.random() < 0.6:
+        start = r.randrange(n)
+        loop = (start, r.randint(start + 1, n), r.randint(1, 4))
+    return model(layers, r.choice([r.randint(20, 120), 64, 192]), r.randint(30, 300), loop=loop, side=r.choice([0, 1, r.randint(2, 70)]),
+                 eps=r.choice([1e-6, 1e-5, 1e-2]))
+
+
 def variant(cfg, **changes):
     """A copy with mixer or mask entries of some layers changed: variant(cfg, l1_size=+1, l1_keep_first=-1)."""
     out = copy.deepcopy(cfg)
