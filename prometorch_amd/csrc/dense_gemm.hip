@@ -1,7 +1,8 @@
 // Prompt products over bfloat16 weights: C[M][N] = A[M][K] . W[N][K]^T on the matrix cores.
 //
 // dense_gemm_kernel (bfloat16 rows): 4 waves, BM x BN output tile, 64 values of K per step.  Tiles go global -> registers ->
-// LDS, two LDS buffers, so a step has one barrier and the next step's loads are in flight while the MFMAs of this one run.
+// LDS; two register sets and two LDS buffers, so a step has one barrier and the loads of the next two steps are in flight
+// while its MFMAs run.
 // LDS rows are 128 bytes, the eight 16-byte pieces of row r stored at piece ^ (r % 8): the fragment reads (32 rows, one
 // piece) and the writes touch every bank evenly.  The product is formed transposed (W rows as the A operand), so that a lane
 // holds four consecutive columns of one output row.
@@ -87,14 +88,15 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
         pb[i] = reinterpret_cast<const u32x4*>(g.W + (int64_t)min(n0 + r, g.N - 1) * g.ldw) + pp;
         lb[i] = r * 128 + ((pp ^ (r & 7)) << 4);
     }
-    u32x4 ra[PA], rb[PB];
-    auto fetch = [&](int st) {
+    u32x4 ra0[PA], rb0[PB], ra1[PA], rb1[PB];
+    auto fetch = [&](int st, u32x4 (&ra)[PA], u32x4 (&rb)[PB]) {
+        st = st < steps ? st : steps - 1;
 #pragma unroll
         for (int i = 0; i < PA; ++i) ra[i] = pa[i][st * 8];
 #pragma unroll
         for (int i = 0; i < PB; ++i) rb[i] = pb[i][st * 8];
     };
-    auto stage = [&](int buf) {
+    auto stage = [&](int buf, const u32x4 (&ra)[PA], const u32x4 (&rb)[PB]) {
 #pragma unroll
         for (int i = 0; i < PA; ++i) *reinterpret_cast<u32x4*>(&s_a[buf][la[i]]) = ra[i];
 #pragma unroll
@@ -107,12 +109,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
         for (int b = 0; b < TN; ++b)
 #pragma unroll
             for (int r = 0; r < 16; ++r) acc[a][b][r] = 0.0f;
-    fetch(first);
-    stage(first & 1);
-    __syncthreads();
-    for (int st = first; st < steps; ++st) {
-        const int buf = st & 1;
-        fetch(st + 1 < steps ? st + 1 : st);
+    auto multiply = [&](int buf) {
 #pragma unroll
         for (int ks = 0; ks < 4; ++ks) {
             const int pc = ((2 * ks + kh) ^ (j & 7)) << 4;
@@ -126,7 +123,20 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
 #pragma unroll
                 for (int b = 0; b < TN; ++b) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fb[b], fa[a], acc[a][b], 0, 0, 0);
         }
-        if (st + 1 < steps) stage(buf ^ 1);
+    };
+    fetch(first, ra0, rb0);
+    fetch(first + 1, ra1, rb1);
+    stage(0, ra0, rb0);
+    __syncthreads();
+    // two steps per trip; a step past the end repeats the last one's loads and is not multiplied
+    for (int st = first; st < steps; st += 2) {
+        fetch(st + 2, ra0, rb0);
+        multiply(0);
+        stage(1, ra1, rb1);
+        __syncthreads();
+        fetch(st + 3, ra1, rb1);
+        if (st + 1 < steps) multiply(1);
+        stage(0, ra0, rb0);
         __syncthreads();
     }
 #pragma unroll
