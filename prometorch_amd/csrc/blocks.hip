@@ -42,6 +42,7 @@ __global__ __launch_bounds__(256) void residual_norm_rows_kernel(float* __restri
     const int n4 = wp / 4;
     auto h_at = [&](int i) {
         float4 v = h4[i];
+#pragma unroll 5
         for (int z = 1; z < slabs; ++z) {
             const float4 p = *reinterpret_cast<const float4*>(h + base + z * slab + 4 * i);
             v = make_float4(v.x + p.x, v.y + p.y, v.z + p.z, v.w + p.w);
@@ -145,6 +146,7 @@ __global__ __launch_bounds__(256) void side_rows_kernel(const SideRows a) {
     const int64_t base = blockIdx.x * a.ld;
     for (int i = threadIdx.x; i < a.dim; i += 256) {
         float v = 0.0f;
+#pragma unroll 4
         for (int z = 0; z < a.slabs; ++z) v += a.g[base + z * a.slab + i];
         put_elem<F32>(a.out, base + i, gelu_tanh(v) * bf16_f(e[i]));
     }
