@@ -35,7 +35,7 @@ def build(verbose: bool = True, jobs: int = 8) -> str:
         if len(procs) >= jobs:
             _drain(procs)
     _drain(procs)
-    tmp = LIB + ".tmp"
+    tmp = os.path.join(CSRC, "build", os.path.basename(LIB))
     cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", tmp]
     if verbose:
         print(" ".join(cmd), flush=True)
@@ -48,7 +48,8 @@ def ensure() -> str:
     """The library, built first if it is not there; processes that start together build it once."""
     import fcntl
     if not os.path.exists(LIB):
-        with open(LIB + ".lock", "w") as lock:
+        os.makedirs(os.path.join(CSRC, "build"), exist_ok=True)
+        with open(os.path.join(CSRC, "build", "lock"), "w") as lock:
             fcntl.flock(lock, fcntl.LOCK_EX)
             if not os.path.exists(LIB):
                 build(verbose=False, jobs=min(16, max(4, len(os.sched_getaffinity(0)))))
