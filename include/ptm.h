@@ -512,7 +512,8 @@ void* ptm_decode_stream(ptm_decoder* d);
  * Weights are bfloat16 matrices (ggml_type PTM_TYPE_BF16), rows zero-padded to multiples of 64 values
  * (ptm_dense_cols); vectors are fp32, zero-padded alike; `vec64` below marks such a vector. */
 #define PTM_TYPE_BF16 30u
-enum { PTM_MIX_ATTENTION = 0, PTM_MIX_LATENT = 1 };
+enum { PTM_MIX_ATTENTION = 0, PTM_MIX_LATENT = 1, PTM_MIX_WKV = 2 };
+enum { PTM_FF_RELU2 = 0, PTM_FF_SWIGLU = 1 };
 enum { PTM_PRECISION_16 = 0, /* bfloat16 caches and prompt GEMM operands, fp32 accumulation and fp32 decode activations */
        PTM_PRECISION_32 = 1  /* fp32 caches and activations throughout (weights stay bfloat16: exact in fp32) */ };
 
@@ -525,6 +526,27 @@ typedef struct {
 } ptm_rotation;
 /* table[max_seq][dims / 2][2] = (cos, sin); angles in double, host memory. */
 int ptm_rope_pairs_host(float* table, int max_seq, const ptm_rotation* rot);
+
+/* PTM_MIX_WKV: o_t = (S + diag(u) k v^T)^T r, S <- diag(w) S + k v^T per head (S [dim][dim], fp32, zero at position 0), with
+ * w = exp(-exp(W_w2 tanh(W_w1 mix_w) + w0)); out = W_o (o / rms(o) per head * norm * silu(W_g mix_g)).  Each of r, k, v, g, w reads
+ * its own mix h + (h of the previous token - h) * mu. */
+typedef struct {
+    int32_t heads, dim, rank;
+    const float* mu;                     /* [5][vec64 hidden], in the order r, k, v, g, w */
+    ptm_qweight w2;                      /* BF16 [heads * dim][rank] */
+    const float *w0, *u, *norm;          /* [heads * dim] */
+} ptm_wkv;
+
+/* A state-space mixer beside the block's attention, on the same input: x, B and C pass a causal convolution and silu; per head
+ * S <- exp(neg_a dt) S + dt B x^T, y = S^T C + D x with dt = softplus(dt + dt_bias); y * silu(z) is RMS-normed in norm_groups equal
+ * parts, times norm * scale.  channels = heads * vdim + 2 * groups * state. */
+typedef struct {
+    int32_t heads, vdim, state, groups, taps, norm_groups;   /* heads 0: none */
+    const float *conv, *conv_b;          /* [channels][taps], the token's own tap last; [channels] */
+    const float *dt_bias, *neg_a, *D;    /* [heads] */
+    const float* norm;                   /* [heads * vdim] */
+    float scale;                         /* 0: 1 */
+} ptm_ssm;
 
 typedef struct {
     int32_t mixer;                       /* PTM_MIX_* */
@@ -544,6 +566,18 @@ typedef struct {
     ptm_qweight side_gate, side_proj;    /* data NULL: no per-layer token input */
     const float* side_norm;              /* vec64 [hidden] */
     int32_t side_offset;                 /* first column of the block's part of the side table */
+    /* attention only: q and k normed per head; v = k as projected (no v rows in `in`, vdim = dim); a term exp(sink[head]) in the
+     * softmax's denominator; attended values times sigmoid of heads * vdim further rows of `in`; then times out_scale (0: 1) */
+    int32_t head_norm, values_are_keys, out_gate;
+    float out_scale;
+    const float* sink;                   /* [heads] or NULL */
+    ptm_wkv wkv;                         /* mixer PTM_MIX_WKV: `in` has the rows [r | k | v | g | W_w1], `out` heads * dim columns */
+    ptm_ssm ssm;                         /* `in` continues with [z | x | B | C | dt], `out` with heads * vdim columns */
+    const float *norm1_bias, *norm2_bias;/* vec64; given: layer norm instead of RMS norm */
+    int32_t ff_kind;                     /* PTM_FF_RELU2: up, down; PTM_FF_SWIGLU: `up` has ff gate rows, then ff up rows */
+    /* decoders with streams, HOST arrays (copied); [0]: mixer, [1]: feed-forward */
+    const float *hc_in[2], *hc_out[2];   /* [streams] */
+    const float* hc_mix[2];              /* [streams from][streams to] */
 } ptm_block;
 
 typedef struct {
@@ -561,6 +595,12 @@ typedef struct {
     int32_t side_dim;
     const float* out_norm;               /* vec64 */
     ptm_qweight lm_head;                 /* BF16 [vocab][hidden] */
+    /* streams > 0: hyper-connections instead of one residual.  That many copies of x; a branch reads u = sum_s in[s] x_s, and
+     * x_t <- sum_s mix[s][t] x_s + out[t] * branch(norm(u)); the head reads their sum.  No post-norms, loop or token input. */
+    int32_t streams;
+    float logit_scale;                   /* 0: 1 */
+    double position_base;                /* > 0: sin and cos of position * position_base^(-2i / hidden) are added to the embedding */
+    const float* out_norm_bias;          /* vec64; given: layer norm */
 } ptm_block_config;
 
 int ptm_dense_cols(int cols);            /* cols rounded up to a multiple of 64 */
@@ -597,6 +637,12 @@ typedef struct {
     int64_t pos0, kv_pos0;
     float scale, softcap;
     int32_t fp32;
+    /* each optional: a term exp(sink[head]) in the denominator; the result times sigmoid(gate[row][head][gate_head]) (fp32, the
+     * first gate_head of the vdim values); times out_scale (0: 1) */
+    const float *sink, *gate;
+    int64_t gate_row;
+    int32_t gate_head;
+    float out_scale;
 } ptm_attention_args;
 int ptm_attention_rows(const ptm_attention_args* a, ptm_stream_t stream);
 

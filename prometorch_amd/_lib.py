@@ -61,26 +61,41 @@ class Rotation(C.Structure):
     _fields_ = [(n, C.c_double) for n in ("base", "factor", "original", "fast", "slow")] + [("dims", C.c_int32)]
 
 
+class Wkv(C.Structure):
+    _fields_ = [("heads", C.c_int32), ("dim", C.c_int32), ("rank", C.c_int32), ("mu", vp), ("w2", QWeight), ("w0", vp), ("u", vp),
+                ("norm", vp)]
+
+
+class Ssm(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("heads", "vdim", "state", "groups", "taps", "norm_groups")] + \
+               [(n, vp) for n in ("conv", "conv_b", "dt_bias", "neg_a", "D", "norm")] + [("scale", f32)]
+
+
 class Block(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "rot_dim", "kv_rank", "window", "keep_first")] + \
                [("scale", f32), ("softcap", f32), ("rot", Rotation), ("in_", QWeight), ("expand", QWeight), ("out", QWeight)] + \
                [(n, vp) for n in ("q_norm", "k_norm", "norm1", "norm1b")] + \
                [("ff", C.c_int32), ("up", QWeight), ("down", QWeight), ("norm2", vp), ("norm2b", vp), ("side_gate", QWeight),
-                ("side_proj", QWeight), ("side_norm", vp), ("side_offset", C.c_int32)]
+                ("side_proj", QWeight), ("side_norm", vp), ("side_offset", C.c_int32)] + \
+               [(n, C.c_int32) for n in ("head_norm", "values_are_keys", "out_gate")] + \
+               [("out_scale", f32), ("sink", vp), ("wkv", Wkv), ("ssm", Ssm), ("norm1_bias", vp), ("norm2_bias", vp),
+                ("ff_kind", C.c_int32)] + [(n, vp * 2) for n in ("hc_in", "hc_out", "hc_mix")]
 
 
 class BlockConfig(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("vocab", "hidden", "n_blocks", "max_seq")] + \
                [("eps", f32), ("precision", C.c_int32), ("use_graph", C.c_int32), ("blocks", C.POINTER(Block)),
                 ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("loop_step", vp),
-                ("embedding", QWeight), ("side_table", QWeight), ("side_dim", C.c_int32), ("out_norm", vp), ("lm_head", QWeight)]
+                ("embedding", QWeight), ("side_table", QWeight), ("side_dim", C.c_int32), ("out_norm", vp), ("lm_head", QWeight),
+                ("streams", C.c_int32), ("logit_scale", f32), ("position_base", C.c_double), ("out_norm_bias", vp)]
 
 
 class AttentionArgs(C.Structure):
     _fields_ = [(n, vp) for n in ("Q", "K1", "K2", "V", "O")] + \
                [(n, i64) for n in ("q_row", "k1_row", "k1_head", "k2_row", "v_row", "v_head", "o_row")] + \
                [(n, C.c_int32) for n in ("rows", "heads", "kv_heads", "dim1", "dim2", "vdim", "window", "keep_first")] + \
-               [("pos0", i64), ("kv_pos0", i64), ("scale", f32), ("softcap", f32), ("fp32", C.c_int32)]
+               [("pos0", i64), ("kv_pos0", i64), ("scale", f32), ("softcap", f32), ("fp32", C.c_int32), ("sink", vp), ("gate", vp),
+                ("gate_row", i64), ("gate_head", C.c_int32), ("out_scale", f32)]
 
 
 class StTensor(C.Structure):

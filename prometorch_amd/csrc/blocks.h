@@ -8,6 +8,10 @@ struct BlockStack;
 int blocks_create(const ptm_block_config& cfg, BlockStack** out);
 void blocks_destroy(BlockStack* b);
 int blocks_runs(const BlockStack* b);
+// Layers that carry state from token to token, which no position can be taken out of again.  blocks_state_copy keeps a copy of
+// all of it, or puts the copy back.
+bool blocks_recurrent(const BlockStack* b);
+int blocks_state_copy(BlockStack* b, bool restore, hipStream_t s);
 // One token (id in *d_token, position *d_past) through all layer runs.  trace: [runs][2][hidden], after the mixer branch and
 // at the end of the layer.
 int blocks_token(BlockStack* b, const int* d_token, const int64_t* d_past, float* trace, hipStream_t s);

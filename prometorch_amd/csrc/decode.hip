@@ -650,6 +650,8 @@ void ptm_decode_destroy(ptm_decoder* d) {
 int ptm_decode_set_past_len(ptm_decoder* d, int64_t past_len) {
     if (!d) return PTM_E_NULL;
     if (past_len < 0 || past_len >= d->cfg.max_seq) return PTM_E_RANGE;
+    // recurrent state stands at past_len tokens: it can start over, not go back to a place in between
+    if (d->blocks && blocks_recurrent(d->blocks) && past_len != 0 && past_len != d->past_len) return PTM_E_STATE;
     d->past_len = past_len;
     d->dev_synced = false;
     return PTM_OK;
@@ -773,7 +775,8 @@ int ptm_decode_prefill(ptm_decoder* d, const int32_t* tokens, int n, int chunk_r
 // The serving loop (promeserve/api_handlers.h:848-923) in one call: prompt, then sample / check for a stop token /
 // feed back until max_new tokens or a stop token (which is not part of the output).  Tokens are generated in chained
 // runs of 16 steps; when a stop token turns up inside a run the steps after it are dropped (the cache rows they wrote
-// lie beyond past_len and are overwritten by whatever comes next).
+// lie beyond past_len and are overwritten by whatever comes next; recurrent state goes back to the run's start and takes the
+// run's steps up to the stop token again).
 int ptm_decode_generate(ptm_decoder* d, const int32_t* prompt, int n_prompt, const ptm_sampling* params,
                         const float* uniforms_host, int max_new, const int32_t* stop_ids, int n_stop, int64_t* out_tokens,
                         int* n_out) {
@@ -793,13 +796,22 @@ int ptm_decode_generate(ptm_decoder* d, const int32_t* prompt, int n_prompt, con
     int token = prompt[n_prompt - 1], produced = 0;
     while (produced < max_new) {
         const int run = max_new - produced < 16 ? max_new - produced : 16;
+        const bool keep = n_stop > 0 && d->blocks && blocks_recurrent(d->blocks);
+        if (keep && (rc = blocks_state_copy(d->blocks, false, d->stream)) != PTM_OK) return rc;
         if ((rc = ptm_decode_sample(d, token, run, uniforms_host + produced, out_tokens + produced)) != PTM_OK) return rc;
         for (int i = 0; i < run; ++i) {
             const int64_t t = out_tokens[produced + i];
             for (int k = 0; k < n_stop; ++k)
                 if (t == stop_ids[k]) {
-                    d->past_len -= run - (i + 1);  // steps i+1.. of the run fed the stop token and what followed it
                     *n_out = produced + i;
+                    if (keep && i + 1 < run) {
+                        d->past_len -= run;
+                        d->dev_synced = false;
+                        if ((rc = blocks_state_copy(d->blocks, true, d->stream)) != PTM_OK) return d->status = rc;
+                        for (int q = 0; q <= i && rc == PTM_OK; ++q) rc = run_steps(d, q ? (int)out_tokens[produced + q - 1] : token, 1);
+                        return rc;
+                    }
+                    d->past_len -= run - (i + 1);  // steps i+1.. of the run fed the stop token and what followed it
                     return PTM_OK;
                 }
         }

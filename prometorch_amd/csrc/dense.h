@@ -29,6 +29,9 @@ __device__ __forceinline__ float gelu_tanh(float z) {
     return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+
 // block-wide sum for WAVES waves; red: WAVES floats of LDS
 template <int WAVES>
 __device__ __forceinline__ float block_sum(float v, float* red) {
@@ -42,11 +45,17 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
     return s;
 }
 
-enum { GEMV_STORE = 0, GEMV_RELU2 = 1, GEMV_SIDE = 2, GEMV_ARGMAX = 3 };
+enum { GEMV_STORE = 0, GEMV_RELU2 = 1, GEMV_SIDE = 2, GEMV_ARGMAX = 3, GEMV_SWIGLU = 4 };
+constexpr int GEMV_SECTIONS = 8;
 
 // y = epilogue(W . prologue(x)).  Vectors are fp32, zero-padded to a multiple of 64 values.
 // Prologue: x' = x + RMS(h) * hw + add0 + add1 (each part optional; x' stored to xout by one workgroup), then RMS(x') * gamma if
 // gamma is given (stored to xn_out by one workgroup).
+// With streams > 0, x is that many vectors x_stride floats apart: x' = sum_s blend[s] x_s + blend[streams] h, and with h the first
+// workgroups store the new streams sum_s store[t][s] x_s + store[t][streams] h to xout (K-padded rows); layer norm if beta is
+// given; then the token shift: rows of section i take x' + (x'_before - x') * mu[i], x'_before from the ring slot of the previous position.
+// With tail_n > 0 (no other prologue), values tail0 .. of x are RMS-normed in tail_parts equal parts, times tail_norm * tail_scale.
+// GEMV_SWIGLU: W holds N gate rows, then N up rows; y = silu(gate) * up.
 struct DenseGemv {
     const uint16_t* W = nullptr;
     int64_t ld = 0;
@@ -65,9 +74,22 @@ struct DenseGemv {
     const int* d_token = nullptr;
     float* part_val = nullptr;       // GEMV_ARGMAX: one (value, index) per workgroup
     int* part_idx = nullptr;
+    int streams = 0;
+    int64_t x_stride = 0;
+    const float *blend = nullptr, *store = nullptr, *beta = nullptr;
+    const float* mu = nullptr;       // [sections][padded K]
+    float* shift = nullptr;          // [2][padded K], by position parity
+    const int64_t* d_past = nullptr;
+    int sections = 0;
+    int section_row[GEMV_SECTIONS + 1] = {};  // first rows; the last entry is N
+    int section_wg[GEMV_SECTIONS + 1] = {};   // first workgroups, set by dense_gemv
+    int tail0 = 0, tail_n = 0, tail_parts = 0;
+    const float* tail_norm = nullptr;
+    float tail_scale = 1.0f;
+    float out_scale = 1.0f;          // factor of every stored y
 };
 int dense_gemv_workgroups(const DenseGemv& g);
-int dense_gemv(const DenseGemv& g, hipStream_t s);
+int dense_gemv(DenseGemv g, hipStream_t s);
 void dense_gemv_init();
 
 // One decode step of a latent mixer around its attention.
@@ -90,8 +112,9 @@ int latent_absorb(const LatentStep& a, hipStream_t s);
 int latent_out(const LatentStep& a, const float* pO, const float* pM, const float* pL, int splits, int o_row, float* out,
                hipStream_t s);
 
-// C = epilogue(A . W^T): GEMM_F32 fp32 C; otherwise element type of the rows (bfloat16, or fp32 when a_fp32)
-enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2 };
+// C = epilogue(A . W^T): GEMM_F32 fp32 C; otherwise element type of the rows (bfloat16, or fp32 when a_fp32).
+// GEMM_SWIGLU: W holds N / 2 gate rows, then N / 2 up rows; C [M][N / 2] = silu(gate) * up.
+enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2, GEMM_SWIGLU = 3 };
 struct DenseGemm {
     const void* A = nullptr;
     int a_fp32 = 0;
@@ -105,7 +128,10 @@ struct DenseGemm {
     // K split over workgroups where the output has too few tiles (GEMM_F32 only): split z leaves its partial sums at
     // C + z * slab; slab_room floats are available for all of them
     int64_t slab = 0, slab_room = 0;
-    int splits = 1;  // set by dense_gemm
+    int splits = 1, tile_cols = 0;  // set by dense_gemm
+    // rows n of W take A + n / section_n * section_a (section_n a multiple of 128; 0: one section)
+    int section_n = 0;
+    int64_t section_a = 0;
 };
 int dense_gemm(DenseGemm g, hipStream_t s, int* splits = nullptr);
 
@@ -120,15 +146,83 @@ struct DecodeAttention {
     const float *q_norm = nullptr, *k_norm = nullptr, *rope = nullptr;
     int dim = 0, vdim_true = 0, rot_dims = 0;
     float eps = 0.0f;
+    int head_norm = 0, values_are_keys = 0;  // q and k normed per head; v = the un-normed k
     void *k_cache = nullptr, *v_cache = nullptr;
     float *pO = nullptr, *pM = nullptr, *pL = nullptr;  // [splits][heads][vdim], [splits][heads] twice
 };
 bool decode_attention_tiled(const ptm_attention_args& a);
 int decode_attention_splits(const ptm_attention_args& a, int max_seq);
 int decode_attention(const DecodeAttention& a, hipStream_t s);
-int decode_attention_merge(const float* pO, const float* pM, const float* pL, int splits, int heads, int vdim, float* out,
+// a: heads, vdim, and the sink, gate and scale of the finished values
+int decode_attention_merge(const float* pO, const float* pM, const float* pL, int splits, const ptm_attention_args& a, float* out,
                            hipStream_t s);
 int attention_rows(const ptm_attention_args& a, const int64_t* d_past, bool q_fp32_out_fp32, hipStream_t s);
+
+// ---- recurrent mixers (recurrent.hip) ----------------------------------------------------------
+bool recurrent_supported(int keys);
+int64_t recurrent_state_floats(int heads, int keys, int columns);
+
+struct WkvStep {
+    const float* proj;        // [r | k | v | g | low-rank]
+    const uint16_t* w2;       // [heads * dim][w2_ld]
+    int64_t w2_ld;
+    int heads, dim, rank;
+    const float *w0, *u, *norm;
+    float eps;
+    const int64_t* d_past;
+    float* state;
+    float* out;               // [heads * dim]
+};
+int wkv_step(const WkvStep& a, hipStream_t s);
+
+struct WkvRows {
+    const float* proj;        // [M][ld]: r, k, v, g, `section` floats apart
+    int64_t ld, section;
+    const float* w;           // [M][w_ld] low-rank decay products
+    int64_t w_ld;
+    int M, heads, dim;
+    const float *w0, *u, *norm;
+    float eps;
+    int64_t pos0;
+    float* state;
+    float* o;                 // [M][o_ld], may be the v columns of proj
+    int64_t o_ld;
+    void* out;                // [M][out_ld]
+    int64_t out_ld;
+    const float* h_last;      // the mixer's last input row, kept for the next token's shift
+    float* shift;
+    int wp;
+};
+int wkv_rows(const WkvRows& a, bool fp32, hipStream_t s);
+int token_shift_rows(const float* h, const float* shift, const float* mu, int n, int rows, int64_t pos0, int wp, bool fp32, void* out, hipStream_t s);
+int tanh_rows(const float* g, int slabs, int64_t slab, int rows, int n, bool fp32, void* out, hipStream_t s);
+
+struct SsmShape {
+    int heads, vdim, state, groups, taps, norm_groups;
+    const float *conv, *conv_b, *dt_bias, *neg_a, *D, *norm;  // neg_a: -exp(A_log)
+    float scale;
+};
+struct SsmStep {
+    SsmShape m;
+    const float* proj;        // [z | x | B | C | dt]
+    const int64_t* d_past;
+    float *ring, *state;      // [taps][channels]; state
+    float* out;               // [heads * vdim], before its norm
+};
+int ssm_step(const SsmStep& a, hipStream_t s);
+struct SsmRows {
+    SsmShape m;
+    const float* proj;        // [M][ld]
+    int64_t ld;
+    int M;
+    int64_t pos0;
+    float eps;
+    float *ring, *state;
+    float* conv;              // [M][x | B | C]
+    void* out;                // [M][out_ld]
+    int64_t out_ld;
+};
+int ssm_rows(const SsmRows& a, bool fp32, hipStream_t s);
 
 int argmax_finish(const float* part_val, const int* part_idx, int n, int64_t* out_index, const ArgmaxAdvance adv, hipStream_t s);
 

@@ -24,6 +24,14 @@ __device__ __forceinline__ void tile_of(int wg, int tiles_m, int tiles_n, int& t
 
 __device__ __forceinline__ float relu2(float v) { return v > 0.0f ? v * v : 0.0f; }
 
+// row of W behind column n of the product.  GEMM_SWIGLU: each 32 columns are 16 gate rows and the 16 up rows of the same values,
+// which one lane's accumulators hold together.
+__device__ __forceinline__ int weight_row(const DenseGemm& g, int n) {
+    if (g.epilogue != GEMM_SWIGLU) return min(n, g.N - 1);
+    const int ff = g.N / 2, v = min((n >> 5) * 16 + (n & 15), ff - 1);
+    return (n & 16) ? ff + v : v;
+}
+
 // four consecutive columns n .. n + 3 of row m
 template <bool F32>
 __device__ __forceinline__ void store4(const DenseGemm& g, int split, int m, int n, float v0, float v1, float v2, float v3) {
@@ -57,6 +65,21 @@ __device__ __forceinline__ void store4(const DenseGemm& g, int split, int m, int
     }
 }
 
+// 32 columns of GEMM_SWIGLU: accumulators 0..7 are gates, 8..15 the ups of the same values
+template <bool F32>
+__device__ __forceinline__ void store_glu(const DenseGemm& g, int m, int n, int kh, const gm_f16& acc) {
+    DenseGemm o = g;
+    o.epilogue = GEMM_ELEM;
+    o.N = g.N / 2;
+#pragma unroll
+    for (int q = 0; q < 2; ++q) {
+        const int v = n / 2 + 8 * q + 4 * kh;
+        if (v < o.N)
+            store4<F32>(o, 0, m, v, silu_f(acc[4 * q]) * acc[8 + 4 * q], silu_f(acc[4 * q + 1]) * acc[9 + 4 * q],
+                        silu_f(acc[4 * q + 2]) * acc[10 + 4 * q], silu_f(acc[4 * q + 3]) * acc[11 + 4 * q]);
+    }
+}
+
 template <int BM, int BN, int WM, int WN>
 __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
     static_assert((BM / WM) * (BN / WN) == 4, "four waves");
@@ -66,12 +89,13 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int j = lane & 31, kh = lane >> 5;
     int tm, tn;
-    const int tiles_m = (g.M + BM - 1) / BM, tiles_n = (g.N + BN - 1) / BN, split = blockIdx.x / (tiles_m * tiles_n);
+    const int tiles_m = (g.M + BM - 1) / BM, tiles_n = (g.tile_cols + BN - 1) / BN, split = blockIdx.x / (tiles_m * tiles_n);
     tile_of(blockIdx.x - split * tiles_m * tiles_n, tiles_m, tiles_n, tm, tn);
     const int m0 = tm * BM, n0 = tn * BN;
     const int wm = (wave % (BM / WM)) * WM, wn = (wave / (BM / WM)) * WN;
     const int all = (g.K + 63) / 64, steps = all * (split + 1) / g.splits, first = all * split / g.splits;
     const uint16_t* A = static_cast<const uint16_t*>(g.A);
+    if (g.section_n > 0) A += n0 / g.section_n * g.section_a;
     const int pr = tid >> 3, pp = tid & 7;  // row and piece of this thread's first staged piece; the others 32 rows on
     const u32x4* pa[PA];
     const u32x4* pb[PB];
@@ -85,7 +109,7 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
 #pragma unroll
     for (int i = 0; i < PB; ++i) {
         const int r = pr + 32 * i;
-        pb[i] = reinterpret_cast<const u32x4*>(g.W + (int64_t)min(n0 + r, g.N - 1) * g.ldw) + pp;
+        pb[i] = reinterpret_cast<const u32x4*>(g.W + (int64_t)weight_row(g, n0 + r) * g.ldw) + pp;
         lb[i] = r * 128 + ((pp ^ (r & 7)) << 4);
     }
     u32x4 ra0[PA], rb0[PB], ra1[PA], rb1[PB];
@@ -144,12 +168,17 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(const DenseGemm g) {
         const int m = m0 + wm + 32 * a + j;
         if (m >= g.M) continue;
 #pragma unroll
-        for (int b = 0; b < TN; ++b)
+        for (int b = 0; b < TN; ++b) {
+            if (g.epilogue == GEMM_SWIGLU) {
+                store_glu<false>(g, m, n0 + wn + 32 * b, kh, acc[a][b]);
+                continue;
+            }
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const int n = n0 + wn + 32 * b + 8 * q + 4 * kh;
                 if (n < g.N) store4<false>(g, split, m, n, acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]);
             }
+        }
     }
 }
 
@@ -158,15 +187,16 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const DenseGemm g) 
     __shared__ float s_a[64 * P], s_b[64 * P];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, j = lane & 31, kh = lane >> 5;
     int tm, tn;
-    tile_of(blockIdx.x, (g.M + 63) / 64, (g.N + 63) / 64, tm, tn);
+    tile_of(blockIdx.x, (g.M + 63) / 64, (g.tile_cols + 63) / 64, tm, tn);
     const int m0 = tm * 64, n0 = tn * 64, wm = (wave & 1) * 32, wn = (wave >> 1) * 32;
     const float* A = static_cast<const float*>(g.A);
+    if (g.section_n > 0) A += n0 / g.section_n * g.section_a;
     gm_f16 acc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) acc[r] = 0.0f;
     const int r0 = tid >> 2, c0 = (tid & 3) * 8;
     const float* pa = A + (int64_t)min(m0 + r0, g.M - 1) * g.lda + c0;
-    const uint16_t* pb = g.W + (int64_t)min(n0 + r0, g.N - 1) * g.ldw + c0;
+    const uint16_t* pb = g.W + (int64_t)weight_row(g, n0 + r0) * g.ldw + c0;
     const int steps = (g.K + BK - 1) / BK;
     for (int st = 0; st < steps; ++st) {
         const float4 a0 = *reinterpret_cast<const float4*>(pa + st * BK), a1 = *reinterpret_cast<const float4*>(pa + st * BK + 4);
@@ -184,6 +214,7 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const DenseGemm g) 
     }
     const int m = m0 + wm + j;
     if (m >= g.M) return;
+    if (g.epilogue == GEMM_SWIGLU) return store_glu<true>(g, m, n0 + wn, kh, acc);
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
         const int n = n0 + wn + 8 * q + 4 * kh;
@@ -194,9 +225,14 @@ __global__ __launch_bounds__(256) void dense_gemm_f32_kernel(const DenseGemm g) 
 int dense_gemm(DenseGemm g, hipStream_t s, int* splits) {
     if (!g.A || !g.W || !g.C) return PTM_E_NULL;
     const int kp = up64(g.K);
-    if (g.M <= 0 || g.N <= 0 || g.K <= 0 || g.lda <= 0 || g.ldw < kp || g.ldc < g.N) return PTM_E_SHAPE;
+    const bool glu = g.epilogue == GEMM_SWIGLU;
+    if (g.M <= 0 || g.N <= 0 || g.K <= 0 || g.lda <= 0 || g.ldw < kp || g.ldc < (glu ? g.N / 2 : g.N)) return PTM_E_SHAPE;
+    if ((glu && (g.N & 1)) || g.section_n < 0 || (g.section_n & 127) || (g.section_a & 7)) return PTM_E_SHAPE;
+    if (glu && splits) return PTM_E_SHAPE;
     if (!aligned16(g.A) || !aligned16(g.W) || !aligned16(g.C) || (g.lda & 7) || (g.ldw & 7)) return PTM_E_ALIGN;
-    auto tiles = [&](int bm, int bn) { return ((int64_t)g.M + bm - 1) / bm * ((g.N + bn - 1) / bn); };
+    const int cols = glu ? (g.N / 2 + 15) / 16 * 32 : g.N;  // gates and ups in whole blocks of 16
+    g.tile_cols = cols;
+    auto tiles = [&](int bm, int bn) { return ((int64_t)g.M + bm - 1) / bm * ((cols + bn - 1) / bn); };
     if (tiles(32, 64) * 16 > 0x7fffffff) return PTM_E_UNSUPPORTED;
     // splits that bring `t` tiles to about `target` workgroups, each with at least four steps of K
     auto split = [&](int64_t t, int64_t target) {

@@ -21,23 +21,155 @@ __device__ __forceinline__ float sq4(float4 v, float s) {
 }
 __device__ __forceinline__ float4 add4(float4 a, float4 b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
 
-template <int LPR, int R, int U, bool PRO>
+// A vector formed from streams, in LDS: blend of the streams and the pending branch, norm, token shift.  sec: section of the
+// workgroup's rows.  PUT(i, v) / GET(i): float4 i of the vector.
+template <typename Put, typename Get>
+__device__ __forceinline__ void stream_prologue(const DenseGemv& a, int sec, float* red, Put put, Get get) {
+    const int tid = threadIdx.x, Kp = (a.K + 63) & ~63, n4 = Kp / 4, S = a.streams;
+    const bool first = blockIdx.x == 0;
+    float mean = 0.0f;
+    float4 prev[2][2];  // both ring slots of the first two pieces, requested before the position is known
+    const int64_t pos = a.mu ? *a.d_past : 0;
+    if (a.mu) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int z = 0; z < 2; ++z) prev[u][z] = ld4(a.shift + (int64_t)z * Kp, min(tid + u * DG_THREADS, n4 - 1));
+    }
+    auto mix = [&](int i, const float* c) {
+        float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
+        for (int t = 0; t < S; ++t) {
+            const float4 x = ld4(a.x + t * a.x_stride, i);
+            const float b = c[t];
+            v = make_float4(fmaf(b, x.x, v.x), fmaf(b, x.y, v.y), fmaf(b, x.z, v.z), fmaf(b, x.w, v.w));
+        }
+        if (a.h) {
+            const float4 x = ld4(a.h, i);
+            const float b = c[S];
+            v = make_float4(fmaf(b, x.x, v.x), fmaf(b, x.y, v.y), fmaf(b, x.z, v.z), fmaf(b, x.w, v.w));
+        }
+        return v;
+    };
+    float sum = 0.0f;
+#pragma unroll 2
+    for (int i = tid; i < n4; i += DG_THREADS) {
+        const float4 v = mix(i, a.blend);
+        sum += (v.x + v.y) + (v.z + v.w);
+        put(i, v);
+    }
+    if (a.h && a.store)  // the new streams
+        for (int t = blockIdx.x; t < S; t += gridDim.x)
+            for (int i = tid; i < n4; i += DG_THREADS) reinterpret_cast<float4*>(a.xout + (int64_t)t * Kp)[i] = mix(i, a.store + (int64_t)t * (S + 1));
+    if (!a.gamma && !a.mu) return;
+    if (a.beta) mean = block_sum<DG_WAVES>(sum, red) / (float)a.K;
+    auto centred = [&](int i, float4 v) {  // padding is not part of the variance
+        v = make_float4(v.x - mean, v.y - mean, v.z - mean, v.w - mean);
+        if (4 * i + 3 >= a.K) {
+            if (4 * i >= a.K) v.x = 0.0f;
+            if (4 * i + 1 >= a.K) v.y = 0.0f;
+            if (4 * i + 2 >= a.K) v.z = 0.0f;
+            v.w = 0.0f;
+        }
+        return v;
+    };
+    float r = 1.0f;
+    if (a.gamma) {
+        float ss = 0.0f;
+        for (int i = tid; i < n4; i += DG_THREADS) ss = sq4(centred(i, get(i)), ss);  // a thread reads the pieces it wrote itself
+        r = 1.0f / sqrtf(block_sum<DG_WAVES>(ss, red) / (float)a.K + a.eps);
+    }
+    auto finish = [&](int i, float4 p) {
+        float4 v = get(i);
+        if (a.gamma) {
+            const float4 g = ld4(a.gamma, i);
+            v = centred(i, v);
+            v = make_float4(v.x * r * g.x, v.y * r * g.y, v.z * r * g.z, v.w * r * g.w);
+            if (a.beta) v = add4(v, ld4(a.beta, i));
+        }
+        if (first && a.xn_out) reinterpret_cast<float4*>(a.xn_out)[i] = v;
+        if (a.mu) {
+            if (first) reinterpret_cast<float4*>(a.shift + (pos & 1) * Kp)[i] = v;
+            if (pos == 0) p = make_float4(0.f, 0.f, 0.f, 0.f);
+            const float4 m = ld4(a.mu + (int64_t)sec * Kp, i);
+            v = make_float4(fmaf(p.x - v.x, m.x, v.x), fmaf(p.y - v.y, m.y, v.y), fmaf(p.z - v.z, m.z, v.z), fmaf(p.w - v.w, m.w, v.w));
+        }
+        put(i, v);
+    };
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int i = tid + u * DG_THREADS;
+        if (i < n4) finish(i, a.mu ? (pos & 1) ? prev[u][0] : prev[u][1] : make_float4(0.f, 0.f, 0.f, 0.f));
+    }
+    for (int i = tid + 2 * DG_THREADS; i < n4; i += DG_THREADS)
+        finish(i, a.mu ? ld4(a.shift + ((pos & 1) ^ 1) * Kp, i) : make_float4(0.f, 0.f, 0.f, 0.f));
+}
+
+// The vector with its tail normed in equal parts; s_r: one float per part.  AT(e): element e of the vector in LDS.
+template <typename Put, typename At>
+__device__ __forceinline__ void tail_prologue(const DenseGemv& a, float* s_r, float* red, Put put, At at) {
+    const int tid = threadIdx.x, Kp = (a.K + 63) & ~63, n4 = Kp / 4, part = a.tail_n / a.tail_parts;
+    for (int i = tid; i < n4; i += DG_THREADS) put(i, ld4(a.x, i));
+    __syncthreads();
+    if (a.tail_parts <= 4) {
+        for (int p = 0; p < a.tail_parts; ++p) {
+            float ss = 0.0f;
+            for (int e = tid; e < part; e += DG_THREADS) {
+                const float v = *at(a.tail0 + p * part + e);
+                ss = fmaf(v, v, ss);
+            }
+            ss = block_sum<DG_WAVES>(ss, red);
+            if (tid == 0) s_r[p] = 1.0f / sqrtf(ss / (float)part + a.eps);
+        }
+    } else {
+        for (int p = tid >> 6; p < a.tail_parts; p += DG_WAVES) {
+            float ss = 0.0f;
+            for (int e = tid & 63; e < part; e += 64) {
+                const float v = *at(a.tail0 + p * part + e);
+                ss = fmaf(v, v, ss);
+            }
+            ss = sum64(ss);
+            if ((tid & 63) == 0) s_r[p] = 1.0f / sqrtf(ss / (float)part + a.eps);
+        }
+    }
+    __syncthreads();
+    for (int e = tid; e < a.tail_n; e += DG_THREADS) {
+        float* v = at(a.tail0 + e);
+        *v = *v * s_r[e / part] * a.tail_norm[e] * a.tail_scale;
+    }
+}
+
+// PRO: what forms the vector - 0: nothing, 1: residual and RMS norm, 2: streams, 3: the tail's norm
+template <int LPR, int R, int U, int PRO, bool GLU>
 __global__ __launch_bounds__(DG_THREADS, 4) void dense_gemv_kernel(const DenseGemv a) {
+    static_assert(!GLU || R % 2 == 0, "a lane holds the gate and the up row of a value");
     extern __shared__ __align__(16) float4 s_x[];  // [2][Kp / 8]
     __shared__ float red[DG_WAVES];
     __shared__ int redi[DG_WAVES];
-    constexpr int RPP = 64 / LPR, RW = RPP * R;
+    constexpr int RPP = 64 / LPR, RW = GLU ? RPP * R / 2 : RPP * R;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int li = lane % LPR, lr = lane / LPR;
     const int Kp = (a.K + 63) & ~63, n4 = Kp / 4, n8 = Kp / 8;
-    const int groups = (a.N + RW - 1) / RW, stride = gridDim.x * DG_WAVES;
+    int sec = 0, row0 = 0, rows = a.N, wg = blockIdx.x, wgs = gridDim.x;
+    if constexpr (PRO == 2) {
+        if (a.sections > 0) {
+            while (sec + 1 < a.sections && wg >= a.section_wg[sec + 1]) ++sec;
+            wg -= a.section_wg[sec];
+            wgs = a.section_wg[sec + 1] - a.section_wg[sec];
+            row0 = a.section_row[sec];
+            rows = a.section_row[sec + 1] - row0;
+        }
+    }
+    const int groups = (rows + RW - 1) / RW, stride = wgs * DG_WAVES;
     const int nb = (n8 + LPR * U - 1) / (LPR * U);
-    const uint32_t bytes = (uint32_t)((int64_t)a.N * a.ld * 2);
+    const uint32_t bytes = (uint32_t)((int64_t)a.N * a.ld * (GLU ? 4 : 2));
     const __amdgpu_buffer_rsrc_t rs = make_rsrc(a.W, (int)bytes);
     auto load = [&](int g, int b, u32x4* w) {
 #pragma unroll
         for (int r = 0; r < R; ++r) {
-            const int row = min(g * RW + r * RPP + lr, a.N - 1);
+            int row;
+            if constexpr (GLU) row = min(g * RW + r / 2 * RPP + lr, rows - 1) + (r & 1) * rows;
+            else row = row0 + min(g * RW + r * RPP + lr, rows - 1);
             const uint32_t base = (uint32_t)row * (uint32_t)(a.ld * 2);
 #pragma unroll
             for (int u = 0; u < U; ++u) {
@@ -49,8 +181,19 @@ __global__ __launch_bounds__(DG_THREADS, 4) void dense_gemv_kernel(const DenseGe
     auto put = [&](int i, float4 v) { s_x[(i & 1) * n8 + (i >> 1)] = v; };
 
     u32x4 cur[R * U], nxt[R * U];
-    int g = blockIdx.x * DG_WAVES + wave, b = 0;
-    if constexpr (!PRO) {
+    int g = wg * DG_WAVES + wave, b = 0;
+    auto at = [&](int e) { return reinterpret_cast<float*>(s_x + ((e >> 2) & 1) * n8 + (e >> 3)) + (e & 3); };
+    if constexpr (PRO == 2) {
+        load(min(g, groups - 1), 0, cur);
+        issue_order_fence();
+        stream_prologue(a, sec, red, put, [&](int i) { return s_x[(i & 1) * n8 + (i >> 1)]; });
+        __syncthreads();
+    } else if constexpr (PRO == 3) {
+        load(min(g, groups - 1), 0, cur);
+        issue_order_fence();
+        tail_prologue(a, reinterpret_cast<float*>(s_x + 2 * n8), red, put, at);
+        __syncthreads();
+    } else if constexpr (PRO == 0) {
         for (int i = tid; i < n4; i += DG_THREADS) put(i, ld4(a.x, i));
         load(min(g, groups - 1), 0, cur);
         __syncthreads();
@@ -129,7 +272,7 @@ __global__ __launch_bounds__(DG_THREADS, 4) void dense_gemv_kernel(const DenseGe
     const int64_t side_row = a.epilogue == GEMV_SIDE ? (int64_t)*a.d_token * a.side_ld + a.side_off : 0;
     float best = -INFINITY;
     int best_i = 0x7fffffff;
-    float acc[R];
+    float acc[R], glu_gate = 0.0f;
 #pragma unroll
     for (int r = 0; r < R; ++r) acc[r] = 0.0f;
     while (g < groups) {
@@ -160,8 +303,18 @@ __global__ __launch_bounds__(DG_THREADS, 4) void dense_gemv_kernel(const DenseGe
             for (int r = 0; r < R; ++r) {
                 float v = LPR == 64 ? sum64(acc[r]) : sum_lanes<LPR == 64 ? 32 : LPR>(acc[r]);
                 acc[r] = 0.0f;
-                const int row = g * RW + r * RPP + lr;
-                if (li == 0 && row < a.N) {
+                if constexpr (GLU) {
+                    const int pair = g * RW + r / 2 * RPP + lr;
+                    if (r & 1) {
+                        if (li == 0 && pair < rows) a.y[pair] = glu_gate * v;
+                    } else {
+                        glu_gate = silu_f(v);
+                    }
+                    continue;
+                }
+                const int row = row0 + g * RW + r * RPP + lr;
+                if (li == 0 && row < row0 + rows) {
+                    v *= a.out_scale;
                     if (a.epilogue == GEMV_RELU2) v = v > 0.0f ? v * v : 0.0f;
                     else if (a.epilogue == GEMV_SIDE) v = gelu_tanh(v) * bf16_f(a.side[side_row + row]);
                     else if (a.epilogue == GEMV_ARGMAX && (v > best || (v == best && row < best_i))) { best = v; best_i = row; }
@@ -197,12 +350,24 @@ struct GemvShape { int kind, rows_per_wave; };
 // rows shorter than a wave's 512 values share a wave; long rows take more chunks of one row, short ones more rows
 GemvShape gemv_shape(const DenseGemv& g) {
     const int kp = up64(g.K), ch = (kp + 511) / 512;
-    if (kp <= 64) return {0, 32};
-    if (kp <= 256) return {1, 8};
+    const bool glu = g.epilogue == GEMV_SWIGLU;
+    if (kp <= 64) return {0, glu ? 16 : 32};
+    if (kp <= 256) return {1, glu ? 4 : 8};
+    if (glu) return ch <= 2 ? GemvShape{2, 2} : GemvShape{3, 1};
     const bool few = g.N <= 2 * DG_WAVES * 256;  // two rows per wave would leave compute units without work
     if (ch <= 2) return few ? GemvShape{5, 1} : GemvShape{2, 4};
     if (ch <= 4 || (ch <= 7 && !few)) return few ? GemvShape{5, 1} : GemvShape{3, 2};
     return {4, 1};
+}
+// 512 workgroups over the sections by their rows, each at least one and at most what its rows occupy
+void section_workgroups(DenseGemv& g) {
+    const int per = gemv_shape(g).rows_per_wave * DG_WAVES;
+    for (int i = 0; i < g.sections; ++i) {
+        const int64_t rows = g.section_row[i + 1] - g.section_row[i];
+        int64_t n = (rows + per - 1) / per, share = (512 * rows + g.N / 2) / g.N;
+        if (n > share) n = share > 0 ? share : 1;
+        g.section_wg[i + 1] = g.section_wg[i] + (int)n;
+    }
 }
 }  // namespace
 
@@ -212,42 +377,86 @@ int dense_gemv_workgroups(const DenseGemv& g) {
     return wgs < 512 ? wgs : 512;
 }
 
-template <bool PRO>
+template <int PRO>
 static void gemv_attr() {
     const int lds = 150 * 1024;
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<8, 4, 1, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<32, 4, 1, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<64, 4, 2, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<64, 2, 4, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<64, 1, 8, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<64, 1, 4, PRO>), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+#define PTM_DG(...) (void)hipFuncSetAttribute(reinterpret_cast<const void*>(dense_gemv_kernel<__VA_ARGS__>), hipFuncAttributeMaxDynamicSharedMemorySize, lds)
+    PTM_DG(8, 4, 1, PRO, false);
+    PTM_DG(32, 4, 1, PRO, false);
+    PTM_DG(64, 4, 2, PRO, false);
+    PTM_DG(64, 2, 4, PRO, false);
+    PTM_DG(64, 1, 8, PRO, false);
+    PTM_DG(64, 1, 4, PRO, false);
+    if constexpr (PRO < 3) {
+        PTM_DG(8, 4, 1, PRO, true);
+        PTM_DG(32, 4, 1, PRO, true);
+        PTM_DG(64, 4, 2, PRO, true);
+        PTM_DG(64, 2, 4, PRO, true);
+    }
+#undef PTM_DG
 }
 // one-time kernel attributes, before anything can be captured
 void dense_gemv_init() {
-    gemv_attr<false>();
-    gemv_attr<true>();
+    gemv_attr<0>();
+    gemv_attr<1>();
+    gemv_attr<2>();
+    gemv_attr<3>();
 }
 
-int dense_gemv(const DenseGemv& g, hipStream_t s) {
-    if (!g.W || !g.x || !g.y) return PTM_E_NULL;
-    if (g.N <= 0 || g.K <= 0 || g.ld < up64(g.K)) return PTM_E_SHAPE;
-    if (up64(g.K) > 36864 || (int64_t)g.N * g.ld * 2 >= (int64_t)0xfffffff0u) return PTM_E_UNSUPPORTED;
-    if (!aligned16(g.W) || !aligned16(g.x) || (g.ld & 7)) return PTM_E_ALIGN;
-    const dim3 grid(dense_gemv_workgroups(g)), block(DG_THREADS);
-    const size_t lds = (size_t)up64(g.K) * 4;
-    const bool pro = g.h || g.add0 || g.add1 || g.gamma || g.xout || g.xn_out;
-#define PTM_DG(LPR, R, U)                                                                            \
-    if (pro) hipLaunchKernelGGL((dense_gemv_kernel<LPR, R, U, true>), grid, block, lds, s, g);       \
-    else hipLaunchKernelGGL((dense_gemv_kernel<LPR, R, U, false>), grid, block, lds, s, g)
+template <int PRO>
+static void gemv_launch(const DenseGemv& g, dim3 grid, size_t lds, hipStream_t s) {
+    const dim3 block(DG_THREADS);
+#define PTM_DG(...) hipLaunchKernelGGL((dense_gemv_kernel<__VA_ARGS__>), grid, block, lds, s, g)
+    if constexpr (PRO < 3) {
+        if (g.epilogue == GEMV_SWIGLU) {
+            switch (gemv_shape(g).kind) {
+                case 0: PTM_DG(8, 4, 1, PRO, true); break;
+                case 1: PTM_DG(32, 4, 1, PRO, true); break;
+                case 2: PTM_DG(64, 4, 2, PRO, true); break;
+                default: PTM_DG(64, 2, 4, PRO, true); break;
+            }
+            return;
+        }
+    }
     switch (gemv_shape(g).kind) {
-        case 0: PTM_DG(8, 4, 1); break;
-        case 1: PTM_DG(32, 4, 1); break;
-        case 2: PTM_DG(64, 4, 2); break;
-        case 3: PTM_DG(64, 2, 4); break;
-        case 4: PTM_DG(64, 1, 8); break;
-        default: PTM_DG(64, 1, 4); break;
+        case 0: PTM_DG(8, 4, 1, PRO, false); break;
+        case 1: PTM_DG(32, 4, 1, PRO, false); break;
+        case 2: PTM_DG(64, 4, 2, PRO, false); break;
+        case 3: PTM_DG(64, 2, 4, PRO, false); break;
+        case 4: PTM_DG(64, 1, 8, PRO, false); break;
+        default: PTM_DG(64, 1, 4, PRO, false); break;
     }
 #undef PTM_DG
+}
+
+int dense_gemv(DenseGemv g, hipStream_t s) {
+    if (!g.W || !g.x || !g.y) return PTM_E_NULL;
+    if (g.N <= 0 || g.K <= 0 || g.ld < up64(g.K)) return PTM_E_SHAPE;
+    const int64_t rows = g.epilogue == GEMV_SWIGLU ? 2 * (int64_t)g.N : g.N;
+    if (up64(g.K) > 36864 || rows * g.ld * 2 >= (int64_t)0xfffffff0u) return PTM_E_UNSUPPORTED;
+    if (!aligned16(g.W) || !aligned16(g.x) || (g.ld & 7)) return PTM_E_ALIGN;
+    if (g.sections > 0) {
+        if (g.sections > GEMV_SECTIONS || g.streams <= 0 || g.section_row[0] != 0 || g.section_row[g.sections] != g.N) return PTM_E_SHAPE;
+        for (int i = 0; i < g.sections; ++i)
+            if (g.section_row[i + 1] <= g.section_row[i]) return PTM_E_SHAPE;
+        section_workgroups(g);
+    }
+    const dim3 grid(g.sections > 0 ? g.section_wg[g.sections] : dense_gemv_workgroups(g));
+    const size_t lds = (size_t)up64(g.K) * 4;
+    if (g.streams > 0) {
+        if (!g.blend || (g.store && !g.xout) || (g.mu && (!g.shift || !g.d_past)) || (g.beta && !g.gamma)) return PTM_E_NULL;
+        if (g.x_stride & 3) return PTM_E_ALIGN;
+        gemv_launch<2>(g, grid, lds, s);
+    } else if (g.tail_n > 0) {
+        if (!g.tail_norm) return PTM_E_NULL;
+        if (g.tail_parts <= 0 || g.tail_n % g.tail_parts || g.tail0 + g.tail_n > g.K) return PTM_E_SHAPE;
+        if (g.epilogue == GEMV_SWIGLU || g.tail_parts > 512) return PTM_E_UNSUPPORTED;
+        gemv_launch<3>(g, grid, lds + (size_t)g.tail_parts * 4, s);
+    } else if (g.h || g.add0 || g.add1 || g.gamma || g.xout || g.xn_out) {
+        gemv_launch<1>(g, grid, lds, s);
+    } else {
+        gemv_launch<0>(g, grid, lds, s);
+    }
     return launch_status();
 }
 

@@ -34,6 +34,12 @@ __device__ __forceinline__ float soft_cap(float s, float cap, float inv_cap) {
     return cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f));
 }
 
+// factor of value dimension v of a finished result: output gate and scale
+__device__ __forceinline__ float out_factor(const ptm_attention_args& a, int64_t row, int head, int v) {
+    const float s = a.out_scale != 0.0f ? a.out_scale : 1.0f;
+    return a.gate && v < a.gate_head ? s * sigmoid_f(a.gate[row * a.gate_row + (int64_t)head * a.gate_head + v]) : s;
+}
+
 __device__ __forceinline__ bool sees(int64_t pos, int64_t key, int window, int keep) {
     return key <= pos && (window <= 0 || pos - key < window || key < keep);
 }
@@ -68,7 +74,7 @@ __global__ __launch_bounds__(64) void attention_rows_kernel(const ptm_attention_
     float acc[VT];
 #pragma unroll
     for (int t = 0; t < VT; ++t) acc[t] = 0.0f;
-    float m = -INFINITY, l = 0.0f;
+    float m = a.sink ? a.sink[h] : -INFINITY, l = a.sink ? 1.0f : 0.0f;
     const int64_t lo = a.window > 0 && pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
     const int64_t keep = a.keep_first < lo ? a.keep_first : lo;
     for (int part = 0; part < 2; ++part) {
@@ -106,7 +112,7 @@ __global__ __launch_bounds__(64) void attention_rows_kernel(const ptm_attention_
     const int64_t o = (int64_t)row * a.o_row + (int64_t)h * a.vdim;
 #pragma unroll
     for (int t = 0; t < VT; ++t)
-        if (lane + 64 * t < a.vdim) put_elem<Q32>(a.O, o + lane + 64 * t, acc[t] * inv);
+        if (lane + 64 * t < a.vdim) put_elem<Q32>(a.O, o + lane + 64 * t, acc[t] * inv * out_factor(a, row, h, lane + 64 * t));
 }
 
 template <bool F32, bool Q32>
@@ -158,7 +164,8 @@ __global__ __launch_bounds__(256, DQ <= 192 && DV <= 128 ? 2 : 1) void attention
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
         for (int r = 0; r < 16; ++r) acc[dt][r] = 0.0f;
-    float m_run = -INFINITY, l_run = 0.0f;
+    // the two lane halves of a query add their sums at the end: one of them holds the sink
+    float m_run = a.sink ? a.sink[head] * LOG2E : -INFINITY, l_run = a.sink && kh == 0 ? 1.0f : 0.0f;
 
     const int64_t p_min = a.pos0 + m_base, p_max = a.pos0 + (m_base + bm < a.rows ? m_base + bm : a.rows) - 1;
     const int wt0 = a.window > 0 && p_min - a.window + 1 > 0 ? (int)((p_min - a.window + 1) / 64) : 0;
@@ -326,7 +333,14 @@ __global__ __launch_bounds__(256, DQ <= 192 && DV <= 128 ? 2 : 1) void attention
 #pragma unroll
         for (int q = 0; q < 4; ++q)
             if (32 * dt + 8 * q < a.vdim) {
-                const float v0 = acc[dt][4 * q] * inv, v1 = acc[dt][4 * q + 1] * inv, v2 = acc[dt][4 * q + 2] * inv, v3 = acc[dt][4 * q + 3] * inv;
+                float v0 = acc[dt][4 * q] * inv, v1 = acc[dt][4 * q + 1] * inv, v2 = acc[dt][4 * q + 2] * inv, v3 = acc[dt][4 * q + 3] * inv;
+                if (a.gate || a.out_scale != 0.0f) {
+                    const int v = 32 * dt + 8 * q + 4 * kh;
+                    v0 *= out_factor(a, row, head, v);
+                    v1 *= out_factor(a, row, head, v + 1);
+                    v2 *= out_factor(a, row, head, v + 2);
+                    v3 *= out_factor(a, row, head, v + 3);
+                }
                 *reinterpret_cast<uint2*>(dst + 32 * dt + 8 * q) =
                     make_uint2((uint32_t)f_bf16(v0) | ((uint32_t)f_bf16(v1) << 16), (uint32_t)f_bf16(v2) | ((uint32_t)f_bf16(v3) << 16));
             }
@@ -348,6 +362,7 @@ static int check_args(const ptm_attention_args& a) {
     if (a.rows <= 0 || a.heads <= 0 || a.kv_heads <= 0 || a.heads % a.kv_heads || a.dim1 <= 0 || a.dim2 < 0 || a.vdim <= 0 ||
         a.window < 0 || a.keep_first < 0 || a.pos0 < 0 || a.kv_pos0 < 0)
         return PTM_E_SHAPE;
+    if (a.gate && a.gate_head <= 0) return PTM_E_SHAPE;
     if (a.kv_pos0 > 0 && (a.keep_first > 0 || a.window <= 0 || a.pos0 - a.window + 1 < a.kv_pos0)) return PTM_E_RANGE;  // a visible key before the array
     if ((a.dim1 | a.dim2 | a.vdim | a.k1_row | a.k1_head | a.k2_row | a.v_row | a.v_head | a.q_row | a.o_row) & 7) return PTM_E_ALIGN;
     if (!aligned16(a.Q) || !aligned16(a.K1) || !aligned16(a.V) || !aligned16(a.O) || (a.K2 && !aligned16(a.K2))) return PTM_E_ALIGN;
@@ -401,7 +416,7 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
     __shared__ __align__(16) uint8_t s_v[64 * VP];
     __shared__ __align__(16) at_s4 s_p[2][4][64];
     __shared__ __align__(16) uint16_t s_newk[RAW ? DQ : 8], s_newv[RAW ? DV : 8];
-    __shared__ float s_m[4][16], s_l[4][16], red[4];
+    __shared__ float s_m[4][16], s_l[4][16], red[4], s_rq[RAW ? 17 : 1];
     const ptm_attention_args& a = d.a;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), j = lane & 15, rg = lane >> 4;
     const int per = a.heads / a.kv_heads, tiles = (per + 15) / 16, dq = a.dim1 + a.dim2;
@@ -463,12 +478,26 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
             const float o = p[c ^ 1] * r * w[c ^ 1], co = cs[2 * (c >> 1)], sn = cs[2 * (c >> 1) + 1];
             return (c & 1) ? v * co + o * sn : v * co - o * sn;
         };
-        const float pq = sumsq_part(d.raw, nq), pk = newest ? sumsq_part(rawk, nkv) : 0.0f;
-        const float rq = 1.0f / sqrtf(block_sum<4>(pq, red) / (float)nq + d.eps);
+        float pk = 0.0f, rq = 0.0f;
+        if (d.head_norm) {  // a wave per head; [16]: the key head
+            for (int h = wave; h < nh + (newest ? 1 : 0); h += 4) {
+                const float* p = h < nh ? d.raw + (h0 + h) * d.dim : rawk + g * d.dim;
+                float ss = 0.0f;
+#pragma unroll 4
+                for (int c = lane; c < d.dim; c += 64) ss = fmaf(p[c], p[c], ss);
+                ss = sum64(ss);
+                if (lane == 0) s_rq[h < nh ? h : 16] = 1.0f / sqrtf(ss / (float)d.dim + d.eps);
+            }
+            __syncthreads();
+        } else {
+            const float pq = sumsq_part(d.raw, nq);
+            pk = newest ? sumsq_part(rawk, nkv) : 0.0f;
+            rq = 1.0f / sqrtf(block_sum<4>(pq, red) / (float)nq + d.eps);
+        }
 #pragma unroll 2
         for (int i = tid; i < nh * DQ; i += 256) {
             const int h = i / DQ, c = i % DQ;
-            const float v = c < d.dim ? turned(d.raw + (h0 + h) * d.dim, d.q_norm + (h0 + h) * d.dim, rq, c) : 0.0f;
+            const float v = c < d.dim ? turned(d.raw + (h0 + h) * d.dim, d.q_norm + (h0 + h) * d.dim, d.head_norm ? s_rq[h] : rq, c) : 0.0f;
             const short hi = bf_bits(v);
             *reinterpret_cast<short*>(s_q[0] + h * QP + c * 2) = hi;
             *reinterpret_cast<short*>(s_q[1] + h * QP + c * 2) = bf_bits(v - bf_val(hi));
@@ -479,8 +508,8 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
             *reinterpret_cast<uint32_t*>(s_q[1] + h * QP + c * 4) = 0;
         }
         if (newest) {
-            const float rk = 1.0f / sqrtf(block_sum<4>(pk, red) / (float)nkv + d.eps);
-            const float* rawv = rawk + nkv + g * d.vdim_true;
+            const float rk = d.head_norm ? s_rq[16] : 1.0f / sqrtf(block_sum<4>(pk, red) / (float)nkv + d.eps);
+            const float* rawv = rawk + (d.values_are_keys ? 0 : nkv) + g * d.vdim_true;
             const bool writer = blockIdx.y % tiles == 0;
             for (int c = tid; c < DQ; c += 256) {
                 const uint16_t b = f_bf16(c < d.dim ? turned(rawk + g * d.dim, d.k_norm + g * d.dim, rk, c) : 0.0f);
@@ -608,11 +637,13 @@ __global__ __launch_bounds__(256, 1) void decode_mfma_kernel(const DecodeAttenti
 // grid (heads, ceil(vdim / 64)): out[h][v] = sum over the splits of their results, weighted by exp(m - max) / total.  Four
 // waves take every fourth split of 64 values; the results are requested before the weights are known.
 __global__ __launch_bounds__(256) void decode_merge_kernel(const float* __restrict__ pO, const float* __restrict__ pM,
-                                                           const float* __restrict__ pL, int splits, int heads, int vdim,
+                                                           const float* __restrict__ pL, int splits, const ptm_attention_args a,
                                                            float* __restrict__ out) {
     __shared__ float s_sum[4][64];
+    const int heads = a.heads, vdim = a.vdim;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.x, v = blockIdx.y * 64 + lane, vc = min(v, vdim - 1);
-    float o[16], mv[4], lv[4], m = -INFINITY;
+    const float sink = a.sink ? a.sink[h] : -INFINITY, factor = out_factor(a, 0, h, vc);
+    float o[16], mv[4], lv[4], m = sink;
 #pragma unroll
     for (int u = 0; u < 16; ++u) o[u] = pO[((int64_t)min(wave + 4 * u, splits - 1) * heads + h) * vdim + vc];
 #pragma unroll
@@ -629,7 +660,9 @@ __global__ __launch_bounds__(256) void decode_merge_kernel(const float* __restri
         mv[u] = expf(mv[u] - m);  // lane + 64 u: split's weight, 0 past the last
         l = fmaf(lv[u], mv[u], l);
     }
-    l = 1.0f / sum64(l);
+    l = sum64(l);
+    if (a.sink) l += expf(sink - m);
+    l = factor / l;
     auto weight = [&](int i) {
         const float w = i < 64 ? mv[0] : i < 128 ? mv[1] : i < 192 ? mv[2] : mv[3];  // wave-uniform i
         return __shfl(w, i & 63, 64);
@@ -643,10 +676,10 @@ __global__ __launch_bounds__(256) void decode_merge_kernel(const float* __restri
     if (wave == 0 && v < vdim) out[(int64_t)h * vdim + v] = (s_sum[0][lane] + s_sum[1][lane]) + (s_sum[2][lane] + s_sum[3][lane]);
 }
 
-int decode_attention_merge(const float* pO, const float* pM, const float* pL, int splits, int heads, int vdim, float* out,
+int decode_attention_merge(const float* pO, const float* pM, const float* pL, int splits, const ptm_attention_args& a, float* out,
                            hipStream_t s) {
     if (splits <= 0 || splits > 256) return PTM_E_UNSUPPORTED;
-    hipLaunchKernelGGL(decode_merge_kernel, dim3(heads, (vdim + 63) / 64), dim3(256), 0, s, pO, pM, pL, splits, heads, vdim, out);
+    hipLaunchKernelGGL(decode_merge_kernel, dim3(a.heads, (a.vdim + 63) / 64), dim3(256), 0, s, pO, pM, pL, splits, a, out);
     return launch_status();
 }
 

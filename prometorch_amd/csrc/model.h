@@ -2,6 +2,7 @@
 #pragma once
 #include "ptm_common.h"
 
+#include <list>
 #include <vector>
 
 struct ptm_model {
@@ -9,6 +10,7 @@ struct ptm_model {
     std::vector<void*> device_allocs;
     std::vector<ptm_layer> layers;
     std::vector<ptm_block> blocks;
+    std::list<std::vector<float>> host_vectors;  // small arrays the blocks point to
     ptm_decode_config cfg{};
     ptm_decoder* dec = nullptr;
 };

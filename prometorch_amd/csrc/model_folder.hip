@@ -221,6 +221,16 @@ struct FolderLoader {
         }
         return PTM_OK;
     }
+    // a tensor's columns at dst column `at` on, all rows
+    int place_columns(HostMatrix& h, const std::string& name, int rows, int cols, int at) const {
+        ptm_st_tensor t;
+        const int rc = tensor(name, rows, cols, &t);
+        if (rc != PTM_OK) return rc;
+        if (strcmp(t.dtype, "BF16") != 0) return PTM_E_UNSUPPORTED;
+        for (int r = 0; r < rows; ++r)
+            memcpy(h.v.data() + (size_t)r * h.ld + at, static_cast<const uint8_t*>(t.data) + 2 * (size_t)r * cols, 2 * (size_t)cols);
+        return PTM_OK;
+    }
     int upload(const HostMatrix& h, ptm_qweight* w) const {
         void* d = nullptr;
         const int rc = model_upload(m, h.v.data(), h.v.size() * 2, &d);
@@ -237,31 +247,47 @@ struct FolderLoader {
         const int rc = place(h, name, rows, cols, 0);
         return rc != PTM_OK ? rc : upload(h, w);
     }
-    // fp32 rows of `cols` values, padded
-    int vectors(const std::string& name, int rows, int cols, bool is_2d, const float** out) const {
+    // a tensor's values as fp32, row by row
+    int values(const std::string& name, int rows, int cols, bool is_2d, std::vector<float>* out) const {
         ptm_st_tensor t;
-        int rc = is_2d ? tensor(name, rows, cols, &t) : tensor(name, cols, 0, &t);
+        const int rc = is_2d ? tensor(name, rows, cols, &t) : tensor(name, cols, 0, &t);
         if (rc != PTM_OK) return rc;
         const bool bf = strcmp(t.dtype, "BF16") == 0;
         if (!bf && strcmp(t.dtype, "F32") != 0) return PTM_E_UNSUPPORTED;
-        std::vector<float> v((size_t)rows * (size_t)up64(cols), 0.0f);
-        for (int r = 0; r < rows; ++r)
-            for (int c = 0; c < cols; ++c) {
-                const size_t at = (size_t)r * cols + c;
-                uint32_t u = 0;
-                if (bf) {
-                    uint16_t b;
-                    memcpy(&b, static_cast<const uint8_t*>(t.data) + 2 * at, 2);
-                    u = (uint32_t)b << 16;
-                } else {
-                    memcpy(&u, static_cast<const uint8_t*>(t.data) + 4 * at, 4);
-                }
-                memcpy(&v[(size_t)r * up64(cols) + c], &u, 4);
+        out->resize((size_t)rows * (size_t)cols);
+        for (size_t i = 0; i < out->size(); ++i) {
+            uint32_t u = 0;
+            if (bf) {
+                uint16_t b;
+                memcpy(&b, static_cast<const uint8_t*>(t.data) + 2 * i, 2);
+                u = (uint32_t)b << 16;
+            } else {
+                memcpy(&u, static_cast<const uint8_t*>(t.data) + 4 * i, 4);
             }
-        void* d = nullptr;
-        if ((rc = model_upload(m, v.data(), v.size() * 4, &d)) != PTM_OK) return rc;
-        *out = static_cast<const float*>(d);
+            memcpy(&(*out)[i], &u, 4);
+        }
         return PTM_OK;
+    }
+    int upload_floats(const std::vector<float>& v, const float** out) const {
+        void* d = nullptr;
+        const int rc = model_upload(m, v.data(), v.size() * 4, &d);
+        if (rc == PTM_OK) *out = static_cast<const float*>(d);
+        return rc;
+    }
+    // fp32 rows of `cols` values, padded
+    int vectors(const std::string& name, int rows, int cols, bool is_2d, const float** out) const {
+        std::vector<float> v, padded((size_t)rows * (size_t)up64(cols), 0.0f);
+        const int rc = values(name, rows, cols, is_2d, &v);
+        if (rc != PTM_OK) return rc;
+        for (int r = 0; r < rows; ++r) memcpy(&padded[(size_t)r * up64(cols)], &v[(size_t)r * cols], 4 * (size_t)cols);
+        return upload_floats(padded, out);
+    }
+    // host copy, owned by the model
+    int host(const std::string& name, int rows, int cols, bool is_2d, const float** out) const {
+        m->host_vectors.emplace_back();
+        const int rc = values(name, rows, cols, is_2d, &m->host_vectors.back());
+        if (rc == PTM_OK) *out = m->host_vectors.back().data();
+        return rc;
     }
     int vector(const std::string& name, int n, const float** out) const { return vectors(name, 1, n, false, out); }
 };
@@ -368,13 +394,188 @@ int load_tovasun(FolderLoader& F, const Json& cfg, ptm_block_config* c) {
     c->blocks = F.m->blocks.data();
     return PTM_OK;
 }
+
+// Grouped-query attention over one projected input, read from `o`: sizes, sink and gate.  Returns the rows of its part of `in`.
+int nadozen_attention_sizes(ConfigReader& R, const Json* o, ptm_block& L) {
+    const Json* mask = o ? o->find("mask") : nullptr;
+    L.heads = R.size(o, "heads");
+    L.kv_heads = R.size(o, "kv_heads");
+    L.dim = R.size(o, "dim");
+    L.vdim = R.size(o, "vdim", L.dim);
+    L.scale = (float)R.real(o, "scale");
+    if (mask && !mask->is_null()) {
+        L.window = R.size(mask, "size");
+        if (L.window <= 0) R.rc = PTM_E_FORMAT;
+    }
+    if (R.rc != PTM_OK || L.heads <= 0 || L.kv_heads <= 0 || L.heads % L.kv_heads || L.dim <= 0 || L.vdim != L.dim) return PTM_E_FORMAT;
+    if ((int64_t)L.heads * up8(L.dim) > 0x3fffff) return PTM_E_UNSUPPORTED;
+    L.mixer = PTM_MIX_ATTENTION;
+    L.rot.base = 1.0;
+    L.head_norm = L.values_are_keys = L.out_gate = 1;
+    return PTM_OK;
+}
+
+// Attention (the projected keys are the values, normed per head for the scores only; a sink; an output gate) and a state-space
+// mixer side by side: one matrix in front of both and one behind.
+int nadozen_parallel(FolderLoader& F, ConfigReader& R, const Json* mix, const std::string& x, int W, ptm_block& L) {
+    const Json *left = mix ? mix->find("left") : nullptr, *right = mix ? mix->find("right") : nullptr;
+    PTM_L(nadozen_attention_sizes(R, left, L));
+    ptm_ssm& m = L.ssm;
+    m.heads = R.size(right, "heads");
+    m.vdim = R.size(right, "vdim");
+    m.state = R.size(right, "state");
+    m.groups = R.size(right, "groups");
+    m.taps = R.size(right, "conv");
+    m.norm_groups = R.size(right, "norm_groups");
+    L.out_scale = (float)R.real(mix, "left_scale");
+    m.scale = (float)R.real(mix, "right_scale");
+    if (R.rc != PTM_OK || m.heads <= 0 || m.vdim <= 0 || m.state <= 0 || m.groups <= 0 || m.taps <= 0 || m.norm_groups <= 0) return PTM_E_FORMAT;
+    if (L.out_scale == 0.0f || m.scale == 0.0f) return PTM_E_UNSUPPORTED;  // a branch that is not there
+    if ((int64_t)m.heads * m.vdim > 0xfffff || (int64_t)m.groups * m.state > 0xfffff) return PTM_E_UNSUPPORTED;
+    const std::string l = x + "left.", r = x + "right.";
+    const int q = L.heads * L.dim, k = L.kv_heads * L.dim, inner = m.heads * m.vdim, channels = inner + 2 * m.groups * m.state,
+              rows = inner + channels + m.heads;
+    HostMatrix in(q + k + q + rows, W);
+    PTM_L(F.place(in, l + "q", q, W, 0));
+    PTM_L(F.place(in, l + "k", k, W, q));
+    PTM_L(F.place(in, l + "g", q, W, q + k));
+    PTM_L(F.place(in, r + "in", rows, W, q + k + q));
+    PTM_L(F.upload(in, &L.in));
+    auto per_head = [&](const std::string& name, int heads, const float** out) {  // weights shared by the heads
+        std::vector<float> v, all;
+        PTM_L(F.values(name, 1, L.dim, false, &v));
+        for (int h = 0; h < heads; ++h) all.insert(all.end(), v.begin(), v.end());
+        return F.upload_floats(all, out);
+    };
+    PTM_L(per_head(l + "q.norm", L.heads, &L.q_norm));
+    PTM_L(per_head(l + "k.norm", L.kv_heads, &L.k_norm));
+    PTM_L(F.vector(l + "sink", L.heads, &L.sink));
+    std::vector<float> v;
+    PTM_L(F.values(r + "conv", channels, m.taps, true, &v));
+    PTM_L(F.upload_floats(v, &m.conv));
+    PTM_L(F.vector(r + "conv.b", channels, &m.conv_b));
+    PTM_L(F.vector(r + "dt_bias", m.heads, &m.dt_bias));
+    PTM_L(F.vector(r + "D", m.heads, &m.D));
+    PTM_L(F.vector(r + "norm", inner, &m.norm));
+    PTM_L(F.values(r + "A_log", 1, m.heads, false, &v));
+    for (float& a : v) a = (float)-std::exp((double)a);
+    PTM_L(F.upload_floats(v, &m.neg_a));
+    HostMatrix out(W, L.heads * up8(L.dim) + inner);
+    PTM_L(F.place(out, l + "o", W, q, 0, 0, 0, L.dim, up8(L.dim)));
+    PTM_L(F.place_columns(out, r + "o", W, inner, L.heads * up8(L.dim)));
+    return F.upload(out, &L.out);
+}
+
+int nadozen_wkv(FolderLoader& F, ConfigReader& R, const Json* mix, const std::string& x, int W, ptm_block& L) {
+    L.mixer = PTM_MIX_WKV;
+    ptm_wkv& m = L.wkv;
+    m.heads = R.size(mix, "heads");
+    m.dim = R.size(mix, "dim");
+    if (R.rc != PTM_OK || m.heads <= 0 || m.dim <= 0) return PTM_E_FORMAT;
+    if ((int64_t)m.heads * m.dim > 0xfffff) return PTM_E_UNSUPPORTED;
+    ptm_st_tensor t;
+    PTM_L(ptm_safetensors_find(F.f, (x + "w1").c_str(), &t));  // its rows are the decay's rank
+    if (t.n_dims != 2 || t.dims[0] <= 0 || t.dims[0] > 0xfffff) return PTM_E_SHAPE;
+    m.rank = (int)t.dims[0];
+    const int hd = m.heads * m.dim;
+    HostMatrix in(4 * hd + m.rank, W);
+    const char* const parts[5] = {"r", "k", "v", "g", "w"};
+    std::vector<float> mu((size_t)5 * up64(W), 0.0f), v;
+    for (int i = 0; i < 5; ++i) {
+        if (i < 4) PTM_L(F.place(in, x + parts[i], hd, W, i * hd));
+        PTM_L(F.values(x + "mu." + parts[i], 1, W, false, &v));
+        memcpy(&mu[(size_t)i * up64(W)], v.data(), 4 * (size_t)W);
+    }
+    PTM_L(F.place(in, x + "w1", m.rank, W, 4 * hd));
+    PTM_L(F.upload(in, &L.in));
+    PTM_L(F.upload_floats(mu, &m.mu));
+    PTM_L(F.matrix(x + "w2", hd, m.rank, &m.w2));
+    PTM_L(F.vector(x + "w0", hd, &m.w0));
+    PTM_L(F.values(x + "u", m.heads, m.dim, true, &v));
+    PTM_L(F.upload_floats(v, &m.u));
+    PTM_L(F.vector(x + "norm", hd, &m.norm));
+    return F.matrix(x + "o", W, hd, &L.out);
+}
+
+// "Nadozen": layers of `wkv` and `parallel` mixers behind layer norms, hyper-connections, a gated-silu feed-forward in some layers,
+// layers that use another one's weights, a position sinusoid on the embedding.
+int load_nadozen(FolderLoader& F, const Json& cfg, ptm_block_config* c) {
+    ConfigReader R;
+    c->vocab = R.size(&cfg, "vocab");
+    c->hidden = R.size(&cfg, "width");
+    c->eps = (float)R.real(cfg.find("norm"), "eps");
+    c->streams = R.size(&cfg, "streams");
+    c->logit_scale = (float)R.real(&cfg, "logit_scale");
+    c->position_base = 10000.0;
+    const Json* layers = cfg.find("layers");
+    if (R.rc != PTM_OK || !layers || layers->kind != Json::Array || layers->items.empty() || layers->items.size() > 4096 || c->vocab <= 0 || c->hidden <= 0 ||
+        c->streams <= 0 || c->logit_scale == 0.0f)
+        return PTM_E_FORMAT;
+    const int n = (int)layers->items.size(), W = c->hidden, S = c->streams;
+    c->n_blocks = n;
+    PTM_L(F.matrix("embed", c->vocab, W, &c->embedding));
+    PTM_L(F.matrix("head", c->vocab, W, &c->lm_head));
+    PTM_L(F.vector("final.norm", W, &c->out_norm));
+    PTM_L(F.vector("final.norm.b", W, &c->out_norm_bias));
+    F.m->blocks.resize((size_t)n);
+    std::vector<int> owner((size_t)n);  // the layer whose tensors layer i uses
+    for (int i = 0; i < n; ++i) {
+        owner[(size_t)i] = i;
+        const Json* of = layers->items[(size_t)i].find("weights_of");
+        if (!of || of->is_null()) continue;
+        const int j = R.size(&layers->items[(size_t)i], "weights_of");
+        if (R.rc != PTM_OK || j >= n) return PTM_E_FORMAT;
+        owner[(size_t)i] = j;
+    }
+    for (int i = 0; i < n; ++i)
+        for (int steps = 0; owner[(size_t)owner[(size_t)i]] != owner[(size_t)i]; ++steps) {
+            if (steps > n) return PTM_E_FORMAT;  // layers that name each other
+            owner[(size_t)i] = owner[(size_t)owner[(size_t)i]];
+        }
+    for (int i = 0; i < n; ++i) {
+        if (owner[(size_t)i] != i) continue;
+        const Json& layer = layers->items[(size_t)i];
+        ptm_block& L = F.m->blocks[(size_t)i];
+        const std::string p = "l" + std::to_string(i) + ".", type = R.text(&layer, "type");
+        const Json *mix = layer.find("mixer"), *mlp = layer.find("mlp");
+        if (R.rc != PTM_OK) return R.rc;
+        if (type == "wkv") PTM_L(nadozen_wkv(F, R, mix, p + "mix.", W, L));
+        else if (type == "parallel") PTM_L(nadozen_parallel(F, R, mix, p + "mix.", W, L));
+        else return PTM_E_UNSUPPORTED;
+        PTM_L(F.vector(p + "norm1", W, &L.norm1));
+        PTM_L(F.vector(p + "norm1.b", W, &L.norm1_bias));
+        if (mlp && !mlp->is_null()) {
+            if (R.text(mlp, "kind") != "dense") return R.rc != PTM_OK ? R.rc : PTM_E_UNSUPPORTED;
+            L.ff = R.size(mlp, "ff");
+            if (R.rc != PTM_OK || L.ff <= 0 || L.ff > 0xfffff) return PTM_E_FORMAT;
+            L.ff_kind = PTM_FF_SWIGLU;
+            HostMatrix up(2 * L.ff, W);
+            PTM_L(F.place(up, p + "mlp.gate", L.ff, W, 0));
+            PTM_L(F.place(up, p + "mlp.up", L.ff, W, L.ff));
+            PTM_L(F.upload(up, &L.up));
+            PTM_L(F.matrix(p + "mlp.down", W, L.ff, &L.down));
+            PTM_L(F.vector(p + "norm2", W, &L.norm2));
+            PTM_L(F.vector(p + "norm2.b", W, &L.norm2_bias));
+        }
+        for (int q = 0; q < (L.ff > 0 ? 2 : 1); ++q) {
+            const std::string h = p + "hc" + std::to_string(q + 1) + ".";
+            PTM_L(F.host(h + "in", 1, S, false, &L.hc_in[q]));
+            PTM_L(F.host(h + "out", 1, S, false, &L.hc_out[q]));
+            PTM_L(F.host(h + "mix", S, S, true, &L.hc_mix[q]));
+        }
+    }
+    for (int i = 0; i < n; ++i)
+        if (owner[(size_t)i] != i) F.m->blocks[(size_t)i] = F.m->blocks[(size_t)owner[(size_t)i]];
+    c->blocks = F.m->blocks.data();
+    return PTM_OK;
+}
 #undef PTM_L
 
 struct Architecture {
     const char* name;
     int (*load)(FolderLoader&, const Json&, ptm_block_config*);
 };
-const Architecture ARCHITECTURES[] = {{"Tovasun", load_tovasun}};
+const Architecture ARCHITECTURES[] = {{"Tovasun", load_tovasun}, {"Nadozen", load_nadozen}};
 
 int load_folder(const std::string& dir, int max_seq, int precision, int use_graph, ptm_model** out) {
     std::string text;
