@@ -154,8 +154,39 @@ def block_model_config(s):
             "token_side": {"dim": s["side"]}}
 
 
-def blocks_main(steps, warmup, only=None):
-    """Decode and prompt throughput of Tovasun models beside the closest existing model of the same size."""
+def nadozen_model_config(s):
+    """[wkv, attention beside state space] pairs at the same width, heads and feed-forward size."""
+    n = s["width"] // 64
+    left = {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5,
+            "mask": {"size": s["long_window"]}}
+    right = {"heads": n, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    mlp = {"kind": "dense", "ff": s["ff"]}
+    layers = [x for _ in range(BLOCK_LAYERS // 2) for x in (
+        {"type": "wkv", "mixer": {"heads": n, "dim": 64}, "rank": 64, "mlp": mlp},
+        {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7, "right_scale": 0.7}, "mlp": mlp})]
+    return {"architecture": "Nadozen", "layers": layers, "norm": {"eps": 1e-6}, "vocab": BLOCK_VOCAB, "width": s["width"], "streams": 4,
+            "logit_scale": 1.0}
+
+
+def decode_state_bytes(cfg, past):
+    """Cache and state bytes a decode step reads (and, of recurrent state, writes), by layer."""
+    total = 0
+    for L in cfg["layers"]:
+        m = L["mixer"]
+        if L["type"] == "latent_attention":
+            total += min(past, m["mask"]["size"]) * (m["kv_rank"] + m["rot_dim"]) * 2
+        elif L["type"] == "wkv":
+            total += 2 * m["heads"] * m["dim"] * m["dim"] * 4
+        else:
+            a = m.get("left", m)
+            total += min(past, a["mask"]["size"]) * 2 * a["kv_heads"] * a["dim"] * 2
+            if "right" in m:
+                total += 2 * m["right"]["heads"] * m["right"]["vdim"] * m["right"]["state"] * 4
+    return total
+
+
+def blocks_main(steps, warmup, only=None, design="tovasun"):
+    """Decode and prompt throughput of a folder design's models beside the closest existing model of the same size."""
     import shutil
     import tempfile
     import torch
@@ -190,13 +221,9 @@ def blocks_main(steps, warmup, only=None):
         r["decode_tok_s"] = 1e3 / r["decode_ms_per_token"]
         return r
 
-    out = {"workload": "tovasun", "layers": BLOCK_LAYERS, "vocab": BLOCK_VOCAB, "past": 2048, "steps": steps, "data": "synthetic, random weights"}
-    for name, s in BLOCK_SHAPES.items():
-        if only and name != only:
-            continue
-        cfg = block_model_config(s)
+    def folder_numbers(name, cfg):
         shapes = fw.tensor_shapes(cfg)
-        folder = tempfile.mkdtemp(prefix="tovasun_bench_")
+        folder = tempfile.mkdtemp(prefix="blocks_bench_")
         try:
             json.dump(cfg, open(os.path.join(folder, "config.json"), "w"))
             one = fw.to_bf16(np.ones(1, np.float32))[0]
@@ -208,14 +235,26 @@ def blocks_main(steps, warmup, only=None):
             log("%s: loaded in %.1fs" % (name, time.time() - t0))
         finally:
             shutil.rmtree(folder)
-        mine = measure(m)
+        r = measure(m)
         m.close()
-        read = sum(2 * int(np.prod(sh)) for n, sh in shapes.items() if n not in ("embed", "side.embed"))
-        kv = BLOCK_LAYERS // 2 * (s["window"] * (s["rank"] + s["rot"]) + 2048 * 2 * s["kv_heads"] * s["dim"]) * 2
-        mine["decode_bytes"] = read + kv
-        mine["decode_hbm_frac"] = (read + kv) / mine["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBS
+        read = sum(2 * int(np.prod(sh)) for n, sh in shapes.items() if n not in ("embed", "side.embed")) + decode_state_bytes(cfg, 2048)
+        r["decode_bytes"] = read
+        r["decode_hbm_frac"] = read / r["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBS
         mats = sum(int(np.prod(sh)) for n, sh in shapes.items() if len(sh) == 2 and n not in ("embed", "side.embed", "head"))
-        mine["prefill_2048_matrix_tflops"] = 2 * mats * 2048 / mine["prefill_2048_ms"] / 1e9
+        r["prefill_2048_matrix_tflops"] = 2 * mats * 2048 / r["prefill_2048_ms"] / 1e9
+        return r
+
+    out = {"workload": design, "layers": BLOCK_LAYERS, "vocab": BLOCK_VOCAB, "past": 2048, "steps": steps, "data": "synthetic, random weights"}
+    for name, s in BLOCK_SHAPES.items():
+        if only and name != only:
+            continue
+        if design == "nadozen":  # the closest model shares the products' kernels and the weights' type
+            out[name] = {"nadozen_bf16": folder_numbers(name, nadozen_model_config(s)), "tovasun_bf16": folder_numbers(name, block_model_config(s))}
+            for k, v in out[name].items():
+                log(name, k, {a: round(b, 3) for a, b in v.items()})
+            torch.cuda.empty_cache()
+            continue
+        mine = folder_numbers(name, block_model_config(s))
         lcfg = dict(synth.QWEN3_4B, hidden=s["width"], n_layers=BLOCK_LAYERS, n_heads=s["heads"], n_kv_heads=s["kv_heads"],
                     head_dim=s["dim"], inter=s["ff"], vocab=BLOCK_VOCAB)
         layers = [synth.make_layer(SEED, i, lcfg) for i in range(BLOCK_LAYERS)]
@@ -263,9 +302,13 @@ def main():
     ap.add_argument("--tovasun", nargs="?", const="all", choices=["all"] + sorted(BLOCK_SHAPES),
                     help="instead of the default workload: Tovasun models (latent and grouped-query attention layers, bfloat16 weights) "
                          "beside the closest existing model at equal sizes")
+    ap.add_argument("--nadozen", nargs="?", const="all", choices=["all"] + sorted(BLOCK_SHAPES),
+                    help="instead of the default workload: Nadozen models (wkv layers, attention beside a state-space mixer, bfloat16 "
+                         "weights) beside Tovasun models of equal size")
     args = ap.parse_args()
-    if args.tovasun:
-        result = blocks_main(args.steps, args.warmup, None if args.tovasun == "all" else args.tovasun)
+    if args.tovasun or args.nadozen:
+        which = args.tovasun or args.nadozen
+        result = blocks_main(args.steps, args.warmup, None if which == "all" else which, "tovasun" if args.tovasun else "nadozen")
         os.write(json_fd, (json.dumps(result) + "\n").encode())
         return
     if args.cpu_child > 0:

@@ -5,6 +5,7 @@ import ctypes as C
 import numpy as np
 import pytest
 
+from folder_helpers import errors, portions
 from oracle import tovasun_oracle as T
 from prometorch_amd import _lib, model as registry, ops
 from prometorch_amd.testing import folder_writer as fw, synth
@@ -15,10 +16,6 @@ pytestmark = pytest.mark.gpu
 # softmax compete, the rounding of q, k and v moves a few positions a long way; rounding the oracle's own q, k, v and norms gives
 # the same positions and the same size (up to 0.16, mean 0.018).
 LIMITS = {"float32": (2e-4, 1e-4, 3e-5), "bfloat16": (0.4, 0.1, 0.03)}
-
-
-def errors(got, want):
-    return np.sqrt(((got - want) ** 2).mean(axis=-1)) / want.std()
 
 
 def assert_close(got, want, precision, what=""):
@@ -41,21 +38,6 @@ def built(tmp_path_factory):
             cache[name] = (path, cfg, w, tokens, T.logits(tokens, w, cfg))
         return cache[name]
     return get
-
-
-def portions(m, tokens, sizes):
-    """Logits at every position, the tokens fed in portions of these sizes (the last size repeats); 1 is a decode step."""
-    m.set_past_len(0)
-    out, at, k = [], 0, 0
-    while at < len(tokens):
-        n = min(sizes[min(k, len(sizes) - 1)], len(tokens) - at)
-        if n == 1:
-            m.step(tokens[at])
-            out.append(m.logits()[None])
-        else:
-            out.append(m.prefill_logits(tokens[at:at + n], range(n)))
-        at, k = at + n, k + 1
-    return np.concatenate(out)
 
 
 # ---- models -----------------------------------------------------------------------------------------
