@@ -30,8 +30,9 @@ MODELS = {
     # every branch at sizes that are multiples of nothing; weights shared by name, also of a layer that comes later
     "odd": model([wkv(3, 13, 5, ff=37), parallel(6, 2, 14, 9, (4, 11, 7, 2, 3, 4), ff=50), 0, wkv(2, 22, 9), 1,
                   parallel(3, 3, 20, 30, (5, 6, 18, 5, 5, 3)), 3], 61, 101, 2),
-    # one stream, one head, one tap, one token of window, one value per head
-    "ones": model([parallel(1, 1, 8, 1, (1, 1, 1, 1, 1, 1), ff=1), wkv(1, 1, 1), parallel(2, 1, 1, 2, (2, 4, 3, 1, 2, 8))], 17, 23, 1, logit_scale=1.0),
+    # one stream, one head, one tap, one token of window, one value per head (no norm over a single value: its sign would turn on the
+    # last bit)
+    "ones": model([parallel(1, 1, 8, 1, (6, 1, 1, 1, 1, 1), ff=1), wkv(1, 6, 1), parallel(2, 1, 4, 2, (1, 8, 3, 1, 2, 1))], 17, 23, 1, logit_scale=1.0),
     # whole sections of 128 rows, states of 64 and 128 keys, windows over several tiles
     "whole": model([wkv(2, 64, 32, ff=96), parallel(4, 2, 64, 100, (4, 32, 128, 1, 4, 1), ff=128), wkv(1, 128, 64), 1], 128, 131, 4),
     # larger heads and states: every tile class of the recurrences, 16 and more query heads per key head, more than four norm parts
