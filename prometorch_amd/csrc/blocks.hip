@@ -477,7 +477,7 @@ struct BlockStack {
     const double* freq = nullptr;
     int branch = 0, r_branch = 0;  // the next branch's number
     const float *pend_store = nullptr, *r_pend_store = nullptr;
-    float *r_hn = nullptr, *r_w = nullptr, *r_conv = nullptr;
+    float *r_hn = nullptr, *r_conv = nullptr, *r_scan = nullptr, *r_decay = nullptr;
     void *r_mix = nullptr, *r_low = nullptr;
     // all recurrent state, and its copy (blocks_state_copy)
     float *state = nullptr, *saved = nullptr;
@@ -503,7 +503,7 @@ static int attn_rows_of(const ptm_block& L) {
     if (latent(L)) return L.heads * (L.dim + L.rot_dim) + L.kv_rank + L.rot_dim;
     return (L.heads + L.kv_heads) * L.dim + (L.values_are_keys ? 0 : L.kv_heads * L.vdim) + (L.out_gate ? L.heads * L.vdim : 0);
 }
-// prompt rows of a wkv mixer: floats between the r, k, v and g of a row
+// prompt rows of a wkv mixer: floats between the r, k, v, g and w of a row
 static int wkv_section(const ptm_block& L) { return up8(L.wkv.heads * L.wkv.dim); }
 static int gate_row(const ptm_block& L) { return attn_rows_of(L) - L.heads * L.vdim; }
 static int qkv_rows(const ptm_block& L) { return attn_rows_of(L) + (has_ssm(L) ? L.ssm.heads * (L.ssm.vdim + 1) + ssm_channels(L.ssm) : 0); }
@@ -1116,18 +1116,22 @@ int blocks_reserve(BlockStack* b, int rows) {
     const ptm_block_config& c = b->cfg;
     const size_t R = (size_t)rows, es = b->f32 ? 4 : 2, W = (size_t)b->wp;
     const size_t S = (size_t)(c.streams > 0 ? c.streams : 1);
-    size_t proj = 0, q = 0, attn = 0, act = 64, kv = 0, shifted = 0, low = 0, decay = 0, conv = 0;
+    size_t proj = 0, q = 0, attn = 0, act = 64, kv = 0, shifted = 0, low = 0, conv = 0, scan = 0, steps = 0;
     for (const ptm_block& L : b->blocks) {
         auto grow = [](size_t& v, size_t n) { v = v > n ? v : n; };
-        grow(proj, (size_t)(wkv(L) ? 4 * wkv_section(L) : up64(qkv_rows(L))));
+        grow(proj, (size_t)(wkv(L) ? 5 * wkv_section(L) : up64(qkv_rows(L))));
         if (wkv(L)) {
             shifted = R * W;
             grow(low, (size_t)up64(L.wkv.rank));
-            grow(decay, (size_t)(L.wkv.heads * L.wkv.dim));
+            grow(scan, (size_t)scan_slabs(L.wkv.dim) * (size_t)(L.wkv.heads * L.wkv.dim));
         } else {
             grow(q, (size_t)q_cols(L));
         }
-        if (has_ssm(L)) grow(conv, (size_t)ssm_channels(L.ssm));
+        if (has_ssm(L)) {
+            grow(conv, (size_t)ssm_channels(L.ssm));
+            grow(scan, (size_t)scan_slabs(L.ssm.state) * (size_t)(L.ssm.heads * L.ssm.vdim));
+            grow(steps, 2 * (size_t)L.ssm.heads);
+        }
         grow(attn, (size_t)up64(attn_cols(L)));
         grow(act, (size_t)up64(L.ff));
         if (latent(L)) grow(kv, expand_positions(b, L, rows) * (size_t)expand_rows(L));
@@ -1137,7 +1141,8 @@ int blocks_reserve(BlockStack* b, int rows) {
     const size_t o_tok = take(4 * R), o_x = take(4 * S * R * W), o_e = take(4 * R * W), o_h = take(4 * (R * W + (size_t)SPLIT_ROOM)), o_p = take(4 * R * proj),
                  o_xn = take(es * R * W), o_q = take(es * R * q), o_at = take(es * R * attn), o_ac = take(es * R * act),
                  o_g = take(es * R * (size_t)up64(c.side_dim > 0 ? c.side_dim : 1)), o_kv = take(es * kv),
-                 o_hn = take(4 * shifted), o_mix = take(es * 5 * shifted), o_low = take(es * R * low), o_w = take(4 * R * decay), o_cv = take(4 * R * conv);
+                 o_hn = take(4 * shifted), o_mix = take(es * 5 * shifted), o_low = take(es * R * low), o_cv = take(4 * R * conv), o_sc = take(4 * R * scan),
+                 o_st = take(4 * R * steps);
     int rc = hip_status(hipMalloc(&b->slab, off));
     if (rc != PTM_OK) return rc;
     if ((rc = hip_status(hipMemset(b->slab, 0, off))) != PTM_OK) return rc;
@@ -1158,8 +1163,9 @@ int blocks_reserve(BlockStack* b, int rows) {
     b->r_hn = (float*)(p + o_hn);
     b->r_mix = p + o_mix;
     b->r_low = p + o_low;
-    b->r_w = (float*)(p + o_w);
     b->r_conv = (float*)(p + o_cv);
+    b->r_scan = (float*)(p + o_sc);
+    b->r_decay = (float*)(p + o_st);
     b->rows = rows;
     return PTM_OK;
 }
@@ -1195,12 +1201,12 @@ static int wkv_prompt(BlockStack* b, const ptm_block& L, const LayerRun& run, in
         return g;
     };
     if (sec == hd && hd % 128 == 0) {
-        DenseGemm g = section(0, 0, 4 * hd, b->r_proj, 4 * sec);
+        DenseGemm g = section(0, 0, 4 * hd, b->r_proj, 5 * sec);
         g.section_n = hd;
         g.section_a = mix;
         PTM_TRY(dense_gemm(g, s));
     } else {
-        for (int i = 0; i < 4; ++i) PTM_TRY(dense_gemm(section(i, i * hd, hd, b->r_proj + i * sec, 4 * sec), s));
+        for (int i = 0; i < 4; ++i) PTM_TRY(dense_gemm(section(i, i * hd, hd, b->r_proj + i * sec, 5 * sec), s));
     }
     // few columns: split over K, the sums taken by the tanh
     DenseGemm g = section(4, 4 * hd, m.rank, b->r_h, up64(m.rank));
@@ -1209,23 +1215,24 @@ static int wkv_prompt(BlockStack* b, const ptm_block& L, const LayerRun& run, in
     int slabs = 1;
     PTM_TRY(dense_gemm(g, s, &slabs));
     PTM_TRY(tanh_rows(b->r_h, slabs, g.slab, M, m.rank, b->f32, b->r_low, s));
-    PTM_TRY(dense_gemm(product(b, m.w2, b->r_low, up64(m.rank), M, GEMM_F32, b->r_w, hd), s));
+    DenseGemm decay = product(b, m.w2, b->r_low, up64(m.rank), M, GEMM_DECAY, b->r_proj + 4 * sec, 5 * sec);
+    decay.bias = m.w0;
+    PTM_TRY(dense_gemm(decay, s));
     WkvRows w{};
     w.proj = b->r_proj;
-    w.ld = w.o_ld = 4 * sec;
+    w.ld = 5 * sec;
     w.section = sec;
-    w.w = b->r_w;
-    w.w_ld = hd;
     w.M = M;
     w.heads = m.heads;
     w.dim = m.dim;
-    w.w0 = m.w0;
     w.u = m.u;
     w.norm = m.norm;
     w.eps = b->cfg.eps;
     w.pos0 = pos0;
     w.state = run.state;
-    w.o = b->r_proj + 2 * sec;
+    w.o = b->r_scan;
+    w.o_ld = hd;
+    w.o_slab = (int64_t)M * hd;
     w.out = b->r_attn;
     w.out_ld = up64(attn_cols(L));
     w.h_last = b->r_hn + (int64_t)(M - 1) * b->wp;
@@ -1311,6 +1318,9 @@ static int attention_prompt(BlockStack* b, const ptm_block& L, const LayerRun& r
         r.ring = run.ring;
         r.state = run.state;
         r.conv = b->r_conv;
+        r.decay = b->r_decay;
+        r.y = b->r_scan;
+        r.y_slab = (int64_t)M * L.ssm.heads * L.ssm.vdim;
         r.out = static_cast<uint8_t*>(b->r_attn) + (size_t)attn_part(L) * es;
         r.out_ld = lda;
         PTM_TRY(ssm_rows(r, f32, s));

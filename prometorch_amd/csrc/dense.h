@@ -114,7 +114,8 @@ int latent_out(const LatentStep& a, const float* pO, const float* pM, const floa
 
 // C = epilogue(A . W^T): GEMM_F32 fp32 C; otherwise element type of the rows (bfloat16, or fp32 when a_fp32).
 // GEMM_SWIGLU: W holds N / 2 gate rows, then N / 2 up rows; C [M][N / 2] = silu(gate) * up.
-enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2, GEMM_SWIGLU = 3 };
+// GEMM_DECAY: fp32 C = exp(-exp(product + bias)).
+enum { GEMM_F32 = 0, GEMM_ELEM = 1, GEMM_RELU2 = 2, GEMM_SWIGLU = 3, GEMM_DECAY = 4 };
 struct DenseGemm {
     const void* A = nullptr;
     int a_fp32 = 0;
@@ -132,6 +133,7 @@ struct DenseGemm {
     // rows n of W take A + n / section_n * section_a (section_n a multiple of 128; 0: one section)
     int section_n = 0;
     int64_t section_a = 0;
+    const float* bias = nullptr;  // [N], GEMM_DECAY
 };
 int dense_gemm(DenseGemm g, hipStream_t s, int* splits = nullptr);
 
@@ -176,24 +178,24 @@ struct WkvStep {
 int wkv_step(const WkvStep& a, hipStream_t s);
 
 struct WkvRows {
-    const float* proj;        // [M][ld]: r, k, v, g, `section` floats apart
+    const float* proj;        // [M][ld]: r, k, v, g and the decays w, `section` floats apart
     int64_t ld, section;
-    const float* w;           // [M][w_ld] low-rank decay products
-    int64_t w_ld;
     int M, heads, dim;
-    const float *w0, *u, *norm;
+    const float *u, *norm;
     float eps;
     int64_t pos0;
     float* state;
-    float* o;                 // [M][o_ld], may be the v columns of proj
-    int64_t o_ld;
+    float* o;                 // [scan_slabs(dim)][M][o_ld], o_slab floats apart
+    int64_t o_ld, o_slab;
+    int groups;               // set by wkv_rows
     void* out;                // [M][out_ld]
     int64_t out_ld;
     const float* h_last;      // the mixer's last input row, kept for the next token's shift
     float* shift;
     int wp;
 };
-int wkv_rows(const WkvRows& a, bool fp32, hipStream_t s);
+int wkv_rows(WkvRows a, bool fp32, hipStream_t s);
+int64_t scan_slabs(int keys);  // partial sums that a scan leaves per row
 int token_shift_rows(const float* h, const float* shift, const float* mu, int n, int rows, int64_t pos0, int wp, bool fp32, void* out, hipStream_t s);
 int tanh_rows(const float* g, int slabs, int64_t slab, int rows, int n, bool fp32, void* out, hipStream_t s);
 
@@ -219,10 +221,14 @@ struct SsmRows {
     float eps;
     float *ring, *state;
     float* conv;              // [M][x | B | C]
+    float* decay;             // [M][2][heads]
+    float* y;                 // [scan_slabs(state)][M][heads * vdim], y_slab floats apart
+    int64_t y_slab;
+    int key_groups;           // set by ssm_rows
     void* out;                // [M][out_ld]
     int64_t out_ld;
 };
-int ssm_rows(const SsmRows& a, bool fp32, hipStream_t s);
+int ssm_rows(SsmRows a, bool fp32, hipStream_t s);
 
 int argmax_finish(const float* part_val, const int* part_idx, int n, int64_t* out_index, const ArgmaxAdvance adv, hipStream_t s);
 

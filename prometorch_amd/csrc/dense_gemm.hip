@@ -41,8 +41,15 @@ __device__ __forceinline__ void store4(const DenseGemm& g, int split, int m, int
         v2 = relu2(v2);
         v3 = relu2(v3);
     }
+    if (g.epilogue == GEMM_DECAY) {
+        auto decay = [&](float v, int k) { return k < g.N ? expf(-expf(v + g.bias[k])) : 0.0f; };
+        v0 = decay(v0, n);
+        v1 = decay(v1, n + 1);
+        v2 = decay(v2, n + 2);
+        v3 = decay(v3, n + 3);
+    }
     const int64_t at = (int64_t)m * g.ldc + n + split * g.slab;
-    if (F32 || g.epilogue == GEMM_F32) {
+    if (F32 || g.epilogue == GEMM_F32 || g.epilogue == GEMM_DECAY) {
         float* c = static_cast<float*>(g.C) + at;
         if (n + 3 < g.N && (g.ldc & 3) == 0) {
             *reinterpret_cast<float4*>(c) = make_float4(v0, v1, v2, v3);
@@ -228,7 +235,8 @@ int dense_gemm(DenseGemm g, hipStream_t s, int* splits) {
     const bool glu = g.epilogue == GEMM_SWIGLU;
     if (g.M <= 0 || g.N <= 0 || g.K <= 0 || g.lda <= 0 || g.ldw < kp || g.ldc < (glu ? g.N / 2 : g.N)) return PTM_E_SHAPE;
     if ((glu && (g.N & 1)) || g.section_n < 0 || (g.section_n & 127) || (g.section_a & 7)) return PTM_E_SHAPE;
-    if (glu && splits) return PTM_E_SHAPE;
+    if (g.epilogue != GEMM_F32 && splits) return PTM_E_SHAPE;  // partial sums have no epilogue
+    if (g.epilogue == GEMM_DECAY && !g.bias) return PTM_E_NULL;
     if (!aligned16(g.A) || !aligned16(g.W) || !aligned16(g.C) || (g.lda & 7) || (g.ldw & 7)) return PTM_E_ALIGN;
     const int cols = glu ? (g.N / 2 + 15) / 16 * 32 : g.N;  // gates and ups in whole blocks of 16
     g.tile_cols = cols;

@@ -359,14 +359,22 @@ GemvShape gemv_shape(const DenseGemv& g) {
     if (ch <= 4 || (ch <= 7 && !few)) return few ? GemvShape{5, 1} : GemvShape{3, 2};
     return {4, 1};
 }
-// 512 workgroups over the sections by their rows, each at least one and at most what its rows occupy
+// At most 512 workgroups (one more would run by itself behind the others): as many as its rows fill for a section of few rows,
+// the rest over the others by their rows.
 void section_workgroups(DenseGemv& g) {
     const int per = gemv_shape(g).rows_per_wave * DG_WAVES;
+    int64_t room = 512, rows_left = 0;
+    auto rows = [&](int i) { return (int64_t)(g.section_row[i + 1] - g.section_row[i]); };
+    auto fill = [&](int i) { return (rows(i) + per - 1) / per; };
+    auto small = [&](int i) { return rows(i) * 16 < g.N && fill(i) <= 16; };
     for (int i = 0; i < g.sections; ++i) {
-        const int64_t rows = g.section_row[i + 1] - g.section_row[i];
-        int64_t n = (rows + per - 1) / per, share = (512 * rows + g.N / 2) / g.N;
-        if (n > share) n = share > 0 ? share : 1;
-        g.section_wg[i + 1] = g.section_wg[i] + (int)n;
+        if (small(i)) room -= fill(i);
+        else rows_left += rows(i);
+    }
+    for (int i = 0; i < g.sections; ++i) {
+        int64_t n = fill(i);
+        if (!small(i) && n > room * rows(i) / rows_left) n = room * rows(i) / rows_left;
+        g.section_wg[i + 1] = g.section_wg[i] + (int)(n > 0 ? n : 1);
     }
 }
 }  // namespace

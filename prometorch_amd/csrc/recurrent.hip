@@ -3,14 +3,19 @@
 //   wkv   o_t = (S + diag(u) k v^T)^T r,  S <- diag(w) S + k v^T          (decay w per key channel and token)
 //   ssm   S <- a S + dt B x^T,  y_t = S^T C + D x                         (decay a per head and token; B, C per group of heads)
 //
-// A state is stored per value column, its key values consecutive and padded: [heads][columns][16 * KPL].  16 lanes share a
-// column, KPL key values each, so a wave holds four columns and a read of the state is consecutive.  The columns of a head do not
-// depend on each other: the prompt kernels walk the tokens one by one with 16 columns per workgroup, the state in registers, the
-// vectors of the next tokens on their way from memory while a tile of tokens is used from LDS.  A sequence's first position starts
-// from zeros instead of the stored state, so nothing has to be cleared between sequences.
+// A state is stored per value column, its key values consecutive and padded: [heads][columns][16 * KPL].
+// One token: 16 lanes share a column, KPL key values each, so a wave holds four columns and a read of the state is consecutive.
+// Prompt rows: neither the columns nor the keys of a state depend on each other, only the sum over the keys does.  A lane is a value
+// column and a wave has KPL keys of 64 columns in registers, so what belongs to a key (r, k, w; B, C) is one value for the whole
+// wave: it is loaded once into a row of 16 lanes and broadcast as a DPP operand of the arithmetic, three instructions per key and
+// token.  A workgroup's four waves add their sums through LDS; up to four workgroups share a head and leave partial sums, which the
+// row kernel behind the scan adds.  The next tile's vectors are on their way while a tile of tokens is used.
+// A sequence's first position starts from zeros instead of the stored state, so nothing has to be cleared between sequences.
 // What a token needs from earlier ones besides the state (the token shift's vector, the convolution's inputs) lies in rings
 // indexed by position; a slot is never read and written by the same launch.
 #include "dense.h"
+
+#include <type_traits>
 
 namespace ptm {
 
@@ -28,6 +33,15 @@ template <int KPL>
 __device__ __forceinline__ void store_keys(float* p, const float (&s)[KPL]) {
 #pragma unroll
     for (int i = 0; i < KPL; i += 4) *reinterpret_cast<float4*>(p + i) = make_float4(s[i], s[i + 1], s[i + 2], s[i + 3]);
+}
+
+// f(integral constants 0 .. N - 1)
+template <int N, int I = 0, typename F>
+__device__ __forceinline__ void static_for(F f) {
+    if constexpr (I < N) {
+        f(std::integral_constant<int, I>{});
+        static_for<N, I + 1>(f);
+    }
 }
 
 // key values per lane for a state of n key channels (0: too many)
@@ -177,100 +191,141 @@ __global__ __launch_bounds__(256) void ssm_step_kernel(const SsmStep a) {
 }
 
 // ---- prompt rows ---------------------------------------------------------------------------------
-// tokens per tile: two tiles of three key vectors each in LDS
-template <int KPL> constexpr int tile_tokens() { return KPL <= 8 ? 16 : KPL == 16 ? 8 : 4; }
+// workgroups that share the keys of a head, four waves of KPL keys each
+static int key_groups(int keys) { return (keys + 4 * keys_per_lane(keys) - 1) / (4 * keys_per_lane(keys)); }
 
-// grid (heads, ceil(dim / 16)), 256 threads
-template <int KPL>
-__global__ __launch_bounds__(256) void wkv_scan_kernel(const WkvRows a) {
-    constexpr int KP = 16 * KPL, TT = tile_tokens<KPL>(), NE = TT * KP / 256;
-    __shared__ __align__(16) float s_r[2][TT * KP], s_k[2][TT * KP], s_w[2][TT * KP];
-    __shared__ float s_v[2][TT * 16];
-    const int tid = threadIdx.x, sub = tid & 15, grp = tid >> 4, h = blockIdx.x, d = a.dim, c = blockIdx.y * 16 + grp;
-    if (h == 0 && blockIdx.y == 0)  // the next token's shift reads the last row
-        for (int i = tid; i < a.wp; i += 256) a.shift[(a.pos0 + a.M - 1) % 2 * a.wp + i] = a.h_last[i];
-    float* state = a.state + ((int64_t)h * d + min(c, d - 1)) * KP + sub * KPL;
-    float S[KPL], u[KPL];
-    if (a.pos0 > 0) load_keys<KPL>(S, state);
+// value of lane N of each row of 16 lanes, as an operand of the next instruction
+template <int N>
+__device__ __forceinline__ float row_lane(float v) { return dpp_f<0x150 + N>(v); }
+
+// Adds the waves' sums of a tile of TT tokens (s_o [4][TT][64]) and stores them: row t0 + t, 64 columns from `out`.
+template <int TT>
+__device__ __forceinline__ void store_tile(const float (*s_o)[TT][64], float* out, int64_t ld, int t0, int M, int columns) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
-    for (int i = 0; i < KPL; ++i) {
-        if (a.pos0 == 0) S[i] = 0.0f;
-        u[i] = sub * KPL + i < d ? a.u[(int64_t)h * d + sub * KPL + i] : 0.0f;
+    for (int q = 0; q < (TT + 3) / 4; ++q) {
+        const int t = wave + 4 * q;
+        if (t < TT && t0 + t < M && lane < columns)
+            out[(int64_t)(t0 + t) * ld + lane] = (s_o[0][t][lane] + s_o[1][t][lane]) + (s_o[2][t][lane] + s_o[3][t][lane]);
     }
-    // element e of a tile: token e / KP, key channel e % KP; a token past the end leaves the state as it is
-    float rr[NE], rk[NE], rw[NE], rv = 0.0f;
-    auto fetch = [&](int t0) {
-#pragma unroll
-        for (int i = 0; i < NE; ++i) {
-            const int e = tid + 256 * i, t = t0 + e / KP, k = e % KP;
-            const bool in = t < a.M && k < d;
-            const int64_t at = (int64_t)min(t, a.M - 1) * a.ld + (int64_t)h * d + min(k, d - 1);
-            const float r0 = a.proj[at], k0 = a.proj[at + a.section], w0 = a.w[(int64_t)min(t, a.M - 1) * a.w_ld + (int64_t)h * d + min(k, d - 1)];
-            rr[i] = in ? r0 : 0.0f;
-            rk[i] = in ? k0 : 0.0f;
-            rw[i] = in ? w0 : -INFINITY;
-        }
-        if (tid < TT * 16) {
-            const int t = t0 + tid / 16, cc = blockIdx.y * 16 + tid % 16;
-            rv = t < a.M && cc < d ? a.proj[(int64_t)t * a.ld + 2 * a.section + (int64_t)h * d + cc] : 0.0f;
-        }
-    };
-    auto stage = [&](int buf) {
-#pragma unroll
-        for (int i = 0; i < NE; ++i) {
-            const int e = tid + 256 * i;
-            s_r[buf][e] = rr[i];
-            s_k[buf][e] = rk[i];
-            s_w[buf][e] = expf(-expf(rw[i] + a.w0[(int64_t)h * d + min(e % KP, d - 1)]));
-        }
-        if (tid < TT * 16) s_v[buf][tid] = rv;
-    };
-    const int tiles = (a.M + TT - 1) / TT;
-    fetch(0);
-    stage(0);
-    __syncthreads();
-    for (int tile = 0; tile < tiles; ++tile) {
-        const int buf = tile & 1;
-        if (tile + 1 < tiles) fetch((tile + 1) * TT);
-        float keep = 0.0f;
-#pragma unroll 4
-        for (int t = 0; t < TT; ++t) {
-            float r[KPL], k[KPL], w[KPL], o = 0.0f;
-            load_keys<KPL>(r, &s_r[buf][t * KP + sub * KPL]);
-            load_keys<KPL>(k, &s_k[buf][t * KP + sub * KPL]);
-            load_keys<KPL>(w, &s_w[buf][t * KP + sub * KPL]);
-            const float v = s_v[buf][t * 16 + grp];
-#pragma unroll
-            for (int i = 0; i < KPL; ++i) {
-                const float kv = k[i] * v;
-                o = fmaf(r[i], fmaf(u[i], kv, S[i]), o);
-                S[i] = fmaf(w[i], S[i], kv);
-            }
-            o = sum16(o);
-            keep = sub == t ? o : keep;
-        }
-        const int t = tile * TT + sub;
-        if (sub < TT && t < a.M && c < d) a.o[(int64_t)t * a.o_ld + (int64_t)h * d + c] = keep;
-        if (tile + 1 < tiles) stage(buf ^ 1);
-        __syncthreads();
-    }
-    if (c < d) store_keys<KPL>(state, S);
 }
 
-// grid rows: each head's o over its root mean square, times norm and silu(gate); a wave per head
-template <bool F32>
-__global__ __launch_bounds__(256) void wkv_out_rows_kernel(const WkvRows a) {
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, d = a.dim;
-    const float *o = a.o + blockIdx.x * a.o_ld, *g = a.proj + blockIdx.x * a.ld + 3 * a.section;
-    for (int h = wave; h < a.heads; h += 4) {
-        float ss = 0.0f;
-        for (int i = lane; i < d; i += 64) ss = fmaf(o[h * d + i], o[h * d + i], ss);
-        const float r = 1.0f / sqrtf(sum64(ss) / (float)d + a.eps);
-        for (int i = lane; i < d; i += 64) {
-            const int c = h * d + i;
-            put_elem<F32>(a.out, blockIdx.x * a.out_ld + c, o[c] * r * a.norm[c] * silu_f(g[c]));
-        }
+// Four keys of 64 columns take a token: o += S^T r, S <- diag(w) S + k v^T.  p: a row of lanes [r | k | w | -], four each.
+// (One block, because the compiler does not fold the broadcasts into the multiply-adds; the wait states are for p.)
+__device__ __forceinline__ void wkv_keys4(float& s0, float& s1, float& s2, float& s3, float& o, float p, float v) {
+    asm("s_nop 1\n\t"
+        "v_fmac_f32_dpp %4, %5, %0 row_newbcast:0 row_mask:0xf bank_mask:0xf\n\t"
+        "v_mul_f32_dpp %0, %5, %0 row_newbcast:8 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %1 row_newbcast:1 row_mask:0xf bank_mask:0xf\n\t"
+        "v_mul_f32_dpp %1, %5, %1 row_newbcast:9 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %2 row_newbcast:2 row_mask:0xf bank_mask:0xf\n\t"
+        "v_mul_f32_dpp %2, %5, %2 row_newbcast:10 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %3 row_newbcast:3 row_mask:0xf bank_mask:0xf\n\t"
+        "v_mul_f32_dpp %3, %5, %3 row_newbcast:11 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %0, %5, %6 row_newbcast:4 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %1, %5, %6 row_newbcast:5 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %2, %5, %6 row_newbcast:6 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %3, %5, %6 row_newbcast:7 row_mask:0xf bank_mask:0xf"
+        : "+&v"(s0), "+&v"(s1), "+&v"(s2), "+&v"(s3), "+&v"(o)
+        : "v"(p), "v"(v));
+}
+
+// grid (heads, key groups * ceil(dim / 64)), 256 threads.  Without the bonus, which the row kernel behind it adds.
+template <int KPL>
+__global__ __launch_bounds__(256, 1) void wkv_scan_kernel(const WkvRows a) {
+    constexpr int KP = 16 * KPL, Q = KPL / 4, TT = 16 / Q;  // Q rows of [r | k | w] of four keys per token
+    __shared__ float s_o[2][4][TT][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), h = blockIdx.x, d = a.dim;
+    const int kg = blockIdx.y % a.groups, c0 = blockIdx.y / a.groups * 64, c = min(c0 + lane, d - 1), k0 = (4 * kg + wave) * KPL;
+    if (h == 0 && blockIdx.y == 0)  // the next token's shift reads the last row
+        for (int i = tid; i < a.wp; i += 256) a.shift[(a.pos0 + a.M - 1) % 2 * a.wp + i] = a.h_last[i];
+    float* state = a.state + ((int64_t)h * d + c) * KP + k0;
+    float S[KPL];
+    if (a.pos0 > 0) load_keys<KPL>(S, state);
+    else
+#pragma unroll
+        for (int i = 0; i < KPL; ++i) S[i] = 0.0f;
+    // lane j of a row of lanes: r (0..3), k (4..7), w (8..11) of key k0 + 4 q + j % 4; keys past the end, and lanes 12..15, are zeros
+    const uint32_t step = (uint32_t)a.ld * 4, bytes = (uint32_t)a.M * step, part = (lane >> 2) & 3;
+    const __amdgpu_buffer_rsrc_t rs = make_rsrc(a.proj, (int)bytes);
+    uint32_t off[Q];
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int key = k0 + 4 * q + (lane & 3);
+        off[q] = key < d && part < 3 ? (uint32_t)((part == 2 ? 4 : part) * a.section + h * d + key) * 4 : bytes;
     }
+    const uint32_t voff = (uint32_t)(2 * a.section + h * d + c) * 4;
+    struct Tile { float p[TT][Q], v[TT]; } A, B;
+    const uint32_t last = bytes - step;
+    auto fetch = [&](Tile& x, int t0) {  // rows past the last repeat it and are not used
+        uint32_t row = min((uint32_t)t0 * step, last);
+#pragma unroll
+        for (int t = 0; t < TT; ++t) {
+#pragma unroll
+            for (int q = 0; q < Q; ++q) x.p[t][q] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(rs, off[q], row, 0));
+            x.v[t] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(rs, voff, row, 0));
+            row = min(row + step, last);
+        }
+        issue_order_fence();
+    };
+    float* out = a.o + kg * a.o_slab + (int64_t)h * d + c0;
+    auto run = [&](const Tile& x, int t0, int buf) {
+        auto token = [&](auto T) {
+            constexpr int t = decltype(T)::value;
+            float o = 0.0f;
+            static_for<Q>([&](auto I) {
+                constexpr int q = decltype(I)::value;
+                wkv_keys4(S[4 * q], S[4 * q + 1], S[4 * q + 2], S[4 * q + 3], o, x.p[t][q], x.v[t]);
+            });
+            s_o[buf][wave][t][lane] = o;
+        };
+        if (t0 + TT <= a.M) static_for<TT>(token);
+        else static_for<TT - 1>([&](auto T) { if (t0 + decltype(T)::value < a.M) token(T); });
+        __syncthreads();
+        store_tile<TT>(s_o[buf], out, a.o_ld, t0, a.M, d - c0);
+    };
+    fetch(A, 0);
+    for (int t0 = 0; t0 < a.M; t0 += 2 * TT) {
+        fetch(B, t0 + TT);
+        run(A, t0, 0);
+        if (t0 + TT >= a.M) break;
+        fetch(A, t0 + 2 * TT);
+        run(B, t0 + TT, 1);
+    }
+    if (c0 + lane < d) store_keys<KPL>(state, S);
+}
+
+// grid (rows, ceil(heads / 4)), a wave per head: o = the scan's sums + the bonus; over its root mean square, times norm and
+// silu(gate).  NV: values per lane.
+template <bool F32, int NV>
+__global__ __launch_bounds__(256) void wkv_out_rows_kernel(const WkvRows a) {
+    const int lane = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6), d = a.dim;
+    if (h >= a.heads) return;
+    const float *p = a.proj + blockIdx.x * a.ld + h * d, *o = a.o + blockIdx.x * a.o_ld + h * d;
+    float x[NV][4], v[NV], g[NV], n[NV], b[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int e = min(lane + 64 * i, d - 1);
+#pragma unroll
+        for (int z = 0; z < 4; ++z) x[i][z] = z < a.groups ? o[z * a.o_slab + e] : 0.0f;
+        v[i] = p[2 * a.section + e];
+        g[i] = p[3 * a.section + e];
+        n[i] = a.norm[h * d + e];
+        b[i] = p[e] * a.u[h * d + e] * p[a.section + e];
+    }
+    float bonus = 0.0f, ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) bonus += lane + 64 * i < d ? b[i] : 0.0f;
+    bonus = sum64(bonus);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        v[i] = lane + 64 * i < d ? fmaf(bonus, v[i], (x[i][0] + x[i][1]) + (x[i][2] + x[i][3])) : 0.0f;
+        ss = fmaf(v[i], v[i], ss);
+    }
+    const float r = 1.0f / sqrtf(sum64(ss) / (float)d + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+        if (lane + 64 * i < d) put_elem<F32>(a.out, blockIdx.x * a.out_ld + h * d + lane + 64 * i, v[i] * r * n[i] * silu_f(g[i]));
 }
 
 // grid (rows, ceil(wp / 1024)): the five inputs h + (h' - h) * mu, [5][rows][wp]
@@ -307,116 +362,162 @@ __global__ __launch_bounds__(64) void tanh_rows_kernel(const float* __restrict__
     }
 }
 
-// grid (rows, ceil(channels / 256)): convolution and silu of x, B and C, [rows][channels]
+// grid (ceil(rows / 8), ceil(channels / 256) + 1): convolution and silu of x, B and C, [rows][channels], eight rows per thread;
+// the last column of workgroups leaves decay and dt, [rows][2][heads]
+constexpr int CONV_ROWS = 8;
 __global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmRows a) {
     const SsmShape& m = a.m;
-    const int inner = m.heads * m.vdim, channels = inner + 2 * m.groups * m.state, ch = blockIdx.y * 256 + threadIdx.x;
-    if (ch >= channels) return;
-    const int row = blockIdx.x;
-    const float *x = a.proj + inner + ch, *w = m.conv + (int64_t)ch * m.taps;
-    float acc = m.conv_b[ch];
-    for (int j = 0; j < m.taps; ++j) {
-        const int64_t p = a.pos0 + row - j;
-        if (p < 0) break;
-        acc = fmaf(w[m.taps - 1 - j], row >= j ? x[(int64_t)(row - j) * a.ld] : a.ring[p % m.taps * channels + ch], acc);
+    const int inner = m.heads * m.vdim, channels = inner + 2 * m.groups * m.state, r0 = blockIdx.x * CONV_ROWS, rows = min(CONV_ROWS, a.M - r0);
+    if (blockIdx.y == gridDim.y - 1) {
+        for (int i = threadIdx.x; i < rows * m.heads; i += 256) {
+            const int64_t row = r0 + i / m.heads;
+            const int h = i % m.heads;
+            const float dt = softplus_f(a.proj[row * a.ld + inner + channels + h] + m.dt_bias[h]);
+            a.decay[row * 2 * m.heads + h] = expf(m.neg_a[h] * dt);
+            a.decay[(row * 2 + 1) * m.heads + h] = dt;
+        }
+        return;
     }
-    a.conv[(int64_t)row * channels + ch] = silu_f(acc);
+    const int ch = blockIdx.y * 256 + threadIdx.x;
+    if (ch >= channels) return;
+    const float *x = a.proj + inner + ch, *w = m.conv + (int64_t)ch * m.taps, bias = m.conv_b[ch];
+    auto input = [&](int row) {  // of row r0 + row, also of rows and positions before
+        const int64_t p = a.pos0 + r0 + row;
+        return r0 + row >= 0 ? x[(int64_t)min(r0 + row, a.M - 1) * a.ld] : p >= 0 ? a.ring[p % m.taps * channels + ch] : 0.0f;
+    };
+    float* out = a.conv + (int64_t)r0 * channels + ch;
+    if (m.taps <= 4) {
+        float in[CONV_ROWS + 3], t[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) t[j] = j < m.taps ? w[m.taps - 1 - j] : 0.0f;
+#pragma unroll
+        for (int i = 0; i < CONV_ROWS + 3; ++i) in[i] = 3 - i < m.taps ? input(i - 3) : 0.0f;
+#pragma unroll
+        for (int r = 0; r < CONV_ROWS; ++r)
+            if (r < rows) out[(int64_t)r * channels] = silu_f(fmaf(t[3], in[r], fmaf(t[2], in[r + 1], fmaf(t[1], in[r + 2], fmaf(t[0], in[r + 3], bias)))));
+    } else {
+        for (int r = 0; r < rows; ++r) {
+            float acc = bias;
+            for (int j = 0; j < m.taps; ++j) acc = fmaf(w[m.taps - 1 - j], input(r - j), acc);
+            out[(int64_t)r * channels] = silu_f(acc);
+        }
+    }
 }
 
-// grid (heads, ceil(vdim / 16)), 256 threads; y takes the place of x in a.conv
+// Four keys of 64 columns take a token: S <- decay S + B dx, y += C S.  p: a row of lanes with B at lanes B0 .. and C at C0 .. .
+template <int B0, int C0>
+__device__ __forceinline__ void ssm_keys4(float& s0, float& s1, float& s2, float& s3, float& y, float p, float decay, float dx) {
+    asm("v_mul_f32 %0, %6, %0\n\t"
+        "v_mul_f32 %1, %6, %1\n\t"
+        "v_mul_f32 %2, %6, %2\n\t"
+        "v_mul_f32 %3, %6, %3\n\t"
+        "v_fmac_f32_dpp %0, %5, %7 row_newbcast:%8 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %1, %5, %7 row_newbcast:%9 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %2, %5, %7 row_newbcast:%10 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %3, %5, %7 row_newbcast:%11 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %0 row_newbcast:%12 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %1 row_newbcast:%13 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %2 row_newbcast:%14 row_mask:0xf bank_mask:0xf\n\t"
+        "v_fmac_f32_dpp %4, %5, %3 row_newbcast:%15 row_mask:0xf bank_mask:0xf"
+        : "+&v"(s0), "+&v"(s1), "+&v"(s2), "+&v"(s3), "+&v"(y)
+        : "v"(p), "v"(decay), "v"(dx), "n"(B0), "n"(B0 + 1), "n"(B0 + 2), "n"(B0 + 3), "n"(C0), "n"(C0 + 1), "n"(C0 + 2), "n"(C0 + 3));
+}
+
+// grid (heads, key groups * ceil(vdim / 64)), 256 threads; without the skip D x, which the row kernel behind it adds
 template <int KPL>
-__global__ __launch_bounds__(256) void ssm_scan_kernel(const SsmRows a) {
-    constexpr int KP = 16 * KPL, TT = tile_tokens<KPL>(), NE = TT * KP / 256;
-    __shared__ __align__(16) float s_b[2][TT * KP], s_c[2][TT * KP];
-    __shared__ float s_x[2][TT * 16], s_a[2][TT], s_dt[2][TT];
+__global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmRows a) {
+    constexpr int KP = 16 * KPL, KQ = KPL < 8 ? KPL : 8, Q = KPL / KQ, TT = 16 / Q;  // Q rows of [B | C] of KQ keys per token
+    constexpr int NG = (TT + 7) / 8;
+    __shared__ float s_o[2][4][TT][64];
     const SsmShape& m = a.m;
-    const int tid = threadIdx.x, sub = tid & 15, grp = tid >> 4, h = blockIdx.x, N = m.state, per = m.heads / m.groups, g = h / per;
-    const int inner = m.heads * m.vdim, channels = inner + 2 * m.groups * N, c = blockIdx.y * 16 + grp;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), h = blockIdx.x, N = m.state;
+    const int per = m.heads / m.groups, g = h / per, inner = m.heads * m.vdim, channels = inner + 2 * m.groups * N;
+    const int kg = blockIdx.y % a.key_groups, c0 = blockIdx.y / a.key_groups * 64, c = min(c0 + lane, m.vdim - 1), k0 = (4 * kg + wave) * KPL;
     // the ring takes the inputs of the last positions
     for (int j = 0; j < m.taps && j < a.M; ++j) {
         const float* row = a.proj + (int64_t)(a.M - 1 - j) * a.ld + inner;
         float* slot = a.ring + (a.pos0 + a.M - 1 - j) % m.taps * channels;
-        if (tid < 16 && (int)blockIdx.y * 16 + tid < m.vdim) slot[h * m.vdim + blockIdx.y * 16 + tid] = row[h * m.vdim + blockIdx.y * 16 + tid];
+        if (kg == 0 && wave == 0 && c0 + lane < m.vdim) slot[h * m.vdim + c] = row[h * m.vdim + c];
         if (h % per == 0 && blockIdx.y == 0)
             for (int i = tid; i < 2 * N; i += 256) {
                 const int ch = inner + (i < N ? 0 : m.groups * N) + g * N + i % N;
                 slot[ch] = row[ch];
             }
     }
-    float* state = a.state + ((int64_t)h * m.vdim + min(c, m.vdim - 1)) * KP + sub * KPL;
+    float* state = a.state + ((int64_t)h * m.vdim + c) * KP + k0;
     float S[KPL];
     if (a.pos0 > 0) load_keys<KPL>(S, state);
     else
 #pragma unroll
         for (int i = 0; i < KPL; ++i) S[i] = 0.0f;
-    const float *Bp = a.conv + inner + g * N, *Cp = Bp + m.groups * N, dtb = m.dt_bias[h], na = m.neg_a[h], D = m.D[h];
-    float rb[NE], rc[NE], rx = 0.0f, rdt = 0.0f;
-    auto fetch = [&](int t0) {
+    // lane j of a row of lanes: B (j < KQ) or C (KQ <= j < 2 KQ) of key k0 + KQ q + j % KQ; the other lanes, and keys past the end,
+    // are zeros
+    const uint32_t step = (uint32_t)channels * 4, bytes = (uint32_t)a.M * step;
+    const __amdgpu_buffer_rsrc_t rs = make_rsrc(a.conv, (int)bytes);
+    uint32_t off[Q];
 #pragma unroll
-        for (int i = 0; i < NE; ++i) {
-            const int e = tid + 256 * i, t = t0 + e / KP, k = e % KP;
-            const bool in = t < a.M && k < N;
-            const int64_t at = (int64_t)min(t, a.M - 1) * channels + min(k, N - 1);
-            const float b0 = Bp[at], c0 = Cp[at];
-            rb[i] = in ? b0 : 0.0f;
-            rc[i] = in ? c0 : 0.0f;
-        }
-        if (tid < TT * 16) {
-            const int t = t0 + tid / 16, cc = blockIdx.y * 16 + tid % 16;
-            rx = t < a.M && cc < m.vdim ? a.conv[(int64_t)t * channels + h * m.vdim + cc] : 0.0f;
-        }
-        if (tid < TT) rdt = t0 + tid < a.M ? a.proj[(int64_t)(t0 + tid) * a.ld + inner + channels + h] + dtb : -INFINITY;
-    };
-    auto stage = [&](int buf) {
-#pragma unroll
-        for (int i = 0; i < NE; ++i) {
-            s_b[buf][tid + 256 * i] = rb[i];
-            s_c[buf][tid + 256 * i] = rc[i];
-        }
-        if (tid < TT * 16) s_x[buf][tid] = rx;
-        if (tid < TT) {  // past the end: dt 0, decay 1
-            const float dt = softplus_f(rdt);
-            s_dt[buf][tid] = dt;
-            s_a[buf][tid] = expf(na * dt);
-        }
-    };
-    const int tiles = (a.M + TT - 1) / TT;
-    fetch(0);
-    stage(0);
-    __syncthreads();
-    for (int tile = 0; tile < tiles; ++tile) {
-        const int buf = tile & 1;
-        if (tile + 1 < tiles) fetch((tile + 1) * TT);
-        float keep = 0.0f;
-#pragma unroll 4
-        for (int t = 0; t < TT; ++t) {
-            float B[KPL], C[KPL], y = 0.0f;
-            load_keys<KPL>(B, &s_b[buf][t * KP + sub * KPL]);
-            load_keys<KPL>(C, &s_c[buf][t * KP + sub * KPL]);
-            const float x = s_x[buf][t * 16 + grp], decay = s_a[buf][t], dx = s_dt[buf][t] * x;
-#pragma unroll
-            for (int i = 0; i < KPL; ++i) {
-                S[i] = fmaf(decay, S[i], B[i] * dx);
-                y = fmaf(S[i], C[i], y);
-            }
-            y = fmaf(D, x, sum16(y));
-            keep = sub == t ? y : keep;
-        }
-        const int t = tile * TT + sub;
-        if (sub < TT && t < a.M && c < m.vdim) a.conv[(int64_t)t * channels + h * m.vdim + c] = keep;
-        if (tile + 1 < tiles) stage(buf ^ 1);
-        __syncthreads();
+    for (int q = 0; q < Q; ++q) {
+        const int j = lane & 15, key = k0 + KQ * q + j % KQ;
+        off[q] = key < N && j < 2 * KQ ? (uint32_t)(inner + (j < KQ ? 0 : m.groups * N) + g * N + key) * 4 : bytes;
     }
-    if (c < m.vdim) store_keys<KPL>(state, S);
+    const uint32_t xoff = (uint32_t)(h * m.vdim + c) * 4;
+    const float* dsrc = a.decay + (lane & 8 ? m.heads : 0) + h;
+    struct Tile { float p[TT][Q], x[TT], d[NG]; } A, B;
+    const uint32_t last = bytes - step;
+    auto fetch = [&](Tile& x, int t0) {  // rows past the last repeat it and are not used
+        uint32_t row = min((uint32_t)t0 * step, last);
+#pragma unroll
+        for (int i = 0; i < NG; ++i) x.d[i] = dsrc[(int64_t)min(t0 + 8 * i + (lane & 7), a.M - 1) * 2 * m.heads];  // decay, then dt, of eight tokens
+#pragma unroll
+        for (int t = 0; t < TT; ++t) {
+#pragma unroll
+            for (int q = 0; q < Q; ++q) x.p[t][q] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(rs, off[q], row, 0));
+            x.x[t] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(rs, xoff, row, 0));
+            row = min(row + step, last);
+        }
+        issue_order_fence();
+    };
+    float* out = a.y + kg * a.y_slab + h * m.vdim + c0;
+    auto run = [&](const Tile& x, int t0, int buf) {
+        auto token = [&](auto T) {
+            constexpr int t = decltype(T)::value;
+            const float decay = row_lane<t % 8>(x.d[t / 8]), dx = row_lane<8 + t % 8>(x.d[t / 8]) * x.x[t];
+            float y = 0.0f;
+            static_for<KPL / 4>([&](auto I) {
+                constexpr int i = 4 * decltype(I)::value, b0 = i % KQ;
+                ssm_keys4<b0, KQ + b0>(S[i], S[i + 1], S[i + 2], S[i + 3], y, x.p[t][i / KQ], decay, dx);
+            });
+            s_o[buf][wave][t][lane] = y;
+        };
+        if (t0 + TT <= a.M) static_for<TT>(token);
+        else static_for<TT - 1>([&](auto T) { if (t0 + decltype(T)::value < a.M) token(T); });
+        __syncthreads();
+        store_tile<TT>(s_o[buf], out, inner, t0, a.M, m.vdim - c0);
+    };
+    fetch(A, 0);
+    for (int t0 = 0; t0 < a.M; t0 += 2 * TT) {
+        fetch(B, t0 + TT);
+        run(A, t0, 0);
+        if (t0 + TT >= a.M) break;
+        fetch(A, t0 + 2 * TT);
+        run(B, t0 + TT, 1);
+    }
+    if (c0 + lane < m.vdim) store_keys<KPL>(state, S);
 }
 
-// grid rows: y * silu(z), normed in equal parts, times norm and the branch's scale
+// grid rows: (the scan's sums + D x) * silu(z), normed in equal parts, times norm and the branch's scale
 template <bool F32>
 __global__ __launch_bounds__(256) void ssm_out_rows_kernel(const SsmRows a) {
     __shared__ float red[4];
     const SsmShape& m = a.m;
     const int tid = threadIdx.x, inner = m.heads * m.vdim, channels = inner + 2 * m.groups * m.state, part = inner / m.norm_groups;
-    const float *y = a.conv + (int64_t)blockIdx.x * channels, *z = a.proj + blockIdx.x * a.ld;
+    const float *y = a.y + (int64_t)blockIdx.x * inner, *x = a.conv + (int64_t)blockIdx.x * channels, *z = a.proj + blockIdx.x * a.ld;
+    auto value = [&](int c) {
+        float s[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) s[k] = k < a.key_groups ? y[k * a.y_slab + c] : 0.0f;
+        return fmaf(m.D[c / m.vdim], x[c], (s[0] + s[1]) + (s[2] + s[3])) * silu_f(z[c]);
+    };
     constexpr int NS = 16;  // values kept in registers: parts of up to 4096
     for (int p = 0; p < m.norm_groups; ++p) {
         const int c0 = p * part;
@@ -424,11 +525,11 @@ __global__ __launch_bounds__(256) void ssm_out_rows_kernel(const SsmRows a) {
 #pragma unroll
         for (int i = 0; i < NS; ++i) {
             const int c = tid + 256 * i;
-            v[i] = c < part ? y[c0 + c] * silu_f(z[c0 + c]) : 0.0f;
+            v[i] = c < part ? value(c0 + c) : 0.0f;
             ss = fmaf(v[i], v[i], ss);
         }
         for (int c = tid + 256 * NS; c < part; c += 256) {
-            const float t = y[c0 + c] * silu_f(z[c0 + c]);
+            const float t = value(c0 + c);
             ss = fmaf(t, t, ss);
         }
         const float r = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)part + a.eps) * m.scale;
@@ -437,8 +538,7 @@ __global__ __launch_bounds__(256) void ssm_out_rows_kernel(const SsmRows a) {
             const int c = tid + 256 * i;
             if (c < part) put_elem<F32>(a.out, blockIdx.x * a.out_ld + c0 + c, v[i] * r * m.norm[c0 + c]);
         }
-        for (int c = tid + 256 * NS; c < part; c += 256)
-            put_elem<F32>(a.out, blockIdx.x * a.out_ld + c0 + c, y[c0 + c] * silu_f(z[c0 + c]) * r * m.norm[c0 + c]);
+        for (int c = tid + 256 * NS; c < part; c += 256) put_elem<F32>(a.out, blockIdx.x * a.out_ld + c0 + c, value(c0 + c) * r * m.norm[c0 + c]);
     }
 }
 
@@ -482,21 +582,33 @@ int tanh_rows(const float* g, int slabs, int64_t slab, int rows, int n, bool fp3
     return launch_status();
 }
 
-int wkv_rows(const WkvRows& a, bool fp32, hipStream_t s) {
-    const dim3 grid(a.heads, (a.dim + 15) / 16);
+int64_t scan_slabs(int keys) { return key_groups(keys); }
+
+int wkv_rows(WkvRows a, bool fp32, hipStream_t s) {
+    if (!recurrent_supported(a.dim)) return PTM_E_UNSUPPORTED;
+    a.groups = key_groups(a.dim);
+    const dim3 grid(a.heads, a.groups * ((a.dim + 63) / 64));
 #define PTM_RUN(KPL) hipLaunchKernelGGL(wkv_scan_kernel<KPL>, grid, dim3(256), 0, s, a)
     PTM_KPL(a.dim, PTM_RUN)
 #undef PTM_RUN
-    if (fp32) hipLaunchKernelGGL(wkv_out_rows_kernel<true>, dim3(a.M), dim3(256), 0, s, a);
-    else hipLaunchKernelGGL(wkv_out_rows_kernel<false>, dim3(a.M), dim3(256), 0, s, a);
+    const dim3 out_grid(a.M, (a.heads + 3) / 4);
+#define PTM_RUN(NV)                                                                                                  \
+    if (fp32) hipLaunchKernelGGL((wkv_out_rows_kernel<true, NV>), out_grid, dim3(256), 0, s, a);                     \
+    else hipLaunchKernelGGL((wkv_out_rows_kernel<false, NV>), out_grid, dim3(256), 0, s, a)
+    if (a.dim <= 64) { PTM_RUN(1); }
+    else if (a.dim <= 128) { PTM_RUN(2); }
+    else { PTM_RUN(8); }
+#undef PTM_RUN
     return launch_status();
 }
 
-int ssm_rows(const SsmRows& a, bool fp32, hipStream_t s) {
+int ssm_rows(SsmRows a, bool fp32, hipStream_t s) {
     const SsmShape& m = a.m;
+    if (!recurrent_supported(m.state)) return PTM_E_UNSUPPORTED;
     const int channels = m.heads * m.vdim + 2 * m.groups * m.state;
-    hipLaunchKernelGGL(ssm_conv_rows_kernel, dim3(a.M, (channels + 255) / 256), dim3(256), 0, s, a);
-    const dim3 grid(m.heads, (m.vdim + 15) / 16);
+    a.key_groups = key_groups(m.state);
+    hipLaunchKernelGGL(ssm_conv_rows_kernel, dim3((a.M + CONV_ROWS - 1) / CONV_ROWS, (channels + 255) / 256 + 1), dim3(256), 0, s, a);
+    const dim3 grid(m.heads, a.key_groups * ((m.vdim + 63) / 64));
 #define PTM_RUN(KPL) hipLaunchKernelGGL(ssm_scan_kernel<KPL>, grid, dim3(256), 0, s, a)
     PTM_KPL(m.state, PTM_RUN)
 #undef PTM_RUN
