@@ -198,42 +198,54 @@ static int key_groups(int keys) { return (keys + 4 * keys_per_lane(keys) - 1) / 
 template <int N>
 __device__ __forceinline__ float row_lane(float v) { return dpp_f<0x150 + N>(v); }
 
-// Adds the waves' sums of a tile of TT tokens (s_o [4][TT][64]) and stores them: row t0 + t, 64 columns from `out`.
+// The waves' sums of a tile of TT tokens (s_o [4][TT][64]), on their way from LDS while the next tile is used: this wave's rows
+// wave, wave + 4, ...
 template <int TT>
-__device__ __forceinline__ void store_tile(const float (*s_o)[TT][64], float* out, int64_t ld, int t0, int M, int columns) {
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+struct TileSums {
+    float v[TT / 4][4];
+    __device__ __forceinline__ void read(const float (*s_o)[TT][64]) {
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
-    for (int q = 0; q < (TT + 3) / 4; ++q) {
-        const int t = wave + 4 * q;
-        if (t < TT && t0 + t < M && lane < columns)
-            out[(int64_t)(t0 + t) * ld + lane] = (s_o[0][t][lane] + s_o[1][t][lane]) + (s_o[2][t][lane] + s_o[3][t][lane]);
+        for (int q = 0; q < TT / 4; ++q)
+#pragma unroll
+            for (int w = 0; w < 4; ++w) v[q][w] = s_o[w][wave + 4 * q][lane];
     }
-}
+    __device__ __forceinline__ void store(float* out, int64_t ld, int t0, int M, int columns) const {
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+#pragma unroll
+        for (int q = 0; q < TT / 4; ++q) {
+            const int t = t0 + wave + 4 * q;
+            if (t < M && lane < columns) out[(int64_t)t * ld + lane] = (v[q][0] + v[q][1]) + (v[q][2] + v[q][3]);
+        }
+    }
+};
 
-// Four keys of 64 columns take a token: o += S^T r, S <- diag(w) S + k v^T.  p: a row of lanes [r | k | w | -], four each.
+// Four keys of 64 columns take four tokens: o += S^T r, S <- diag(w) S + k v^T.  p[t]: a row of lanes [r | k | w | -], four each.
 // (One block, because the compiler does not fold the broadcasts into the multiply-adds; the wait states are for p.)
-__device__ __forceinline__ void wkv_keys4(float& s0, float& s1, float& s2, float& s3, float& o, float p, float v) {
-    asm("s_nop 1\n\t"
-        "v_fmac_f32_dpp %4, %5, %0 row_newbcast:0 row_mask:0xf bank_mask:0xf\n\t"
-        "v_mul_f32_dpp %0, %5, %0 row_newbcast:8 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %1 row_newbcast:1 row_mask:0xf bank_mask:0xf\n\t"
-        "v_mul_f32_dpp %1, %5, %1 row_newbcast:9 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %2 row_newbcast:2 row_mask:0xf bank_mask:0xf\n\t"
-        "v_mul_f32_dpp %2, %5, %2 row_newbcast:10 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %3 row_newbcast:3 row_mask:0xf bank_mask:0xf\n\t"
-        "v_mul_f32_dpp %3, %5, %3 row_newbcast:11 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %0, %5, %6 row_newbcast:4 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %1, %5, %6 row_newbcast:5 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %2, %5, %6 row_newbcast:6 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %3, %5, %6 row_newbcast:7 row_mask:0xf bank_mask:0xf"
-        : "+&v"(s0), "+&v"(s1), "+&v"(s2), "+&v"(s3), "+&v"(o)
-        : "v"(p), "v"(v));
+#define PTM_DPP(n) " row_newbcast:" n " row_mask:0xf bank_mask:0xf\n\t"
+#define PTM_WKV_TOKEN(O, P, V)                                   \
+    "v_fmac_f32_dpp %" O ", %" P ", %0" PTM_DPP("0")             \
+    "v_mul_f32_dpp %0, %" P ", %0" PTM_DPP("8")                  \
+    "v_fmac_f32_dpp %" O ", %" P ", %1" PTM_DPP("1")             \
+    "v_mul_f32_dpp %1, %" P ", %1" PTM_DPP("9")                  \
+    "v_fmac_f32_dpp %" O ", %" P ", %2" PTM_DPP("2")             \
+    "v_mul_f32_dpp %2, %" P ", %2" PTM_DPP("10")                 \
+    "v_fmac_f32_dpp %" O ", %" P ", %3" PTM_DPP("3")             \
+    "v_mul_f32_dpp %3, %" P ", %3" PTM_DPP("11")                 \
+    "v_fmac_f32_dpp %0, %" P ", %" V PTM_DPP("4")                \
+    "v_fmac_f32_dpp %1, %" P ", %" V PTM_DPP("5")                \
+    "v_fmac_f32_dpp %2, %" P ", %" V PTM_DPP("6")                \
+    "v_fmac_f32_dpp %3, %" P ", %" V PTM_DPP("7")
+__device__ __forceinline__ void wkv_keys4(float* s, float (&o)[4], float p0, float p1, float p2, float p3, float v0, float v1, float v2, float v3) {
+    asm("s_nop 1\n\t" PTM_WKV_TOKEN("4", "8", "12") PTM_WKV_TOKEN("5", "9", "13") PTM_WKV_TOKEN("6", "10", "14") PTM_WKV_TOKEN("7", "11", "15")
+        : "+&v"(s[0]), "+&v"(s[1]), "+&v"(s[2]), "+&v"(s[3]), "+&v"(o[0]), "+&v"(o[1]), "+&v"(o[2]), "+&v"(o[3])
+        : "v"(p0), "v"(p1), "v"(p2), "v"(p3), "v"(v0), "v"(v1), "v"(v2), "v"(v3));
 }
 
 // grid (heads, key groups * ceil(dim / 64)), 256 threads.  Without the bonus, which the row kernel behind it adds.
 template <int KPL>
 __global__ __launch_bounds__(256, 1) void wkv_scan_kernel(const WkvRows a) {
-    constexpr int KP = 16 * KPL, Q = KPL / 4, TT = 16 / Q;  // Q rows of [r | k | w] of four keys per token
+    constexpr int KP = 16 * KPL, Q = KPL / 4, TT = Q < 4 ? 16 / Q : 4;  // Q rows of [r | k | w] of four keys per token
     __shared__ float s_o[2][4][TT][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), h = blockIdx.x, d = a.dim;
     const int kg = blockIdx.y % a.groups, c0 = blockIdx.y / a.groups * 64, c = min(c0 + lane, d - 1), k0 = (4 * kg + wave) * KPL;
@@ -269,29 +281,41 @@ __global__ __launch_bounds__(256, 1) void wkv_scan_kernel(const WkvRows a) {
         issue_order_fence();
     };
     float* out = a.o + kg * a.o_slab + (int64_t)h * d + c0;
-    auto run = [&](const Tile& x, int t0, int buf) {
-        auto token = [&](auto T) {
-            constexpr int t = decltype(T)::value;
-            float o = 0.0f;
-            static_for<Q>([&](auto I) {
-                constexpr int q = decltype(I)::value;
-                wkv_keys4(S[4 * q], S[4 * q + 1], S[4 * q + 2], S[4 * q + 3], o, x.p[t][q], x.v[t]);
-            });
-            s_o[buf][wave][t][lane] = o;
-        };
-        if (t0 + TT <= a.M) static_for<TT>(token);
-        else static_for<TT - 1>([&](auto T) { if (t0 + decltype(T)::value < a.M) token(T); });
+    TileSums<TT> sums;
+    auto run = [&](Tile& x, int t0, int buf) {  // a token past the last leaves the state as it is
+        if (t0 > 0) sums.read(s_o[buf ^ 1]);
+        if (t0 + TT > a.M) {
+            const float keep = part == 2 ? 1.0f : 0.0f;
+#pragma unroll
+            for (int t = 0; t < TT; ++t)
+                if (t0 + t >= a.M)
+#pragma unroll
+                    for (int q = 0; q < Q; ++q) x.p[t][q] = keep;
+        }
+#pragma unroll
+        for (int t = 0; t < TT; t += 4) {
+            float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int q = 0; q < Q; ++q)
+                wkv_keys4(S + 4 * q, o, x.p[t][q], x.p[t + 1][q], x.p[t + 2][q], x.p[t + 3][q], x.v[t], x.v[t + 1], x.v[t + 2], x.v[t + 3]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s_o[buf][wave][t + i][lane] = o[i];
+        }
+        if (t0 > 0) sums.store(out, a.o_ld, t0 - TT, a.M, d - c0);
         __syncthreads();
-        store_tile<TT>(s_o[buf], out, a.o_ld, t0, a.M, d - c0);
     };
     fetch(A, 0);
-    for (int t0 = 0; t0 < a.M; t0 += 2 * TT) {
+    int t0 = 0;
+    for (;; t0 += 2 * TT) {
         fetch(B, t0 + TT);
         run(A, t0, 0);
         if (t0 + TT >= a.M) break;
         fetch(A, t0 + 2 * TT);
         run(B, t0 + TT, 1);
+        if (t0 + 2 * TT >= a.M) { t0 += TT; break; }
     }
+    sums.read(s_o[t0 / TT & 1]);
+    sums.store(out, a.o_ld, t0, a.M, d - c0);
     if (c0 + lane < d) store_keys<KPL>(state, S);
 }
 
@@ -404,23 +428,31 @@ __global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmRows a) {
     }
 }
 
-// Four keys of 64 columns take a token: S <- decay S + B dx, y += C S.  p: a row of lanes with B at lanes B0 .. and C at C0 .. .
+// Four keys of 64 columns take four tokens: S <- decay S + B dx, y += C S.  p[t]: a row of lanes with B at lanes B0 .. and C at
+// C0 .. .
+#define PTM_DECAY(S, D) "v_mul_f32 %" S ", %" D ", %" S "\n\t"
+#define PTM_SSM_TAKE(P, X)                                       \
+    "v_fmac_f32_dpp %0, %" P ", %" X PTM_DPP("%20")              \
+    "v_fmac_f32_dpp %1, %" P ", %" X PTM_DPP("%21")              \
+    "v_fmac_f32_dpp %2, %" P ", %" X PTM_DPP("%22")              \
+    "v_fmac_f32_dpp %3, %" P ", %" X PTM_DPP("%23")
+#define PTM_SSM_GIVE(Y, P, S, C) "v_fmac_f32_dpp %" Y ", %" P ", %" S PTM_DPP("%" C)
+#define PTM_SSM_GIVE_NEXT(Y, P, D)                               \
+    PTM_SSM_GIVE(Y, P, "0", "24") PTM_DECAY("0", D)              \
+    PTM_SSM_GIVE(Y, P, "1", "25") PTM_DECAY("1", D)              \
+    PTM_SSM_GIVE(Y, P, "2", "26") PTM_DECAY("2", D)              \
+    PTM_SSM_GIVE(Y, P, "3", "27") PTM_DECAY("3", D)
 template <int B0, int C0>
-__device__ __forceinline__ void ssm_keys4(float& s0, float& s1, float& s2, float& s3, float& y, float p, float decay, float dx) {
-    asm("v_mul_f32 %0, %6, %0\n\t"
-        "v_mul_f32 %1, %6, %1\n\t"
-        "v_mul_f32 %2, %6, %2\n\t"
-        "v_mul_f32 %3, %6, %3\n\t"
-        "v_fmac_f32_dpp %0, %5, %7 row_newbcast:%8 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %1, %5, %7 row_newbcast:%9 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %2, %5, %7 row_newbcast:%10 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %3, %5, %7 row_newbcast:%11 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %0 row_newbcast:%12 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %1 row_newbcast:%13 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %2 row_newbcast:%14 row_mask:0xf bank_mask:0xf\n\t"
-        "v_fmac_f32_dpp %4, %5, %3 row_newbcast:%15 row_mask:0xf bank_mask:0xf"
-        : "+&v"(s0), "+&v"(s1), "+&v"(s2), "+&v"(s3), "+&v"(y)
-        : "v"(p), "v"(decay), "v"(dx), "n"(B0), "n"(B0 + 1), "n"(B0 + 2), "n"(B0 + 3), "n"(C0), "n"(C0 + 1), "n"(C0 + 2), "n"(C0 + 3));
+__device__ __forceinline__ void ssm_keys4(float* s, float (&y)[4], float p0, float p1, float p2, float p3, const float* decay, const float* dx) {
+    asm(PTM_DECAY("0", "12") PTM_DECAY("1", "12") PTM_DECAY("2", "12") PTM_DECAY("3", "12")
+        PTM_SSM_TAKE("8", "16") PTM_SSM_GIVE_NEXT("4", "8", "13")
+        PTM_SSM_TAKE("9", "17") PTM_SSM_GIVE_NEXT("5", "9", "14")
+        PTM_SSM_TAKE("10", "18") PTM_SSM_GIVE_NEXT("6", "10", "15")
+        PTM_SSM_TAKE("11", "19")
+        PTM_SSM_GIVE("7", "11", "0", "24") PTM_SSM_GIVE("7", "11", "1", "25") PTM_SSM_GIVE("7", "11", "2", "26") PTM_SSM_GIVE("7", "11", "3", "27")
+        : "+&v"(s[0]), "+&v"(s[1]), "+&v"(s[2]), "+&v"(s[3]), "+&v"(y[0]), "+&v"(y[1]), "+&v"(y[2]), "+&v"(y[3])
+        : "v"(p0), "v"(p1), "v"(p2), "v"(p3), "v"(decay[0]), "v"(decay[1]), "v"(decay[2]), "v"(decay[3]), "v"(dx[0]), "v"(dx[1]), "v"(dx[2]), "v"(dx[3]),
+          "n"(B0), "n"(B0 + 1), "n"(B0 + 2), "n"(B0 + 3), "n"(C0), "n"(C0 + 1), "n"(C0 + 2), "n"(C0 + 3));
 }
 
 // grid (heads, key groups * ceil(vdim / 64)), 256 threads; without the skip D x, which the row kernel behind it adds
@@ -478,30 +510,48 @@ __global__ __launch_bounds__(256, 1) void ssm_scan_kernel(const SsmRows a) {
         issue_order_fence();
     };
     float* out = a.y + kg * a.y_slab + h * m.vdim + c0;
-    auto run = [&](const Tile& x, int t0, int buf) {
-        auto token = [&](auto T) {
+    TileSums<TT> sums;
+    auto run = [&](Tile& x, int t0, int buf) {  // a token past the last leaves the state as it is
+        if (t0 > 0) sums.read(s_o[buf ^ 1]);
+        float decay[TT], dx[TT];
+        static_for<TT>([&](auto T) {
             constexpr int t = decltype(T)::value;
-            const float decay = row_lane<t % 8>(x.d[t / 8]), dx = row_lane<8 + t % 8>(x.d[t / 8]) * x.x[t];
-            float y = 0.0f;
+            decay[t] = row_lane<t % 8>(x.d[t / 8]);
+            dx[t] = row_lane<8 + t % 8>(x.d[t / 8]) * x.x[t];
+        });
+        if (t0 + TT > a.M) {
+#pragma unroll
+            for (int t = 0; t < TT; ++t)
+                if (t0 + t >= a.M) {
+                    decay[t] = 1.0f;
+                    dx[t] = 0.0f;
+                }
+        }
+#pragma unroll
+        for (int t = 0; t < TT; t += 4) {
+            float y[4] = {0.0f, 0.0f, 0.0f, 0.0f};
             static_for<KPL / 4>([&](auto I) {
-                constexpr int i = 4 * decltype(I)::value, b0 = i % KQ;
-                ssm_keys4<b0, KQ + b0>(S[i], S[i + 1], S[i + 2], S[i + 3], y, x.p[t][i / KQ], decay, dx);
+                constexpr int i = 4 * decltype(I)::value, b0 = i % KQ, q = i / KQ;
+                ssm_keys4<b0, KQ + b0>(S + i, y, x.p[t][q], x.p[t + 1][q], x.p[t + 2][q], x.p[t + 3][q], decay + t, dx + t);
             });
-            s_o[buf][wave][t][lane] = y;
-        };
-        if (t0 + TT <= a.M) static_for<TT>(token);
-        else static_for<TT - 1>([&](auto T) { if (t0 + decltype(T)::value < a.M) token(T); });
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s_o[buf][wave][t + i][lane] = y[i];
+        }
+        if (t0 > 0) sums.store(out, inner, t0 - TT, a.M, m.vdim - c0);
         __syncthreads();
-        store_tile<TT>(s_o[buf], out, inner, t0, a.M, m.vdim - c0);
     };
     fetch(A, 0);
-    for (int t0 = 0; t0 < a.M; t0 += 2 * TT) {
+    int t0 = 0;
+    for (;; t0 += 2 * TT) {
         fetch(B, t0 + TT);
         run(A, t0, 0);
         if (t0 + TT >= a.M) break;
         fetch(A, t0 + 2 * TT);
         run(B, t0 + TT, 1);
+        if (t0 + 2 * TT >= a.M) { t0 += TT; break; }
     }
+    sums.read(s_o[t0 / TT & 1]);
+    sums.store(out, inner, t0, a.M, m.vdim - c0);
     if (c0 + lane < m.vdim) store_keys<KPL>(state, S);
 }
 
