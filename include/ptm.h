@@ -503,12 +503,17 @@ void* ptm_decode_stream(ptm_decoder* d);
  *   x += RMSNorm(mixer(RMSNorm(x, norm1)), norm1b);   x += RMSNorm(W_down relu(W_up RMSNorm(x, norm2))^2, norm2b)
  *   and with a per-layer token input: g = gelu_tanh(W_gate x) * e, e = the block's part of the token's row of a second
  *   embedding table; x += RMSNorm(W_proj g, side_norm)
+ *   (streams > 0 in the configuration: hyper-connections around every branch instead, without post-norms; see there)
  * Mixers:
- *   PTM_MIX_ATTENTION  GQA; q and k RMS-normed over the whole projection, rotated, scores scale * q.k, optionally
+ *   PTM_MIX_ATTENTION  GQA; q and k RMS-normed over the whole projection (or per head), rotated, scores scale * q.k, optionally
  *                      softcap * tanh(score / softcap), sliding window with kept first positions (both mixers take these)
  *   PTM_MIX_LATENT     q per head [dim | rot_dim]; one latent c (RMS-normed) and one rotated key part per position are
  *                      cached; per head k = [W_uk c | rotated part], v = W_uv c.  A decode step never expands the cache:
  *                      W_uk moves onto the query and W_uv onto the attended latent.
+ *   PTM_MIX_WKV        time mixing with a decayed matrix state per head (ptm_wkv); an attention block may have a state-space mixer
+ *                      beside it (ptm_ssm).  Their state belongs to the sequence: it starts over at position 0 and has no
+ *                      way back, so ptm_decode_set_past_len takes 0 or the current position of such a decoder (else
+ *                      PTM_E_STATE)
  * Weights are bfloat16 matrices (ggml_type PTM_TYPE_BF16), rows zero-padded to multiples of 64 values
  * (ptm_dense_cols); vectors are fp32, zero-padded alike; `vec64` below marks such a vector. */
 #define PTM_TYPE_BF16 30u
@@ -716,7 +721,8 @@ int ptm_safetensors_tensor_at(const ptm_safetensors* f, int64_t i, ptm_st_tensor
 int ptm_safetensors_find(const ptm_safetensors* f, const char* name, ptm_st_tensor* out);
 
 /* Any model: a .gguf file (ptm_model_load_gguf; precision chooses the fp16 or fp32 cache) or a folder, whose config.json
- * names the architecture: "Tovasun" (a list of attention / latent_attention layers, optionally with a loop and a per-layer
+ * names the architecture: "Nadozen" (wkv layers and attention beside state-space mixers, hyper-connections, shared weights) or
+ * "Tovasun" (a list of attention / latent_attention layers, optionally with a loop and a per-layer
  * token input). */
 int ptm_model_load(const char* path, int max_seq, int precision, int use_graph, ptm_model** out);
 

@@ -535,7 +535,7 @@ static int ssm_check(const ptm_ssm& m) {
     if (m.vdim <= 0 || m.state <= 0 || m.groups <= 0 || m.heads % m.groups || m.taps <= 0 || m.norm_groups <= 0 || m.heads > 36864 || m.vdim > 36864 ||
         (int64_t)m.heads * m.vdim > 36864 || (int64_t)m.heads * m.vdim % m.norm_groups)
         return PTM_E_SHAPE;
-    if (!recurrent_supported(m.state) || m.norm_groups > 512 || m.taps > 4096) return PTM_E_UNSUPPORTED;
+    if (!recurrent_supported(m.state) || m.norm_groups > 512 || m.taps > 4096 || (int64_t)m.groups * m.state > 36864) return PTM_E_UNSUPPORTED;
     return m.conv && m.conv_b && m.dt_bias && m.neg_a && m.D && m.norm ? PTM_OK : PTM_E_NULL;
 }
 
@@ -1136,9 +1136,10 @@ int blocks_reserve(BlockStack* b, int rows) {
         grow(act, (size_t)up64(L.ff));
         if (latent(L)) grow(kv, expand_positions(b, L, rows) * (size_t)expand_rows(L));
     }
+    const size_t wide = W > low ? W : low;  // r_h also takes the decay's low-rank products
     size_t off = 0;
     auto take = [&](size_t bytes) { const size_t o = off; off += (bytes + 511) & ~(size_t)255; return o; };
-    const size_t o_tok = take(4 * R), o_x = take(4 * S * R * W), o_e = take(4 * R * W), o_h = take(4 * (R * W + (size_t)SPLIT_ROOM)), o_p = take(4 * R * proj),
+    const size_t o_tok = take(4 * R), o_x = take(4 * S * R * W), o_e = take(4 * R * W), o_h = take(4 * (R * wide + (size_t)SPLIT_ROOM)), o_p = take(4 * R * proj),
                  o_xn = take(es * R * W), o_q = take(es * R * q), o_at = take(es * R * attn), o_ac = take(es * R * act),
                  o_g = take(es * R * (size_t)up64(c.side_dim > 0 ? c.side_dim : 1)), o_kv = take(es * kv),
                  o_hn = take(4 * shifted), o_mix = take(es * 5 * shifted), o_low = take(es * R * low), o_cv = take(4 * R * conv), o_sc = take(4 * R * scan),
@@ -1153,7 +1154,7 @@ int blocks_reserve(BlockStack* b, int rows) {
     b->r_emb = (float*)(p + o_e);
     b->r_h = (float*)(p + o_h);
     b->r_proj = (float*)(p + o_p);
-    b->r_h_room = (int64_t)(R * W) + SPLIT_ROOM;
+    b->r_h_room = (int64_t)(R * wide) + SPLIT_ROOM;
     b->r_xn = p + o_xn;
     b->r_q = p + o_q;
     b->r_attn = p + o_at;
